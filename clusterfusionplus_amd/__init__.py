@@ -18,9 +18,11 @@ import sys as _sys
 
 _here = _os.path.dirname(_os.path.abspath(__file__))
 _missing = [n for n in ("libcfpp.so", "_clusterfusion.so") if not _os.path.exists(_os.path.join(_here, n))]
-# `python -m clusterfusionplus_amd.build` has to get past this file on a fresh checkout: for that one command
-# the package imports without its operators; every other import without the libraries fails here.
-_building = "clusterfusionplus_amd.build" in getattr(_sys, "orig_argv", [])
+# These commands build the libraries they need themselves and have to get past this file on a fresh checkout: for them the
+# package imports without its operators; every other import without the libraries fails here.
+_argv = getattr(_sys, "orig_argv", [])
+_building = any(a == "-m" and m in ("clusterfusionplus_amd", "clusterfusionplus_amd.build", "clusterfusionplus_amd.trace")
+                for a, m in zip(_argv, _argv[1:]))
 
 if _missing and not _building:
     raise ImportError(
@@ -40,3 +42,8 @@ if not _missing:
 
     __all__ += ["NeoxConfig", "PYTHIA_2B8", "PYTHIA_6B9", "NeoxDecoder", "layer_tensor_order", "rope_tables",
                 "layer_tensors_from_hf", "kv_cache_from_hf", "config_from_hf", "stack_tensors_from_hf"]
+
+    from .engine import Engine, Request  # noqa: E402
+    from .registry import architectures, load_model  # noqa: E402
+
+    __all__ += ["Engine", "Request", "architectures", "load_model"]

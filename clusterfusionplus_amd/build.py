@@ -1,10 +1,11 @@
-"""In-tree build of the two native libraries (no JIT cache, no install step):
+"""In-tree build of the native libraries (no JIT cache, no install step):
 
   libcfpp.so          HIP kernels + the C ABI of include/cfpp.h, compiled by hipcc for gfx950
-  _clusterfusion.so   the PyTorch binding (host C++ only), compiled by g++ against libtorch
+  _clusterfusion.so   the PyTorch binding of libcfpp.so (host C++ only), compiled by g++ against libtorch
+  libcfpp_seq.so      HIP kernels + the C ABI of include/cfpp_seq.h (sequence models: prefill and decode), bound by ctypes
 
-Both land next to this file so that they travel with the source tree.
-`python -m clusterfusionplus_amd.build` rebuilds both.
+They land next to this file so that they travel with the source tree.
+`python -m clusterfusionplus_amd.build` rebuilds all of them.
 """
 from __future__ import annotations
 
@@ -19,6 +20,7 @@ CSRC = os.path.join(PKG, "csrc")
 INCLUDE = os.path.join(ROOT, "include")
 LIB = os.path.join(PKG, "libcfpp.so")
 EXT = os.path.join(PKG, "_clusterfusion.so")
+SEQ_LIB = os.path.join(PKG, "libcfpp_seq.so")
 ROCM = os.environ.get("ROCM_PATH", "/opt/rocm")
 
 HIPCC_FLAGS = [
@@ -33,6 +35,7 @@ HIPCC_FLAGS = [
     # resolves the binding's dependency on "libcfpp.so" to it
     "-Wl,-soname,libcfpp.so",
 ]
+SEQ_FLAGS = [f.replace("libcfpp.so", "libcfpp_seq.so") for f in HIPCC_FLAGS]
 
 
 def _run(cmd):
@@ -57,20 +60,51 @@ def build_lib(trace: bool = False, out: str = LIB):
     return out
 
 
+def build_seq(out: str = SEQ_LIB):
+    """libcfpp_seq.so.  Written under a name of its own and moved into place, so that a process that finds the library
+    finds a whole one."""
+    part = f"{out}.{os.getpid()}.part"
+    hipcc = os.path.join(ROCM, "bin", "hipcc")
+    try:
+        _run([hipcc, *SEQ_FLAGS, f"-I{INCLUDE}", f"-I{CSRC}", os.path.join(CSRC, "seq_kernels.hip"), "-o", part])
+        os.replace(part, out)
+    finally:
+        if os.path.exists(part):
+            os.unlink(part)
+    return out
+
+
+def ensure_seq():
+    """Builds libcfpp_seq.so if it is not there (what a fresh checkout needs to run a sequence model, and no more)."""
+    if not os.path.exists(SEQ_LIB):
+        build_seq()
+
+
+def ensure_neox():
+    """Builds libcfpp.so and its PyTorch binding if they are not there."""
+    if not os.path.exists(LIB):
+        build_lib()
+    if not os.path.exists(EXT):
+        build_ext()
+
+
 def resource_report(out=None):
-    """Compiles the HIP library with the compiler's kernel-resource-usage remarks and returns one line per kernel:
+    """Compiles the HIP libraries with the compiler's kernel-resource-usage remarks and returns one line per kernel:
     VGPRs, AGPRs, scratch bytes per lane (register spills), static LDS bytes per workgroup, waves per SIMD."""
     import re
     import tempfile
     hipcc = os.path.join(ROCM, "bin", "hipcc")
+    remarks = ""
     with tempfile.TemporaryDirectory() as tmp:
-        cmd = [hipcc, *HIPCC_FLAGS, "-Rpass-analysis=kernel-resource-usage", f"-I{INCLUDE}", f"-I{CSRC}",
-               os.path.join(CSRC, "cfpp_kernels.hip"), "-o", os.path.join(tmp, "libcfpp.so")]
-        res = subprocess.run(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
-    if res.returncode != 0:
-        raise RuntimeError("resource report: compilation failed\n" + res.stdout[-2000:])
+        for flags, src in ((HIPCC_FLAGS, "cfpp_kernels.hip"), (SEQ_FLAGS, "seq_kernels.hip")):
+            cmd = [hipcc, *flags, "-Rpass-analysis=kernel-resource-usage", f"-I{INCLUDE}", f"-I{CSRC}",
+                   os.path.join(CSRC, src), "-o", os.path.join(tmp, "lib.so")]
+            res = subprocess.run(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
+            if res.returncode != 0:
+                raise RuntimeError("resource report: compilation failed\n" + res.stdout[-2000:])
+            remarks += res.stdout
     rows = []
-    for block in re.split(r"remark: [^\n]*Function Name: ", res.stdout)[1:]:
+    for block in re.split(r"remark: [^\n]*Function Name: ", remarks)[1:]:
         name = block.split()[0]
         nice = subprocess.run(["c++filt", name], stdout=subprocess.PIPE, text=True).stdout.strip() or name
         if nice.startswith("_Z"):
@@ -80,9 +114,10 @@ def resource_report(out=None):
             if m:
                 n = int(m.group(1))
                 base = name[m.end():m.end() + n]
-                targs = re.match(r"I((?:L[ib]\d+E)+)E", name[m.end() + n:])
+                targs = re.match(r"I((?:DF16b|f)?)((?:L[ib]\d+E)+)E", name[m.end() + n:])
                 if targs:
-                    vals = [v if k == "i" else ("true" if v == "1" else "false") for k, v in re.findall(r"L([ib])(\d+)E", targs.group(1))]
+                    vals = [{"DF16b": "bf16", "f": "float"}[targs.group(1)]] if targs.group(1) else []
+                    vals += [v if k == "i" else ("true" if v == "1" else "false") for k, v in re.findall(r"L([ib])(\d+)E", targs.group(2))]
                     base += "<" + ", ".join(vals) + ">"
                 nice = base
         nice = nice.replace("(anonymous namespace)::", "").replace("void ", "")
@@ -131,6 +166,7 @@ def build_stream_probe(out=os.path.join(PKG, "stream_probe_bin")):
 def build_all():
     build_lib()
     build_ext()
+    build_seq()
 
 
 if __name__ == "__main__":
@@ -141,11 +177,14 @@ if __name__ == "__main__":
     ap.add_argument("--stream-probe", action="store_true", help="only build the bare read probes (stream_probe.py runs them)")
     ap.add_argument("--resource-report", action="store_true",
                     help="only print registers, scratch, LDS and occupancy of every kernel (compiler remarks)")
+    ap.add_argument("--seq", action="store_true", help="only build the sequence models' library")
     a = ap.parse_args()
     if a.stream_probe:
         build_stream_probe()
     elif a.resource_report:
         print(resource_report())
+    elif a.seq:
+        build_seq()
     elif a.trace_lib:
         build_lib(trace=True, out=a.trace_lib)
     else:

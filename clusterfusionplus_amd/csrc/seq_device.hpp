@@ -1,0 +1,246 @@
+// Device-side building blocks of the sequence models (prefill in portions + decode) for gfx950.
+//
+// Everything is written in units of 16 bytes, so that one body serves both element types: 8 bf16 values (one
+// v_mfma_f32_16x16x32_bf16 per unit and lane) or 4 fp32 values (four v_mfma_f32_16x16x4_f32, true fp32).  The order of k
+// inside a product is free as long as both operands use the same one.
+//
+// Matrix products put the weight rows (attention: keys, value columns) on the MFMA's row operand and the tokens (attention:
+// query columns) on its column operand: a lane then holds four consecutive rows of one token, which makes the stores wide,
+// puts the interleaved gate and up rows of one output into the same lane, and leaves the softmax of a query in the lanes
+// of one column.
+#pragma once
+#include "cfpp_device.hpp"
+
+namespace cfpp {
+
+typedef __bf16 bf16_t;
+typedef __bf16 bf16x2_t __attribute__((ext_vector_type(2)));
+typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+typedef uint32_t u32x2 __attribute__((ext_vector_type(2)));
+
+constexpr int kRowBytes = 128;                    // matrix rows are padded to this
+constexpr int kSeqThreads = 256;                  // threads of every sequence kernel: four waves
+constexpr int kSeqWaves = kSeqThreads / kWave;
+constexpr float kLog2e = 1.4426950408889634f;
+
+template <typename T> struct Unit;                // elements in 16 bytes
+template <> struct Unit<bf16_t> { static constexpr int n = 8; };
+template <> struct Unit<float> { static constexpr int n = 4; };
+
+__device__ __forceinline__ float to_f32(bf16_t v) { return (float)v; }
+__device__ __forceinline__ float to_f32(float v) { return v; }
+template <typename T> __device__ __forceinline__ T from_f32(float v) { return (T)v; }
+
+template <typename T> __device__ __forceinline__ f32x4 mma16(u32x4 a, u32x4 b, f32x4 c);
+template <> __device__ __forceinline__ f32x4 mma16<bf16_t>(u32x4 a, u32x4 b, f32x4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), c, 0, 0, 0);
+}
+template <> __device__ __forceinline__ f32x4 mma16<float>(u32x4 a, u32x4 b, f32x4 c) {
+    const f32x4 fa = __builtin_bit_cast(f32x4, a), fb = __builtin_bit_cast(f32x4, b);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) c = __builtin_amdgcn_mfma_f32_16x16x4f32(fa[j], fb[j], c, 0, 0, 0);
+    return c;
+}
+
+// dot product of two 16-byte units, accumulated in fp32
+template <typename T> __device__ __forceinline__ float dot16(u32x4 w, u32x4 x, float acc);
+template <> __device__ __forceinline__ float dot16<bf16_t>(u32x4 w, u32x4 x, float acc) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const uint32_t wj = w[j], xj = x[j];             // (a bit cast of a vector's element itself reads element 0)
+        acc = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2_t, wj), __builtin_bit_cast(bf16x2_t, xj), acc, false);
+    }
+    return acc;
+}
+template <> __device__ __forceinline__ float dot16<float>(u32x4 w, u32x4 x, float acc) {
+    const f32x4 fw = __builtin_bit_cast(f32x4, w), fx = __builtin_bit_cast(f32x4, x);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc = fmadd(fw[j], fx[j], acc);
+    return acc;
+}
+
+// 64 lanes copy 64 units from memory straight to LDS; the lanes' units land next to each other from `lds` (wave-uniform) on
+__device__ __forceinline__ void copy_to_lds16(const void* g, void* lds) {
+    __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(uintptr_t)g,
+                                     (__attribute__((address_space(3))) void*)(uintptr_t)lds, 16, 0, 0);
+}
+
+// sum over the workgroup, in every thread, in a fixed order; `red` holds kSeqWaves floats (2 of them: two sums at a time)
+__device__ __forceinline__ float block_sum(float v, float* red) {
+    v = wave_sum(v);
+    __syncthreads();
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    return (red[0] + red[1]) + (red[2] + red[3]);
+}
+
+__device__ __forceinline__ float inv_rms(float sum_sq, int n, float eps) { return 1.0f / sqrtf(sum_sq / (float)n + eps); }
+__device__ __forceinline__ float relu2(float v) { v = fmaxf(v, 0.0f); return v * v; }
+__device__ __forceinline__ float soft_cap(float v, float cap) { return cap > 0.0f ? cap * tanhf(v / cap) : v; }
+
+// Element d of one head after the norm over the whole projection (inv, w) and the rotation; `row` is the head's slice of
+// the projection, `w` of the norm weight, `cs` the (cos, sin) pairs of the position.
+__device__ __forceinline__ float norm_rotate(const float* __restrict__ row, const float* __restrict__ w, float inv, int d, int rot,
+                                             const float2* __restrict__ cs) {
+    const float a = row[d] * inv * w[d];
+    if (d >= rot) return a;
+    const float b = row[d ^ 1] * inv * w[d ^ 1];
+    const float2 t = cs[d >> 1];
+    return (d & 1) ? a * t.x + b * t.y : a * t.x - b * t.y;
+}
+
+// First position of position p's chunk (chunk 0: the whole past).
+__device__ __forceinline__ int chunk_start(int p, int chunk) { return chunk > 0 ? (p / chunk) * chunk : 0; }
+
+// ------------------------------------------------------------------------------------------------
+// attention
+// ------------------------------------------------------------------------------------------------
+// A wave works on 16 query columns; lane l belongs to column l & 15 and to row group g = l >> 4.  Scores of a 16-key tile
+// are one MFMA result: the lane holds keys 4g .. 4g + 3 of its column.  Those registers are the column operand of the
+// second product as they are: its k slots are taken in the order in which the lanes hold the keys, and the transposed value
+// tile in LDS (V^T, one row of keys per value column) is read in the same order.
+//
+// Attention weights stay in 32 bits.  With bf16 matrices they are split into a high and a low bf16 part, which carry 16
+// bits of the weight into the product, and both parts are multiplied.
+template <typename T, int KT> struct VtTile {
+    static constexpr int pitch = KT * (int)sizeof(T) + 16;      // bytes; 16 more than the keys: rows start in different banks
+};
+
+// 4 keys x one unit of value columns per step, transposed on the way into LDS.  `rowp(key)` is the address of a key's
+// value row, for keys 0 .. KT - 1 of the tile; threads tid of nthreads share the tile.
+template <typename T, int KT, int NT, int NTHREADS, typename RowPtr>
+__device__ __forceinline__ void stage_vt(char* vt, int vunits, int tid, RowPtr rowp) {
+    constexpr int UE = Unit<T>::n, KG = KT / 4;
+    constexpr int ITERS = (KG * (NT / UE) + NTHREADS - 1) / NTHREADS;
+    constexpr int BATCH = ITERS < 2 ? ITERS : 2;
+#pragma unroll
+    for (int it0 = 0; it0 < ITERS; it0 += BATCH) {
+        u32x4 r[BATCH][4];
+#pragma unroll
+        for (int b = 0; b < BATCH; ++b) {
+            const int idx = tid + (it0 + b) * NTHREADS, kg = idx % KG, vc = idx / KG;
+            if (vc < vunits) {
+#pragma unroll
+                for (int j = 0; j < 4; ++j) r[b][j] = ld16(rowp(kg * 4 + j) + (size_t)vc * 16);
+            }
+        }
+#pragma unroll
+        for (int b = 0; b < BATCH; ++b) {
+            const int idx = tid + (it0 + b) * NTHREADS, kg = idx % KG, vc = idx / KG;
+            if (vc < vunits) {
+                if constexpr (sizeof(T) == 2) {
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) {
+                        const int sh = (e & 1) * 16;
+                        const uint32_t a = (r[b][0][e >> 1] >> sh) & 0xffffu, bb = (r[b][1][e >> 1] >> sh) & 0xffffu;
+                        const uint32_t c = (r[b][2][e >> 1] >> sh) & 0xffffu, d = (r[b][3][e >> 1] >> sh) & 0xffffu;
+                        u32x2 v = {a | (bb << 16), c | (d << 16)};
+                        *reinterpret_cast<u32x2*>(vt + (vc * 8 + e) * VtTile<T, KT>::pitch + kg * 8) = v;
+                    }
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        u32x4 v = {r[b][0][e], r[b][1][e], r[b][2][e], r[b][3][e]};
+                        *reinterpret_cast<u32x4*>(vt + (vc * 4 + e) * VtTile<T, KT>::pitch + kg * 16) = v;
+                    }
+                }
+            }
+        }
+    }
+}
+
+template <int NT> struct AttnState {              // of one column tile
+    float m, l;                                   // running maximum (log2 domain) and denominator, the same in every row group
+    f32x4 acc[NT / 16];                           // value columns 16 i + 4 g + r of the lane's column
+};
+
+template <int NT>
+__device__ __forceinline__ void attn_reset(AttnState<NT>& st) {
+    st.m = kNegBig;
+    st.l = 0.0f;
+#pragma unroll
+    for (int i = 0; i < NT / 16; ++i) st.acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+}
+
+// s[kt][r]: scores (already times scale * log2 e; kNegBig and below: not seen) of keys 16 kt + 4 g + r.  Turns them into
+// weights relative to the new maximum and rescales the state.
+template <int NT, int NKT>
+__device__ __forceinline__ void attn_softmax(AttnState<NT>& st, f32x4 (&s)[NKT], int vtiles) {
+    float mx = kNegBig;
+#pragma unroll
+    for (int kt = 0; kt < NKT; ++kt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s[kt][r]);
+    mx = fmaxf(mx, xor_shfl(mx, 16));
+    mx = fmaxf(mx, xor_shfl(mx, 32));
+    const float m = fmaxf(st.m, mx);
+    const float c = fast_exp2(st.m - m);
+    float sum = 0.0f;
+#pragma unroll
+    for (int kt = 0; kt < NKT; ++kt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            // (a key that is not seen has weight zero also where the column has seen nothing yet and m is kNegBig itself)
+            const float p = s[kt][r] > kNegBig ? fast_exp2(s[kt][r] - m) : 0.0f;
+            s[kt][r] = p;
+            sum += p;
+        }
+    sum += xor_shfl(sum, 16);
+    sum += xor_shfl(sum, 32);
+    st.l = st.l * c + sum;
+    st.m = m;
+#pragma unroll
+    for (int i = 0; i < NT / 16; ++i)
+        if (i < vtiles) st.acc[i] *= c;
+}
+
+__device__ __forceinline__ uint32_t pack_bf16(float a, float b) {
+    bf16x2_t v = {(bf16_t)a, (bf16_t)b};
+    return __builtin_bit_cast(uint32_t, v);
+}
+
+// acc += V^T p for the keys of one tile
+template <typename T, int NT, int KT>
+__device__ __forceinline__ void attn_pv(AttnState<NT>& st, const f32x4 (&p)[KT / 16], const char* vt, int vtiles, int lane) {
+    const int col = lane & 15, g = lane >> 4;
+    if constexpr (sizeof(T) == 2) {
+        u32x4 hi[KT / 32], lo[KT / 32];
+#pragma unroll
+        for (int s = 0; s < KT / 32; ++s)
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {
+                const f32x4 v = p[2 * s + h];
+                f32x4 rest;
+#pragma unroll
+                for (int r = 0; r < 4; ++r) rest[r] = v[r] - (float)(bf16_t)v[r];
+                hi[s][2 * h] = pack_bf16(v[0], v[1]);
+                hi[s][2 * h + 1] = pack_bf16(v[2], v[3]);
+                lo[s][2 * h] = pack_bf16(rest[0], rest[1]);
+                lo[s][2 * h + 1] = pack_bf16(rest[2], rest[3]);
+            }
+#pragma unroll
+        for (int i = 0; i < NT / 16; ++i)
+            if (i < vtiles) {
+                const char* row = vt + (i * 16 + col) * VtTile<T, KT>::pitch + g * 8;
+#pragma unroll
+                for (int s = 0; s < KT / 32; ++s) {
+                    const u32x2 a = *reinterpret_cast<const u32x2*>(row + s * 64), b = *reinterpret_cast<const u32x2*>(row + s * 64 + 32);
+                    const u32x4 f = {a.x, a.y, b.x, b.y};
+                    st.acc[i] = mma16<T>(f, hi[s], st.acc[i]);
+                    st.acc[i] = mma16<T>(f, lo[s], st.acc[i]);
+                }
+            }
+    } else {
+#pragma unroll
+        for (int i = 0; i < NT / 16; ++i)
+            if (i < vtiles) {
+                const char* row = vt + (i * 16 + col) * VtTile<T, KT>::pitch + g * 16;
+#pragma unroll
+                for (int s = 0; s < KT / 16; ++s)
+                    st.acc[i] = mma16<T>(*reinterpret_cast<const u32x4*>(row + s * 64), __builtin_bit_cast(u32x4, p[s]), st.acc[i]);
+            }
+    }
+}
+
+}  // namespace cfpp

@@ -1,0 +1,1657 @@
+// Kernels and host side of the sequence models (include/cfpp_seq.h).
+//
+// Prefill (a portion of T tokens): per layer
+//   k_seq_gemm (q, k, v rows + bias) -> k_seq_qkv_finish (norms over the projections, rotation, value mixing) -> k_seq_attn ->
+//   k_seq_append (what later portions can see goes into the cache) -> k_seq_gemm (output rows) -> k_seq_postnorm ->
+//   k_seq_gemm (up rows with the activation) -> k_seq_gemm (down rows) -> k_seq_postnorm;
+//   table experts: the same two products over tiles of tokens sorted by expert (k_seq_route), plus the shared expert's.
+// Decode (one token): five launches per layer, each with its neighbours' work fused in:
+//   k_seq_gemv (residual sum + norm of the sublayer before | q, k, v rows + bias)
+//   k_seq_attn_decode (norms, rotation, value mixing, cache append, split-KV attention, merge)
+//   k_seq_gemv (output rows)
+//   k_seq_gemv (residual sum + norm | up rows of the chosen and the shared experts | activation)
+//   k_seq_gemv (down rows of all of them, weighted and summed)
+// then k_seq_gemv over the vocabulary (both last norms | head rows | soft cap | best logit per workgroup) and k_seq_pick.
+#include <hip/hip_runtime.h>
+#include <math.h>
+#include <stdint.h>
+#include <string.h>
+
+#include <algorithm>
+#include <map>
+#include <new>
+#include <utility>
+#include <vector>
+
+#include "cfpp_seq.h"
+#include "seq_device.hpp"
+
+using namespace cfpp;
+
+namespace {
+
+enum : int { kStToken = 0, kStPos = 1, kStSteps = 2, kStSlot = 3 };
+constexpr int kAttnCols = 16;          // query columns of a decode item (one MFMA column tile)
+constexpr int kMaxSeqSplit = 64;       // KV splits of a decode step
+
+// ------------------------------------------------------------------------------------------------
+// small kernels
+// ------------------------------------------------------------------------------------------------
+__global__ void k_seq_set_state(int* state, int slot, int token, int pos, int steps) {
+    if (threadIdx.x == 0) {
+        state[kStToken] = token;
+        state[kStPos] = pos;
+        state[kStSlot] = slot;
+        if (steps >= 0) state[kStSteps] = steps;
+    }
+}
+
+__global__ void k_seq_fill_zero(u32x4* p, size_t n) {
+    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) p[i] = u32x4{0, 0, 0, 0};
+}
+
+// One workgroup per token: embedding row -> residual stream (fp32) and product input (T).
+template <typename T>
+__global__ __launch_bounds__(kSeqThreads) void k_seq_embed(const int* __restrict__ tokens, const char* __restrict__ embed, int pitch, int width,
+                                                           float* __restrict__ x, char* __restrict__ xb) {
+    const int t = blockIdx.x;
+    const T* e = reinterpret_cast<const T*>(embed + (size_t)tokens[t] * pitch);
+    T* o = reinterpret_cast<T*>(xb + (size_t)t * pitch);
+    for (int i = threadIdx.x; i < width; i += kSeqThreads) {
+        x[(size_t)t * width + i] = to_f32(e[i]);
+        o[i] = e[i];
+    }
+}
+
+// x <- norm(alpha x + y + slot_weight * sum_j ys[t, j]); one workgroup per token.  `rows`: take the token rows[t] instead of
+// t and only write xb (the last norm, on the rows whose logits are wanted).
+struct SeqPostNorm {
+    const float* x;
+    float* x_out;            // may be x
+    const float* y;          // nullable
+    const float* ys;         // nullable: [T][top][width], outputs of the chosen experts
+    int top;
+    float slot_weight;
+    const float* w;
+    float alpha, eps;
+    int width;
+    char* xb;
+    int pitch;
+    const int* rows;
+    float* copy;             // nullable: receives the new residual row too
+};
+template <typename T>
+__global__ __launch_bounds__(kSeqThreads) void k_seq_postnorm(SeqPostNorm a) {
+    __shared__ float red[kSeqWaves];
+    extern __shared__ __align__(16) float ts[];
+    const int t = a.rows != nullptr ? a.rows[blockIdx.x] : (int)blockIdx.x;
+    const float* x = a.x + (size_t)t * a.width;
+    float ss = 0.0f;
+    for (int i = threadIdx.x; i < a.width; i += kSeqThreads) {
+        float s = 0.0f;
+        if (a.ys != nullptr) {
+            const float* ys = a.ys + (size_t)t * a.top * a.width + i;
+            for (int j = 0; j < a.top; ++j) s += ys[(size_t)j * a.width];
+            s *= a.slot_weight;
+        }
+        if (a.y != nullptr) s += a.y[(size_t)t * a.width + i];
+        const float v = a.rows != nullptr ? x[i] : fmadd(a.alpha, x[i], s);
+        ts[i] = v;
+        ss = fmadd(v, v, ss);
+    }
+    const float inv = inv_rms(block_sum(ss, red), a.width, a.eps);
+    T* xb = reinterpret_cast<T*>(a.xb + (size_t)blockIdx.x * a.pitch);
+    for (int i = threadIdx.x; i < a.width; i += kSeqThreads) {
+        const float v = ts[i] * inv * (1.0f + a.w[i]);
+        if (a.rows == nullptr) {
+            a.x_out[(size_t)t * a.width + i] = v;
+            if (a.copy != nullptr) a.copy[(size_t)t * a.width + i] = v;
+        }
+        xb[i] = from_f32<T>(v);
+    }
+}
+
+// One workgroup per token: raw q | k | v rows (fp32, biases included) -> norm over all of q and all of k, rotation, value
+// mixing -> q [T][H][Dp], portion k [G][cap][Dp] and v [G][cap][Vp].
+struct SeqQkv {
+    const float* qkv;
+    int ld;
+    const float *qn, *kn;
+    const float2* cs;        // [positions][rot / 2]
+    float eps, lambda;
+    int H, G, D, Dp, V, Vp, rot, pos0, cap;
+    int v_role;              // 0: plain, 1: this layer's values are the ones later layers mix in, 2: mix
+    float* v_first;          // [T][G * V]
+    char *q, *k, *v;
+};
+template <typename T>
+__global__ __launch_bounds__(kSeqThreads) void k_seq_qkv_finish(SeqQkv a) {
+    __shared__ float red[kSeqWaves];
+    const int t = blockIdx.x, nq = a.H * a.D, nk = a.G * a.D, nv = a.G * a.V;
+    const float* q = a.qkv + (size_t)t * a.ld;
+    const float *k = q + nq, *v = k + nk;
+    float sq = 0.0f, sk = 0.0f;
+    for (int i = threadIdx.x; i < nq; i += kSeqThreads) sq = fmadd(q[i], q[i], sq);
+    for (int i = threadIdx.x; i < nk; i += kSeqThreads) sk = fmadd(k[i], k[i], sk);
+    const float iq = inv_rms(block_sum(sq, red), nq, a.eps), ik = inv_rms(block_sum(sk, red), nk, a.eps);
+    const float2* cs = a.cs + (size_t)(a.pos0 + t) * (a.rot / 2);
+    T* qo = reinterpret_cast<T*>(a.q) + (size_t)t * a.H * a.Dp;
+    T* ko = reinterpret_cast<T*>(a.k) + (size_t)t * a.Dp;
+    T* vo = reinterpret_cast<T*>(a.v) + (size_t)t * a.Vp;
+    // (the padding of a row is written too: layers of other sizes share these buffers)
+    for (int i = threadIdx.x; i < a.H * a.Dp; i += kSeqThreads) {
+        const int h = i / a.Dp, d = i - h * a.Dp;
+        qo[i] = from_f32<T>(d < a.D ? norm_rotate(q + h * a.D, a.qn + h * a.D, iq, d, a.rot, cs) : 0.0f);
+    }
+    for (int i = threadIdx.x; i < a.G * a.Dp; i += kSeqThreads) {
+        const int g = i / a.Dp, d = i - g * a.Dp;
+        ko[(size_t)g * a.cap * a.Dp + d] = from_f32<T>(d < a.D ? norm_rotate(k + g * a.D, a.kn + g * a.D, ik, d, a.rot, cs) : 0.0f);
+    }
+    for (int i = threadIdx.x; i < a.G * a.Vp; i += kSeqThreads) {
+        const int g = i / a.Vp, d = i - g * a.Vp;
+        float x = 0.0f;
+        if (d < a.V) {
+            float* first = a.v_first + (size_t)t * nv + g * a.V + d;
+            x = v[g * a.V + d];
+            if (a.v_role == 1) *first = x;
+            if (a.v_role == 2) x = (1.0f - a.lambda) * x + a.lambda * *first;
+        }
+        vo[(size_t)g * a.cap * a.Vp + d] = from_f32<T>(x);
+    }
+}
+
+// Portion rows -> cache rows: one workgroup per kept position.
+struct SeqAppend { const char *k, *v; char *kc, *vc; int G, krow, vrow, cap, rows, first, row0; };
+__global__ __launch_bounds__(kSeqThreads) void k_seq_append(SeqAppend a) {
+    const int t = a.first + blockIdx.x, r = a.row0 + blockIdx.x;
+    const int ku = a.krow / 16, vu = a.vrow / 16;
+    for (int i = threadIdx.x; i < a.G * (ku + vu); i += kSeqThreads) {
+        const int g = i / (ku + vu), u = i - g * (ku + vu);
+        if (u < ku)
+            *reinterpret_cast<u32x4*>(a.kc + ((size_t)g * a.rows + r) * a.krow + u * 16) = ld16(a.k + ((size_t)g * a.cap + t) * a.krow + u * 16);
+        else
+            *reinterpret_cast<u32x4*>(a.vc + ((size_t)g * a.rows + r) * a.vrow + (u - ku) * 16) = ld16(a.v + ((size_t)g * a.cap + t) * a.vrow + (u - ku) * 16);
+    }
+}
+
+// ------------------------------------------------------------------------------------------------
+// matrix products of a portion: out[token][row] = W[row] . a[token]
+// ------------------------------------------------------------------------------------------------
+enum : int { kEpiF32 = 0, kEpiRelu2 = 1, kEpiGated = 2, kEpiHead = 3 };
+struct SeqGemm {
+    const char* w;           // [n rows][kbytes]
+    const char* a;           // [tokens][lda bytes]
+    int n, m, kbytes, lda;
+    const float* bias;       // nullable (kEpiF32)
+    float* yf;               // kEpiF32 / kEpiHead: [tokens][ldy]
+    int ldy;
+    char* yt;                // kEpiRelu2 / kEpiGated: T, [tokens][ldyt bytes]
+    int ldyt;
+    float cap;
+    // tiles of tokens sorted by expert (tile_off null: a plain product)
+    const int* tile_off;     // [experts + 1] prefix sums of tiles
+    const int* row_off;      // [experts + 1] prefix sums of sorted slots
+    const int* slots;        // sorted slots: token * top + j
+    int experts, slot_div;   // input row of slot s: s / slot_div
+    size_t w_stride;
+};
+
+// rows of 128 bytes: units of row r are stored at unit ^ swz(r), which spreads 16 consecutive rows over all banks
+__device__ __forceinline__ int swz128(int row) { return (row >> 1) & 7; }
+
+template <typename T, int BW, int BT, int EPI>
+__global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemm(SeqGemm p) {
+    constexpr int MI = BW / 32, NI = BT / 32;            // 16 x 16 tiles of a wave; waves are 2 (rows) x 2 (tokens)
+    constexpr int WI = BW / 32, AI = BT / 32;            // 1 KB copies per wave and k step
+    __shared__ __align__(1024) char lds[2][(BW + BT) * kRowBytes];
+    const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63;
+    const int wr = wave >> 1, wc = wave & 1;
+
+    const int tiles_w = (p.n + BW - 1) / BW;
+    int tw, tt, m = p.m, row0 = 0;
+    const char* w = p.w;
+    {
+        // every XCD works on a contiguous range of tiles; inside it tiles go through groups of up to 8 token tiles
+        const int total = gridDim.x, per = total / 8, rem = total % 8, xcd = blockIdx.x % 8, i = blockIdx.x / 8;
+        const int id = xcd * per + min(xcd, rem) + i;
+        if (p.tile_off != nullptr) {
+            tt = id / tiles_w;
+            tw = id - tt * tiles_w;
+            if (tt >= p.tile_off[p.experts]) return;
+            int lo = 0, hi = p.experts;                  // last expert whose first tile is <= tt
+            while (hi - lo > 1) {
+                const int mid = (lo + hi) >> 1;
+                if (p.tile_off[mid] <= tt) lo = mid; else hi = mid;
+            }
+            // (experts without tokens have no tiles: skip to the one that owns the tile)
+            while (p.tile_off[lo + 1] <= tt) ++lo;
+            w += (size_t)lo * p.w_stride;
+            row0 = p.row_off[lo] + (tt - p.tile_off[lo]) * BT;
+            m = p.row_off[lo + 1] - row0;
+            tt = 0;
+        } else {
+            const int tiles_t = (p.m + BT - 1) / BT, group = 8 * tiles_w, gi = id / group, first = gi * 8;
+            const int gs = min(8, tiles_t - first), r = id - gi * group;
+            tt = first + r % gs;
+            tw = r / gs;
+        }
+    }
+    const char* src_w[WI];
+    const char* src_a[AI];
+#pragma unroll
+    for (int i = 0; i < WI; ++i) {
+        const int r = wave * (BW / 4) + i * 8 + (lane >> 3);
+        src_w[i] = w + (size_t)min(tw * BW + r, p.n - 1) * p.kbytes + ((lane & 7) ^ swz128(r)) * 16;
+    }
+#pragma unroll
+    for (int i = 0; i < AI; ++i) {
+        const int r = wave * (BT / 4) + i * 8 + (lane >> 3);
+        int tok = min(tt * BT + r, m - 1);
+        if (p.tile_off != nullptr) tok = p.slots[row0 + tok] / p.slot_div;
+        src_a[i] = p.a + (size_t)tok * p.lda + ((lane & 7) ^ swz128(r)) * 16;
+    }
+    auto stage = [&](int buf, int k) {
+        char* base = lds[buf];
+#pragma unroll
+        for (int i = 0; i < WI; ++i) copy_to_lds16(src_w[i] + k, base + (wave * (BW / 4) + i * 8) * kRowBytes);
+#pragma unroll
+        for (int i = 0; i < AI; ++i) copy_to_lds16(src_a[i] + k, base + BW * kRowBytes + (wave * (BT / 4) + i * 8) * kRowBytes);
+    };
+    f32x4 acc[MI][NI];
+#pragma unroll
+    for (int i = 0; i < MI; ++i)
+#pragma unroll
+        for (int j = 0; j < NI; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+
+    const int col = lane & 15, g = lane >> 4, nk = p.kbytes / kRowBytes;
+    stage(0, 0);
+    for (int k = 0; k < nk; ++k) {
+        __syncthreads();                                 // this step's tile has arrived; the other buffer is free
+        if (k + 1 < nk) stage((k + 1) & 1, (k + 1) * kRowBytes);
+        const char* lw = lds[k & 1];
+        const char* la = lw + BW * kRowBytes;
+#pragma unroll
+        for (int s = 0; s < 2; ++s) {
+            u32x4 fw[MI], fa[NI];
+#pragma unroll
+            for (int i = 0; i < MI; ++i) {
+                const int r = wr * (BW / 2) + i * 16 + col;
+                fw[i] = *reinterpret_cast<const u32x4*>(lw + r * kRowBytes + ((s * 4 + g) ^ swz128(r)) * 16);
+            }
+#pragma unroll
+            for (int j = 0; j < NI; ++j) {
+                const int r = wc * (BT / 2) + j * 16 + col;
+                fa[j] = *reinterpret_cast<const u32x4*>(la + r * kRowBytes + ((s * 4 + g) ^ swz128(r)) * 16);
+            }
+#pragma unroll
+            for (int i = 0; i < MI; ++i)
+#pragma unroll
+                for (int j = 0; j < NI; ++j) acc[i][j] = mma16<T>(fw[i], fa[j], acc[i][j]);
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < NI; ++j) {
+        const int tl = tt * BT + wc * (BT / 2) + j * 16 + col;
+        if (tl >= m) continue;
+        const int row = p.tile_off != nullptr ? p.slots[row0 + tl] : tl;
+#pragma unroll
+        for (int i = 0; i < MI; ++i) {
+            const int n0 = tw * BW + wr * (BW / 2) + i * 16 + g * 4;
+            const f32x4 v = acc[i][j];
+            if constexpr (EPI == kEpiF32 || EPI == kEpiHead) {
+                float* y = p.yf + (size_t)row * p.ldy + n0;
+                f32x4 o = v;
+                if (EPI == kEpiF32 && p.bias != nullptr) {
+#pragma unroll
+                    for (int r = 0; r < 4; ++r)
+                        if (n0 + r < p.n) o[r] += p.bias[n0 + r];
+                }
+                if (EPI == kEpiHead) {
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) o[r] = soft_cap(o[r], p.cap);
+                }
+                if (n0 + 3 < p.n && (p.ldy & 3) == 0) {
+                    *reinterpret_cast<f32x4*>(y) = o;
+                } else {
+#pragma unroll
+                    for (int r = 0; r < 4; ++r)
+                        if (n0 + r < p.n) y[r] = o[r];
+                }
+            } else if constexpr (EPI == kEpiRelu2) {
+                T* y = reinterpret_cast<T*>(p.yt + (size_t)row * p.ldyt) + n0;
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+                    if (n0 + r < p.n) y[r] = from_f32<T>(relu2(v[r]));
+            } else {
+                T* y = reinterpret_cast<T*>(p.yt + (size_t)row * p.ldyt) + n0 / 2;
+#pragma unroll
+                for (int r = 0; r < 4; r += 2)
+                    if (n0 + r < p.n) y[r / 2] = from_f32<T>(silu(v[r]) * v[r + 1]);
+            }
+        }
+    }
+}
+
+// Slots (token * top + j) sorted by expert, per layer with table experts: one workgroup per such layer.
+struct SeqRoute { const int* table; int* tile_off; int* row_off; int* slots; int experts, top; };
+__global__ __launch_bounds__(1024) void k_seq_route(const SeqRoute* layers, const int* __restrict__ tokens, int T, int bt) {
+    extern __shared__ int sh[];
+    const SeqRoute a = layers[blockIdx.x];
+    int *cnt = sh, *next = sh + a.experts;
+    for (int e = threadIdx.x; e < a.experts; e += blockDim.x) cnt[e] = 0;
+    __syncthreads();
+    const int n = T * a.top;
+    for (int s = threadIdx.x; s < n; s += blockDim.x) {
+        const int t = s / a.top;
+        atomicAdd(&cnt[a.table[(size_t)tokens[t] * a.top + (s - t * a.top)]], 1);
+    }
+    __syncthreads();
+    if (threadIdx.x == 0) {
+        int rows = 0, tiles = 0;
+        for (int e = 0; e < a.experts; ++e) {
+            const int c = cnt[e];
+            a.row_off[e] = rows;
+            a.tile_off[e] = tiles;
+            next[e] = rows;
+            rows += c;
+            tiles += (c + bt - 1) / bt;
+        }
+        a.row_off[a.experts] = rows;
+        a.tile_off[a.experts] = tiles;
+    }
+    __syncthreads();
+    for (int s = threadIdx.x; s < n; s += blockDim.x) {
+        const int t = s / a.top;
+        a.slots[atomicAdd(&next[a.table[(size_t)tokens[t] * a.top + (s - t * a.top)]], 1)] = s;
+    }
+}
+
+// ------------------------------------------------------------------------------------------------
+// attention of a portion
+// ------------------------------------------------------------------------------------------------
+// The query columns of one key / value head are (token, head of the group), head fastest; a workgroup takes 64 CT of them
+// and walks the keys its tokens can see, first the cached ones, then the portion's own.  The softmax is online, the sink is
+// added to the denominator at the end.
+struct SeqAttn {
+    const char *q, *k, *v, *kc, *vc;
+    char* out;
+    const float* sink;
+    int T, H, R, dsteps, krow, vrow, V, vtiles, pos0, chunk, cap, rows, ldo;
+    float scale_log2;
+};
+template <int UN> __device__ __forceinline__ int swz_key(int row) { return UN == 8 ? (row >> 1) & 7 : row & 15; }
+
+template <typename T, int NT, int CT>
+__global__ __launch_bounds__(kSeqThreads) void k_seq_attn(SeqAttn a) {
+    constexpr int KT = sizeof(T) == 2 ? 64 : 32;
+    constexpr int NB = NT * (int)sizeof(T), UN = NB / 16, RPC = 1024 / NB;   // bytes and units of a key row in LDS, rows per copy
+    __shared__ __align__(1024) char ks[KT * NB];
+    __shared__ __align__(16) char vt[NT * VtTile<T, KT>::pitch];
+    const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, col = lane & 15, g = lane >> 4;
+    const int gq = blockIdx.y, ncols = a.T * a.R, c0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * 64 * CT;
+
+    int tok[CT], head[CT], pq[CT], first[CT];
+    bool mine[CT];
+    u32x4 qf[CT][NB / 64];
+    AttnState<NT> st[CT];
+#pragma unroll
+    for (int ct = 0; ct < CT; ++ct) {
+        const int c = c0 + (wave * CT + ct) * 16 + col, cc = min(c, ncols - 1);
+        mine[ct] = c < ncols;
+        tok[ct] = cc / a.R;
+        head[ct] = gq * a.R + (cc - tok[ct] * a.R);
+        pq[ct] = a.pos0 + tok[ct];
+        first[ct] = chunk_start(pq[ct], a.chunk);
+        const char* qr = a.q + ((size_t)tok[ct] * a.H + head[ct]) * a.krow + g * 16;
+#pragma unroll
+        for (int s = 0; s < NB / 64; ++s)
+            if (s < a.dsteps) qf[ct][s] = ld16(qr + s * 64);
+        attn_reset(st[ct]);
+    }
+    const int t_first = c0 / a.R, t_last = min(a.T - 1, (c0 + 64 * CT - 1) / a.R);
+    const int k_first = chunk_start(a.pos0 + t_first, a.chunk), k_end = a.pos0 + t_last + 1;
+    const int dunits = a.krow / 16, vunits = a.vrow / 16;
+
+    for (int seg = 0; seg < 2; ++seg) {
+        const int lo = seg == 0 ? k_first : max(k_first, a.pos0), hi = seg == 0 ? min(k_end, a.pos0) : k_end;
+        if (lo >= hi) continue;
+        // row of position p: base + p * row bytes
+        const int base_pos = seg == 0 ? chunk_start(a.pos0, a.chunk) : a.pos0;
+        const size_t row0 = (size_t)gq * (seg == 0 ? a.rows : a.cap);
+        const char* kb = (seg == 0 ? a.kc : a.k) + row0 * a.krow;
+        const char* vb = (seg == 0 ? a.vc : a.v) + row0 * a.vrow;
+        for (int k0 = lo; k0 < hi; k0 += KT) {
+            __syncthreads();
+            for (int i = wave; i < KT / RPC; i += kSeqWaves) {
+                const int r = i * RPC + lane / UN;
+                int u = (lane % UN) ^ swz_key<UN>(r);
+                if (u >= dunits) u = 0;
+                copy_to_lds16(kb + (size_t)(min(k0 + r, hi - 1) - base_pos) * a.krow + u * 16, ks + i * 1024);
+            }
+            stage_vt<T, KT, NT, kSeqThreads>(vt, vunits, tid, [&](int key) { return vb + (size_t)(min(k0 + key, hi - 1) - base_pos) * a.vrow; });
+            __syncthreads();
+            f32x4 s[CT][KT / 16];
+#pragma unroll
+            for (int kt = 0; kt < KT / 16; ++kt) {
+#pragma unroll
+                for (int ct = 0; ct < CT; ++ct) s[ct][kt] = f32x4{0.f, 0.f, 0.f, 0.f};
+                const int r = kt * 16 + col;
+#pragma unroll
+                for (int d = 0; d < NB / 64; ++d)
+                    if (d < a.dsteps) {
+                        const u32x4 kf = *reinterpret_cast<const u32x4*>(ks + r * NB + ((d * 4 + g) ^ swz_key<UN>(r)) * 16);
+#pragma unroll
+                        for (int ct = 0; ct < CT; ++ct) s[ct][kt] = mma16<T>(kf, qf[ct][d], s[ct][kt]);
+                    }
+            }
+#pragma unroll
+            for (int ct = 0; ct < CT; ++ct) {
+#pragma unroll
+                for (int kt = 0; kt < KT / 16; ++kt)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) {
+                        const int key = k0 + kt * 16 + g * 4 + r;
+                        const bool see = key < hi && key <= pq[ct] && key >= first[ct];
+                        s[ct][kt][r] = see ? s[ct][kt][r] * a.scale_log2 : kNegBig;
+                    }
+                attn_softmax<NT, KT / 16>(st[ct], s[ct], a.vtiles);
+                attn_pv<T, NT, KT>(st[ct], s[ct], vt, a.vtiles, lane);
+            }
+        }
+    }
+#pragma unroll
+    for (int ct = 0; ct < CT; ++ct) {
+        if (!mine[ct]) continue;
+        const float snk = a.sink[head[ct]] * kLog2e, m = fmaxf(st[ct].m, snk), c = fast_exp2(st[ct].m - m);
+        const float f = c / (st[ct].l * c + fast_exp2(snk - m));
+        T* o = reinterpret_cast<T*>(a.out + (size_t)tok[ct] * a.ldo) + head[ct] * a.V;
+#pragma unroll
+        for (int i = 0; i < NT / 16; ++i)
+            if (i < a.vtiles) {
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const int v = i * 16 + g * 4 + r;
+                    if (v < a.V) o[v] = from_f32<T>(st[ct].acc[i][r] * f);
+                }
+            }
+    }
+}
+
+// ------------------------------------------------------------------------------------------------
+// attention of one token
+// ------------------------------------------------------------------------------------------------
+// Workgroup (split, key / value head x group of 16 query heads).  Its prologue makes q from the raw projection; the split
+// that holds the newest position also makes that position's k and v rows and appends them.  Every wave takes every fourth
+// tile of the split's keys; the waves merge in LDS, the splits through memory, by the workgroup that arrives last.
+struct SeqAttnDec {
+    const float* qkv;
+    const float *qn, *kn, *sink;
+    const float2* cs;
+    const int* state;
+    char *kc, *vc;           // this layer's caches, slot 0
+    size_t k_slot, v_slot;   // bytes per slot
+    float* v_first;
+    char* out;               // T [H * V]
+    float* part;             // [items][ns][16][Vp + 2]
+    int* cnt;                // [items][kHeadCntStride], self-resetting
+    float eps, lambda, scale_log2;
+    int v_role, H, G, R, nct, D, V, rot, chunk, krow, vrow, dsteps, vtiles, rows, ns;
+};
+template <typename T, int NT> struct DecTile { static constexpr int kt = sizeof(T) == 2 ? 32 : (NT <= 128 ? 32 : 16); };
+
+template <typename T, int NT>
+__global__ __launch_bounds__(kSeqThreads) void k_seq_attn_decode(SeqAttnDec a) {
+    constexpr int KT = DecTile<T, NT>::kt, NB = NT * (int)sizeof(T);
+    constexpr int VB = NT * VtTile<T, KT>::pitch, MB = kAttnCols * NT * 4;
+    __shared__ __align__(16) char buf[kSeqWaves * (VB > MB ? VB : MB)];
+    __shared__ __align__(16) char qs[kAttnCols * NB];
+    __shared__ float red[kSeqWaves], wm[kSeqWaves][kAttnCols], wl[kSeqWaves][kAttnCols];
+    __shared__ float sm[kMaxSeqSplit][kAttnCols], sl[kMaxSeqSplit][kAttnCols];
+    __shared__ int last;
+    const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, col = lane & 15, g = lane >> 4;
+    const int item = blockIdx.y, gq = item / a.nct, cols0 = (item - gq * a.nct) * kAttnCols, ncols = min(kAttnCols, a.R - cols0);
+    const int pos = a.state[kStPos], slot = a.state[kStSlot];
+    const int k_first = chunk_start(pos, a.chunk), n = pos - k_first + 1;
+    const int tile = KT * kSeqWaves;
+    const int per = ((n + a.ns - 1) / a.ns + tile - 1) / tile * tile, nsplit = (n + per - 1) / per;
+    const int sp = blockIdx.x;
+    if (sp >= nsplit) return;
+    const int k0 = k_first + sp * per, k1 = min(k0 + per, pos + 1);
+    char* kc = a.kc + slot * a.k_slot + (size_t)gq * a.rows * a.krow;
+    char* vc = a.vc + slot * a.v_slot + (size_t)gq * a.rows * a.vrow;
+    const float2* cs = a.cs + (size_t)pos * (a.rot / 2);
+
+    const int nq = a.H * a.D, nk = a.G * a.D, nv = a.G * a.V;
+    const float *q = a.qkv, *k = q + nq, *v = k + nk;
+    {
+        float sq = 0.0f;
+        for (int i = tid; i < nq; i += kSeqThreads) sq = fmadd(q[i], q[i], sq);
+        const float iq = inv_rms(block_sum(sq, red), nq, a.eps);
+        const int dp = a.krow / (int)sizeof(T);
+        for (int i = tid; i < kAttnCols * dp; i += kSeqThreads) {
+            const int c = i / dp, d = i - c * dp, h = gq * a.R + cols0 + c;
+            float x = 0.0f;
+            if (c < ncols && d < a.D) x = norm_rotate(q + (size_t)h * a.D, a.qn + (size_t)h * a.D, iq, d, a.rot, cs);
+            reinterpret_cast<T*>(qs)[c * NT + d] = from_f32<T>(x);
+        }
+    }
+    if (k1 == pos + 1) {
+        float sk = 0.0f;
+        for (int i = tid; i < nk; i += kSeqThreads) sk = fmadd(k[i], k[i], sk);
+        const float ik = inv_rms(block_sum(sk, red), nk, a.eps);
+        T* ko = reinterpret_cast<T*>(kc + (size_t)(pos - k_first) * a.krow);
+        T* vo = reinterpret_cast<T*>(vc + (size_t)(pos - k_first) * a.vrow);
+        for (int d = tid; d < a.D; d += kSeqThreads)
+            ko[d] = from_f32<T>(norm_rotate(k + (size_t)gq * a.D, a.kn + (size_t)gq * a.D, ik, d, a.rot, cs));
+        for (int d = tid; d < a.V; d += kSeqThreads) {
+            float x = v[gq * a.V + d];
+            if (a.v_role == 1) a.v_first[gq * a.V + d] = x;
+            if (a.v_role == 2) x = (1.0f - a.lambda) * x + a.lambda * a.v_first[gq * a.V + d];
+            vo[d] = from_f32<T>(x);
+        }
+    }
+    __syncthreads();
+    u32x4 qf[NB / 64];
+#pragma unroll
+    for (int s = 0; s < NB / 64; ++s)
+        if (s < a.dsteps) qf[s] = *reinterpret_cast<const u32x4*>(qs + col * NB + s * 64 + g * 16);
+
+    AttnState<NT> st;
+    attn_reset(st);
+    char* vt = buf + wave * VB;
+    for (int kb = k0 + wave * KT; kb < k1; kb += tile) {
+        f32x4 s[KT / 16];
+#pragma unroll
+        for (int kt = 0; kt < KT / 16; ++kt) {
+            const char* kr = kc + (size_t)(min(kb + kt * 16 + col, k1 - 1) - k_first) * a.krow + g * 16;
+            u32x4 kf[NB / 64];
+#pragma unroll
+            for (int d = 0; d < NB / 64; ++d)
+                if (d < a.dsteps) kf[d] = ld16(kr + d * 64);
+            s[kt] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int d = 0; d < NB / 64; ++d)
+                if (d < a.dsteps) s[kt] = mma16<T>(kf[d], qf[d], s[kt]);
+        }
+        stage_vt<T, KT, NT, kWave>(vt, a.vrow / 16, lane, [&](int key) { return vc + (size_t)(min(kb + key, k1 - 1) - k_first) * a.vrow; });
+#pragma unroll
+        for (int kt = 0; kt < KT / 16; ++kt)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) s[kt][r] = kb + kt * 16 + g * 4 + r < k1 ? s[kt][r] * a.scale_log2 : kNegBig;
+        attn_softmax<NT, KT / 16>(st, s, a.vtiles);
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+        __builtin_amdgcn_wave_barrier();                 // the tile in LDS belongs to this wave alone
+        attn_pv<T, NT, KT>(st, s, vt, a.vtiles, lane);
+        __builtin_amdgcn_wave_barrier();
+    }
+    // waves of the workgroup
+    __syncthreads();
+    float* wacc = reinterpret_cast<float*>(buf);         // [wave][column][NT]
+    if (g == 0) {
+        wm[wave][col] = st.m;
+        wl[wave][col] = st.l;
+    }
+#pragma unroll
+    for (int i = 0; i < NT / 16; ++i)
+        if (i < a.vtiles) *reinterpret_cast<f32x4*>(wacc + (wave * kAttnCols + col) * NT + i * 16 + g * 4) = st.acc[i];
+    __syncthreads();
+    const int vp = a.vtiles * 16, stride = vp + 2;
+    float* part = a.part + (size_t)item * a.ns * kAttnCols * stride;
+    for (int i = tid; i < ncols * vp; i += kSeqThreads) {
+        const int c = i / vp, x = i - c * vp;
+        const float m = fmaxf(fmaxf(wm[0][c], wm[1][c]), fmaxf(wm[2][c], wm[3][c]));
+        float acc = 0.0f, l = 0.0f;
+#pragma unroll
+        for (int w = 0; w < kSeqWaves; ++w) {
+            const float f = fast_exp2(wm[w][c] - m);
+            acc = fmadd(wacc[(w * kAttnCols + c) * NT + x], f, acc);
+            l = fmadd(wl[w][c], f, l);
+        }
+        if (nsplit == 1) {
+            const int h = gq * a.R + cols0 + c;
+            const float snk = a.sink[h] * kLog2e, mm = fmaxf(m, snk), f = fast_exp2(m - mm);
+            if (x < a.V) reinterpret_cast<T*>(a.out)[(size_t)h * a.V + x] = from_f32<T>(acc * f / (l * f + fast_exp2(snk - mm)));
+        } else {
+            float* pr = part + ((size_t)sp * kAttnCols + c) * stride;
+            st_agent(pr + 2 + x, acc);
+            if (x == 0) {
+                st_agent(pr, m);
+                st_agent(pr + 1, l);
+            }
+        }
+    }
+    if (nsplit == 1) return;
+    drain_memory_ops();
+    __syncthreads();
+    if (tid == 0) {
+        int* ctr = a.cnt + item * kHeadCntStride;
+        const int done = __hip_atomic_fetch_add(ctr, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == nsplit - 1;
+        if (done) __hip_atomic_store(ctr, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        last = done;
+    }
+    __syncthreads();
+    if (!last) return;
+    for (int i = tid; i < nsplit * ncols; i += kSeqThreads) {
+        const int s = i / ncols, c = i - s * ncols;
+        const float* pr = part + ((size_t)s * kAttnCols + c) * stride;
+        sm[s][c] = ld_agent(pr);
+        sl[s][c] = ld_agent(pr + 1);
+    }
+    __syncthreads();
+    for (int i = tid; i < ncols * vp; i += kSeqThreads) {
+        const int c = i / vp, x = i - c * vp, h = gq * a.R + cols0 + c;
+        const float snk = a.sink[h] * kLog2e;
+        float m = snk;
+        for (int s = 0; s < nsplit; ++s) m = fmaxf(m, sm[s][c]);
+        float acc = 0.0f, l = fast_exp2(snk - m);
+#pragma unroll 8
+        for (int s = 0; s < nsplit; ++s) {
+            const float f = fast_exp2(sm[s][c] - m);
+            acc = fmadd(ld_agent(part + ((size_t)s * kAttnCols + c) * stride + 2 + x), f, acc);
+            l = fmadd(sl[s][c], f, l);
+        }
+        if (x < a.V) reinterpret_cast<T*>(a.out)[(size_t)h * a.V + x] = from_f32<T>(acc / l);
+    }
+}
+
+// ------------------------------------------------------------------------------------------------
+// matrix-vector products of one token
+// ------------------------------------------------------------------------------------------------
+// A wave streams whole weight rows: 1 KB per wave-wide load, eight loads per step, two steps in flight, the first two
+// requested before the prologue.  The input sits in LDS.  Rows go to waves in equal contiguous shares.
+//
+// ROWS: the outputs are the rows of up to `top` chosen matrices and of one that is always there, one after the other.
+// KCAT: every output is the sum of the products with the rows of these matrices (the chosen ones weighted 1 / top); the
+// inputs lie one after the other in LDS.  top == 0: a plain matrix.
+enum : int { kInVector = 0, kInNorm = 1, kInEmbed = 2 };
+struct SeqGemv {
+    int input;
+    const float *x, *y;      // kInNorm: the residual row and the sublayer's output that is still to be added
+    float* x_out;            // ... where the new residual row goes (not x)
+    float* copy;             // nullable: a second copy
+    const float *nw, *nw2;   // norm weights; nw2 (nullable): a second norm follows
+    float alpha, eps;
+    int width;
+    const char* embed;
+    int embed_pitch;
+    const int* state;
+    const char* xin;         // kInVector: the T inputs; chosen ones at multiples of seg_e bytes, the other at top * seg_e
+    int seg_e;
+    // matrices
+    const char *w_e, *w_s;   // chosen (matrix stride e_stride) and always-on rows
+    size_t e_stride;
+    int pitch_e, pitch_s;    // row bytes
+    const int* table;
+    int top, units_e, units_s;   // ROWS: output units per chosen matrix and of the other; KCAT: units_s outputs
+    // outputs
+    const float* bias;
+    float* yf;
+    char* yt;                // T; ROWS: a chosen matrix' outputs at multiples of seg_y bytes
+    int seg_y;
+    float cap;
+    float* best_v;           // kEpiHead: best logit of every workgroup and its row
+    int* best_i;
+};
+constexpr int kGemvChunk = 1024;      // bytes of a row per wave-wide load
+constexpr int kGemvLoads = 8;         // loads per step
+
+template <typename T, int EPI, bool KCAT>
+__global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
+    constexpr int UR = EPI == kEpiGated ? 2 : 1;         // rows per output
+    extern __shared__ __align__(16) char smem[];
+    __shared__ float red[kSeqWaves];
+    __shared__ float bv[kSeqWaves];
+    __shared__ int bi[kSeqWaves];
+    const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63;
+
+    const int nch_e = (p.pitch_e + kGemvChunk - 1) / kGemvChunk, nch_s = (p.pitch_s + kGemvChunk - 1) / kGemvChunk;
+    const int nch_all_e = KCAT ? p.top * nch_e : 0;      // chunks of the chosen part of a row
+    const int nch = KCAT ? nch_all_e + nch_s : nch_s;
+    const int total = KCAT ? p.units_s : p.top * p.units_e + p.units_s;
+    const int nw = gridDim.x * kSeqWaves, gw = blockIdx.x * kSeqWaves + wave;
+    const int u0 = mul_div(total, gw, nw), u1 = mul_div(total, gw + 1, nw);
+    int expert = 0;                                      // lane j: the j-th chosen matrix
+    if (p.top > 0) {
+        const int tok = p.state[kStToken];
+        if (lane < p.top) expert = p.table[(size_t)tok * p.top + lane];
+    }
+    const int steps_row = (nch + kGemvLoads - 1) / kGemvLoads, nsteps = (u1 - u0) * UR * steps_row;
+
+    // base of row `r` of output `u` (ROWS), or of segment `seg`'s row (KCAT)
+    auto rows_base = [&](int u, int r) -> const char* {
+        if (u < p.top * p.units_e) {
+            const int b = u / p.units_e;
+            return p.w_e + (size_t)__builtin_amdgcn_readlane(expert, b) * p.e_stride + (size_t)((u - b * p.units_e) * UR + r) * p.pitch_e;
+        }
+        return p.w_s + (size_t)((u - p.top * p.units_e) * UR + r) * p.pitch_s;
+    };
+    struct Cursor { int u, r, c; };                      // output, row of it, first chunk of the step
+    auto advance = [&](Cursor& k) {
+        k.c += kGemvLoads;
+        if (k.c >= nch) {
+            k.c = 0;
+            if (++k.r == UR) {
+                k.r = 0;
+                ++k.u;
+            }
+        }
+    };
+    auto request = [&](const Cursor& k, u32x4 (&b)[kGemvLoads]) {
+        if constexpr (!KCAT) {
+            const char* row = rows_base(k.u, k.r);
+#pragma unroll
+            for (int i = 0; i < kGemvLoads; ++i)
+                if (k.c + i < nch) b[i] = ld_stream16(row + min((k.c + i) * kGemvChunk + lane * 16, p.pitch_s - 16));
+        } else {
+            int seg = k.c < nch_all_e ? k.c / nch_e : p.top, cc = k.c < nch_all_e ? k.c - seg * nch_e : k.c - nch_all_e;
+#pragma unroll
+            for (int i = 0; i < kGemvLoads; ++i)
+                if (k.c + i < nch) {
+                    const bool e = seg < p.top;
+                    const char* row = e ? p.w_e + (size_t)__builtin_amdgcn_readlane(expert, seg) * p.e_stride + (size_t)k.u * p.pitch_e
+                                        : p.w_s + (size_t)k.u * p.pitch_s;
+                    b[i] = ld_stream16(row + min(cc * kGemvChunk + lane * 16, (e ? p.pitch_e : p.pitch_s) - 16));
+                    if (++cc == (e ? nch_e : nch_s)) {
+                        cc = 0;
+                        ++seg;
+                    }
+                }
+        }
+    };
+    u32x4 b0[kGemvLoads], b1[kGemvLoads];
+    Cursor ask{u0, 0, 0}, use{u0, 0, 0};
+    if (nsteps > 0) { request(ask, b0); advance(ask); }
+    if (nsteps > 1) { request(ask, b1); advance(ask); }
+
+    // ---- prologue: the input into LDS, zeros up to whole chunks
+    T* xs = reinterpret_cast<T*>(smem);
+    if (p.input == kInVector) {
+        for (int i = tid; i < nch * (kGemvChunk / 16); i += kSeqThreads) {
+            const int c = i / (kGemvChunk / 16), o = i - c * (kGemvChunk / 16);
+            const bool e = c < nch_all_e;
+            const int seg = e ? c / nch_e : p.top, off = (e ? c - seg * nch_e : c - nch_all_e) * kGemvChunk + o * 16;
+            u32x4 v = {0, 0, 0, 0};
+            if (off < (e ? p.pitch_e : p.pitch_s)) v = ld16(p.xin + (size_t)seg * p.seg_e + off);
+            reinterpret_cast<u32x4*>(smem)[i] = v;
+        }
+    } else {
+        for (int i = p.width + tid; i < nch * kGemvChunk / (int)sizeof(T); i += kSeqThreads) xs[i] = from_f32<T>(0.0f);
+        const bool keep = blockIdx.x == 0;
+        if (p.input == kInEmbed) {
+            const T* e = reinterpret_cast<const T*>(p.embed + (size_t)p.state[kStToken] * p.embed_pitch);
+            for (int i = tid; i < p.width; i += kSeqThreads) {
+                xs[i] = e[i];
+                if (keep) p.x_out[i] = to_f32(e[i]);
+            }
+        } else {
+            float* ts = reinterpret_cast<float*>(smem + nch * kGemvChunk);
+            float ss = 0.0f;
+            const int w4 = (p.width & 3) ? 0 : p.width / 4;
+            for (int i = tid; i < w4; i += kSeqThreads) {
+                const f32x4 x = reinterpret_cast<const f32x4*>(p.x)[i], y = reinterpret_cast<const f32x4*>(p.y)[i];
+                f32x4 t;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    t[j] = fmadd(p.alpha, x[j], y[j]);
+                    ss = fmadd(t[j], t[j], ss);
+                }
+                reinterpret_cast<f32x4*>(ts)[i] = t;
+            }
+            for (int i = w4 * 4 + tid; i < p.width; i += kSeqThreads) {
+                const float t = fmadd(p.alpha, p.x[i], p.y[i]);
+                ss = fmadd(t, t, ss);
+                ts[i] = t;
+            }
+            float inv = inv_rms(block_sum(ss, red), p.width, p.eps);
+            ss = 0.0f;
+            for (int i = tid; i < p.width; i += kSeqThreads) {
+                const float v = ts[i] * inv * (1.0f + p.nw[i]);
+                ss = fmadd(v, v, ss);
+                if (keep) {
+                    p.x_out[i] = v;
+                    if (p.copy != nullptr) p.copy[i] = v;
+                }
+                if (p.nw2 != nullptr) ts[i] = v; else xs[i] = from_f32<T>(v);
+            }
+            if (p.nw2 != nullptr) {
+                __syncthreads();
+                inv = inv_rms(block_sum(ss, red), p.width, p.eps);
+                for (int i = tid; i < p.width; i += kSeqThreads) xs[i] = from_f32<T>(ts[i] * inv * (1.0f + p.nw2[i]));
+            }
+        }
+    }
+    __syncthreads();
+
+    // ---- the rows
+    float acc = 0.0f, gate = 0.0f, top_v = -INFINITY;
+    int top_i = 0;
+    const float we = p.top > 0 ? 1.0f / (float)p.top : 1.0f;
+    auto consume = [&](const u32x4 (&b)[kGemvLoads]) {
+#pragma unroll
+        for (int i = 0; i < kGemvLoads; ++i)
+            if (use.c + i < nch) {
+                const u32x4 x = *reinterpret_cast<const u32x4*>(smem + (use.c + i) * kGemvChunk + lane * 16);
+                if constexpr (KCAT)
+                    acc = use.c + i < nch_all_e ? fmadd(we, dot16<T>(b[i], x, 0.0f), acc) : dot16<T>(b[i], x, acc);
+                else
+                    acc = dot16<T>(b[i], x, acc);
+            }
+        if (use.c + kGemvLoads >= nch) {
+            const float v = wave_sum(acc);
+            acc = 0.0f;
+            if constexpr (EPI == kEpiF32) {
+                if (lane == 0) p.yf[use.u] = p.bias != nullptr ? v + p.bias[use.u] : v;
+            } else if constexpr (EPI == kEpiHead) {
+                const float z = soft_cap(v, p.cap);
+                if (lane == 0) p.yf[use.u] = z;
+                if (z > top_v) {
+                    top_v = z;
+                    top_i = use.u;
+                }
+            } else if constexpr (EPI == kEpiRelu2) {
+                if (lane == 0) reinterpret_cast<T*>(p.yt)[use.u] = from_f32<T>(relu2(v));
+            } else {
+                if (use.r == 0) {
+                    gate = v;
+                } else if (lane == 0) {
+                    const int b = use.u < p.top * p.units_e ? use.u / p.units_e : p.top;
+                    reinterpret_cast<T*>(p.yt + (size_t)b * p.seg_y)[use.u - b * p.units_e] = from_f32<T>(silu(gate) * v);
+                }
+            }
+        }
+        advance(use);
+    };
+    for (int s = 0; s < nsteps; s += 2) {
+        consume(b0);
+        if (s + 2 < nsteps) { request(ask, b0); advance(ask); }
+        if (s + 1 < nsteps) {
+            consume(b1);
+            if (s + 3 < nsteps) { request(ask, b1); advance(ask); }
+        }
+    }
+    if constexpr (EPI == kEpiHead) {
+        if (lane == 0) {
+            bv[wave] = top_v;
+            bi[wave] = top_i;
+        }
+        __syncthreads();
+        if (tid == 0) {
+            for (int w = 1; w < kSeqWaves; ++w)
+                if (bv[w] > bv[0]) {
+                    bv[0] = bv[w];
+                    bi[0] = bi[w];
+                }
+            p.best_v[blockIdx.x] = bv[0];
+            p.best_i[blockIdx.x] = bi[0];
+        }
+    }
+}
+
+// The largest logit (lowest row on ties) becomes the next step's token.
+__global__ __launch_bounds__(kSeqThreads) void k_seq_pick(const float* best_v, const int* best_i, int n, int* state, int* history, int history_cap) {
+    __shared__ float v[kSeqThreads];
+    __shared__ int r[kSeqThreads];
+    float bv = -INFINITY;
+    int bi = 0x7fffffff;
+    for (int i = threadIdx.x; i < n; i += kSeqThreads)
+        if (best_v[i] > bv || (best_v[i] == bv && best_i[i] < bi)) {
+            bv = best_v[i];
+            bi = best_i[i];
+        }
+    v[threadIdx.x] = bv;
+    r[threadIdx.x] = bi;
+    for (int h = kSeqThreads / 2; h > 0; h /= 2) {
+        __syncthreads();
+        if ((int)threadIdx.x < h) {
+            const int o = threadIdx.x + h;
+            if (v[o] > v[threadIdx.x] || (v[o] == v[threadIdx.x] && r[o] < r[threadIdx.x])) {
+                v[threadIdx.x] = v[o];
+                r[threadIdx.x] = r[o];
+            }
+        }
+    }
+    if (threadIdx.x == 0) {
+        const int tok = r[0] == 0x7fffffff ? 0 : r[0];     // (no finite logit: any row will do, but it must be one)
+        if (state[kStSteps] < history_cap) history[state[kStSteps]] = tok;
+        state[kStToken] = tok;
+        state[kStPos] += 1;
+        state[kStSteps] += 1;
+    }
+}
+
+// angle = position * base^(-2i / dims), evaluated in double and rounded once
+__global__ void k_seq_rope_table(float2* t, const double* freq, int half, int positions) {
+    const size_t n = (size_t)positions * half;
+    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
+        const double a = (double)(i / half) * freq[i % half];
+        t[i] = make_float2((float)cos(a), (float)sin(a));
+    }
+}
+
+// ================================================================================================
+// host side
+// ================================================================================================
+int up_to(int a, int b) { return (a + b - 1) / b * b; }
+int ceil_div(int a, int b) { return (a + b - 1) / b; }
+size_t pitch_of(int K, int esize) { return (size_t)up_to(K * esize, kRowBytes); }
+
+struct LayerPlan {
+    cfpp_seq_layer d;
+    int R, nct, Dp, Vp, krow, vrow, rows, n_qkv, v_role, NT;
+    float2* cs;
+    char *kc, *vc;
+    int ns;
+    int route;               // index among the layers with table experts, -1: none
+};
+
+}  // namespace
+
+struct cfpp_seq {
+    cfpp_seq_desc d;
+    std::vector<LayerPlan> layers;
+    int esize, cus, portion, device, xpitch;
+    std::vector<void*> owned;
+    size_t bytes = 0;
+    bool failed = false;
+    // portion buffers
+    int *tokens, *want;
+    float *x, *qkv, *y, *ys, *v_first;
+    char *xb, *q, *k, *v, *o, *h, *hs, *wb;
+    int ld_qkv;
+    SeqRoute* routes;
+    std::vector<SeqRoute> host_routes;
+    int max_experts = 0;
+    // decode buffers
+    int* state;
+    int *history, *cnt, *best_i;
+    float *dx[2], *dy, *dres, *logits, *part, *best_v;
+    int history_cap, pos = 0, launches = 0, head_grid = 0;
+    hipGraphExec_t graph = nullptr;
+    hipStream_t capture = nullptr;
+
+    template <typename P> P* alloc(size_t n) {
+        void* p = nullptr;
+        const size_t b = (std::max<size_t>(n, 1) * sizeof(P) + 255) / 256 * 256;
+        if (failed || hipMalloc(&p, b) != hipSuccess) {
+            failed = true;
+            return nullptr;
+        }
+        owned.push_back(p);
+        bytes += b;
+        hipLaunchKernelGGL(k_seq_fill_zero, dim3((unsigned)std::min<size_t>((b / 16 + 255) / 256, 4096)), dim3(256), 0, nullptr,
+                           reinterpret_cast<u32x4*>(p), b / 16);
+        return reinterpret_cast<P*>(p);
+    }
+};
+
+namespace {
+
+int last_error() {
+    const hipError_t e = hipGetLastError();
+    return e == hipSuccess ? CFPP_OK : (int)e;
+}
+
+// dynamic LDS beyond the default limit has to be asked for, once per kernel
+template <typename K>
+void allow_lds(K kernel, size_t bytes) {
+    if (bytes > 65536) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes);
+}
+
+// ---- portions ----------------------------------------------------------------------------------
+// max_tiles: upper bound of the expert products' token tiles (their number is known on the device only)
+template <typename T, int EPI>
+void launch_gemm(const SeqGemm& g, int max_tiles, bool big, hipStream_t st) {
+    const int tile = big ? 128 : 64, tw = ceil_div(g.n, tile), tt = g.tile_off != nullptr ? max_tiles : ceil_div(g.m, tile);
+    if (big) hipLaunchKernelGGL((k_seq_gemm<T, 128, 128, EPI>), dim3(tw * tt), dim3(kSeqThreads), 0, st, g);
+    else hipLaunchKernelGGL((k_seq_gemm<T, 64, 64, EPI>), dim3(tw * tt), dim3(kSeqThreads), 0, st, g);
+}
+
+// large tiles where they still give every compute unit one
+template <typename T, int EPI>
+void gemm(const cfpp_seq* s, const SeqGemm& g, hipStream_t st) {
+    launch_gemm<T, EPI>(g, 0, ceil_div(g.n, 128) * ceil_div(g.m, 128) >= s->cus, st);
+}
+
+// tokens per tile of the expert products
+int expert_tile(const LayerPlan& L, int n) { return (long long)n * L.d.top >= 96LL * L.d.experts ? 128 : 64; }
+
+template <typename T, int EPI>
+void expert_gemm(const cfpp_seq* s, const LayerPlan& L, SeqGemm g, int n, hipStream_t st) {
+    const SeqRoute& r = s->host_routes[L.route];
+    const int bt = expert_tile(L, n), slots = n * L.d.top;
+    g.m = slots;
+    g.tile_off = r.tile_off;
+    g.row_off = r.row_off;
+    g.slots = r.slots;
+    g.experts = L.d.experts;
+    launch_gemm<T, EPI>(g, slots / bt + std::min(L.d.experts, slots), bt == 128, st);
+}
+
+template <typename T, int NT>
+void launch_attn(const SeqAttn& a, int G, int cus, hipStream_t st) {
+    const int cols = a.T * a.R;
+    if (ceil_div(cols, 128) * G >= 2 * cus)
+        hipLaunchKernelGGL((k_seq_attn<T, NT, 2>), dim3(ceil_div(cols, 128), G), dim3(kSeqThreads), 0, st, a);
+    else
+        hipLaunchKernelGGL((k_seq_attn<T, NT, 1>), dim3(ceil_div(cols, 64), G), dim3(kSeqThreads), 0, st, a);
+}
+
+template <typename T>
+void postnorm(const cfpp_seq* s, const SeqPostNorm& n, int rows, hipStream_t st) {
+    const size_t lds = (size_t)s->d.width * 4;
+    allow_lds(k_seq_postnorm<T>, lds);
+    hipLaunchKernelGGL(k_seq_postnorm<T>, dim3(rows), dim3(kSeqThreads), lds, st, n);
+}
+
+// One portion: n tokens (device, s->tokens) at positions pos .. pos + n - 1.  want: device places (n_want of them), logits rows.
+template <typename T>
+int run_portion(cfpp_seq* s, int slot, int n, int pos, int n_want, float* logits, float* residuals, size_t residual_stride, hipStream_t st) {
+    const int width = s->d.width, xp = s->xpitch;
+    hipLaunchKernelGGL(k_seq_embed<T>, dim3(n), dim3(kSeqThreads), 0, st, s->tokens, (const char*)s->d.embed, xp, width, s->x, s->xb);
+    if (!s->host_routes.empty()) {
+        // (one tile size for every layer of the launch: the layers share it when they share top and the expert count)
+        for (size_t i = 0; i < s->layers.size(); ++i) {
+            const LayerPlan& L = s->layers[i];
+            if (L.route < 0) continue;
+            size_t j = i + 1, count = 1;
+            for (; j < s->layers.size(); ++j) {
+                const LayerPlan& M = s->layers[j];
+                if (M.route < 0) continue;
+                if (expert_tile(M, n) != expert_tile(L, n)) break;
+                ++count;
+            }
+            const size_t lds = (size_t)s->max_experts * 8;
+            allow_lds(k_seq_route, lds);
+            hipLaunchKernelGGL(k_seq_route, dim3((unsigned)count), dim3(1024), lds, st, s->routes + L.route, s->tokens, n, expert_tile(L, n));
+            i = j - 1;
+        }
+    }
+    for (size_t li = 0; li < s->layers.size(); ++li) {
+        const LayerPlan& L = s->layers[li];
+        const cfpp_seq_layer& d = L.d;
+        float* copy = residuals != nullptr ? residuals + li * residual_stride : nullptr;
+        SeqGemm g{};
+        g.w = (const char*)d.w_qkv;
+        g.a = s->xb;
+        g.n = L.n_qkv;
+        g.m = n;
+        g.kbytes = g.lda = xp;
+        g.bias = d.b_qkv;
+        g.yf = s->qkv;
+        g.ldy = s->ld_qkv;
+        gemm<T, kEpiF32>(s, g, st);
+
+        const int cap = s->portion;
+        SeqQkv f{s->qkv, s->ld_qkv, d.q_norm, d.k_norm, L.cs, s->d.eps, d.v_lambda, d.heads, d.kv_heads, d.dim, L.Dp, d.vdim, L.Vp,
+                 d.rot_dims, pos, cap, L.v_role, s->v_first, s->q, s->k, s->v};
+        hipLaunchKernelGGL(k_seq_qkv_finish<T>, dim3(n), dim3(kSeqThreads), 0, st, f);
+
+        char* kc = L.kc + (size_t)slot * d.kv_heads * L.rows * L.krow;
+        char* vc = L.vc + (size_t)slot * d.kv_heads * L.rows * L.vrow;
+        const int op = (int)pitch_of(d.heads * d.vdim, s->esize);
+        SeqAttn a{s->q, s->k, s->v, kc, vc, s->o, d.sink, n, d.heads, L.R, L.krow / 64, L.krow, L.vrow, d.vdim, L.Vp / 16, pos, d.chunk, cap,
+                  L.rows, op, d.scale * kLog2e};
+        if (L.NT == 64) launch_attn<T, 64>(a, d.kv_heads, s->cus, st);
+        else if (L.NT == 128) launch_attn<T, 128>(a, d.kv_heads, s->cus, st);
+        else launch_attn<T, 256>(a, d.kv_heads, s->cus, st);
+
+        const int last = pos + n - 1, cs0 = d.chunk > 0 ? last / d.chunk * d.chunk : 0, first = std::max(pos, cs0) - pos;
+        SeqAppend ap{s->k, s->v, kc, vc, d.kv_heads, L.krow, L.vrow, cap, L.rows, first, pos + first - cs0};
+        hipLaunchKernelGGL(k_seq_append, dim3(n - first), dim3(kSeqThreads), 0, st, ap);
+
+        g = SeqGemm{};
+        g.w = (const char*)d.w_o;
+        g.a = s->o;
+        g.n = width;
+        g.m = n;
+        g.kbytes = g.lda = op;
+        g.yf = s->y;
+        g.ldy = width;
+        gemm<T, kEpiF32>(s, g, st);
+        SeqPostNorm pn{};
+        pn.x = pn.x_out = s->x;
+        pn.y = s->y;
+        pn.w = d.norm1;
+        pn.alpha = s->d.alpha;
+        pn.eps = s->d.eps;
+        pn.width = width;
+        pn.xb = s->xb;
+        pn.pitch = xp;
+        pn.copy = d.ff_kind == CFPP_SEQ_FF_NONE ? copy : nullptr;
+        postnorm<T>(s, pn, n, st);
+        if (d.ff_kind == CFPP_SEQ_FF_NONE) continue;
+        pn.w = d.norm2;
+        pn.copy = copy;
+
+        if (d.ff_kind == CFPP_SEQ_FF_RELU2) {
+            const int hp = (int)pitch_of(d.ff, s->esize);
+            g = SeqGemm{};
+            g.w = (const char*)d.w_up;
+            g.a = s->xb;
+            g.n = d.ff;
+            g.m = n;
+            g.kbytes = g.lda = xp;
+            g.yt = s->h;
+            g.ldyt = hp;
+            gemm<T, kEpiRelu2>(s, g, st);
+            g = SeqGemm{};
+            g.w = (const char*)d.w_down;
+            g.a = s->h;
+            g.n = width;
+            g.m = n;
+            g.kbytes = g.lda = hp;
+            g.yf = s->y;
+            g.ldy = width;
+            gemm<T, kEpiF32>(s, g, st);
+        } else {
+            const int hp = (int)pitch_of(d.ff, s->esize);
+            g = SeqGemm{};
+            g.w = (const char*)d.w_up;
+            g.w_stride = (size_t)2 * d.ff * xp;
+            g.a = s->xb;
+            g.n = 2 * d.ff;
+            g.kbytes = g.lda = xp;
+            g.yt = s->h;
+            g.ldyt = hp;
+            g.slot_div = d.top;
+            expert_gemm<T, kEpiGated>(s, L, g, n, st);
+            g = SeqGemm{};
+            g.w = (const char*)d.w_down;
+            g.w_stride = (size_t)width * hp;
+            g.a = s->h;
+            g.n = width;
+            g.kbytes = g.lda = hp;
+            g.yf = s->ys;
+            g.ldy = width;
+            g.slot_div = 1;
+            expert_gemm<T, kEpiF32>(s, L, g, n, st);
+            pn.ys = s->ys;
+            pn.top = d.top;
+            pn.slot_weight = 1.0f / (float)d.top;
+            pn.y = nullptr;
+            if (d.shared_ff > 0) {
+                const int sp = (int)pitch_of(d.shared_ff, s->esize);
+                g = SeqGemm{};
+                g.w = (const char*)d.w_shared_up;
+                g.a = s->xb;
+                g.n = 2 * d.shared_ff;
+                g.m = n;
+                g.kbytes = g.lda = xp;
+                g.yt = s->hs;
+                g.ldyt = sp;
+                gemm<T, kEpiGated>(s, g, st);
+                g = SeqGemm{};
+                g.w = (const char*)d.w_shared_down;
+                g.a = s->hs;
+                g.n = width;
+                g.m = n;
+                g.kbytes = g.lda = sp;
+                g.yf = s->y;
+                g.ldy = width;
+                gemm<T, kEpiF32>(s, g, st);
+                pn.y = s->y;
+            }
+        }
+        postnorm<T>(s, pn, n, st);
+    }
+    if (n_want > 0) {
+        SeqPostNorm pn{};
+        pn.x = s->x;
+        pn.w = s->d.final_norm;
+        pn.eps = s->d.eps;
+        pn.width = width;
+        pn.xb = s->wb;
+        pn.pitch = xp;
+        pn.rows = s->want;
+        postnorm<T>(s, pn, n_want, st);
+        SeqGemm g{};
+        g.w = (const char*)s->d.head;
+        g.a = s->wb;
+        g.n = s->d.vocab;
+        g.m = n_want;
+        g.kbytes = g.lda = xp;
+        g.yf = logits;
+        g.ldy = s->d.vocab;
+        g.cap = s->d.softcap;
+        gemm<T, kEpiHead>(s, g, st);
+    }
+    return last_error();
+}
+
+// ---- one token ---------------------------------------------------------------------------------
+template <typename T, int EPI, bool KCAT>
+int gemv(const cfpp_seq* s, const SeqGemv& p, hipStream_t st) {
+    const int nch_e = ceil_div(p.pitch_e, kGemvChunk), nch_s = ceil_div(p.pitch_s, kGemvChunk);
+    const int nch = KCAT ? p.top * nch_e + nch_s : nch_s;
+    const size_t lds = (size_t)nch * kGemvChunk + (p.input == kInNorm ? (size_t)p.width * 4 : 0);
+    const int total = KCAT ? p.units_s : p.top * p.units_e + p.units_s;
+    const int grid = std::max(1, std::min(2 * s->cus, ceil_div(total, kSeqWaves)));
+    allow_lds(k_seq_gemv<T, EPI, KCAT>, lds);
+    hipLaunchKernelGGL((k_seq_gemv<T, EPI, KCAT>), dim3(grid), dim3(kSeqThreads), lds, st, p);
+    return grid;
+}
+
+template <typename T, int NT>
+void launch_attn_decode(const SeqAttnDec& a, hipStream_t st) {
+    hipLaunchKernelGGL((k_seq_attn_decode<T, NT>), dim3(a.ns, a.G * a.nct), dim3(kSeqThreads), 0, st, a);
+}
+
+// Enqueues one step for the device-side state.  pick: also choose the next token.
+template <typename T>
+int run_step(cfpp_seq* s, bool head, bool pick, float* residuals, hipStream_t st) {
+    const int width = s->d.width, xp = s->xpitch;
+    int cur = 0, launches = 0;             // dx[cur]: the residual row before the sum that is still pending
+    const float* pending = nullptr;        // norm weight of that sum
+    float* pending_copy = nullptr;
+    auto input = [&](SeqGemv& p) {
+        p.state = s->state;
+        p.width = width;
+        p.eps = s->d.eps;
+        p.alpha = s->d.alpha;
+        if (pending == nullptr) {
+            p.input = kInEmbed;
+            p.embed = (const char*)s->d.embed;
+            p.embed_pitch = xp;
+            p.x_out = s->dx[cur];
+        } else {
+            p.input = kInNorm;
+            p.x = s->dx[cur];
+            p.y = s->dy;
+            p.x_out = s->dx[cur ^ 1];
+            p.copy = pending_copy;
+            p.nw = pending;
+            cur ^= 1;
+        }
+        pending_copy = nullptr;
+    };
+    for (size_t li = 0; li < s->layers.size(); ++li) {
+        const LayerPlan& L = s->layers[li];
+        const cfpp_seq_layer& d = L.d;
+        float* copy = residuals != nullptr ? residuals + li * width : nullptr;
+        SeqGemv p{};
+        input(p);
+        p.w_s = (const char*)d.w_qkv;
+        p.pitch_s = xp;
+        p.units_s = L.n_qkv;
+        p.bias = d.b_qkv;
+        p.yf = s->qkv;
+        gemv<T, kEpiF32, false>(s, p, st);
+
+        SeqAttnDec a{s->qkv, d.q_norm, d.k_norm, d.sink, L.cs, s->state, L.kc, L.vc, (size_t)d.kv_heads * L.rows * L.krow,
+                     (size_t)d.kv_heads * L.rows * L.vrow, s->v_first, s->o, s->part, s->cnt, s->d.eps, d.v_lambda, d.scale * kLog2e, L.v_role,
+                     d.heads, d.kv_heads, L.R, L.nct, d.dim, d.vdim, d.rot_dims, d.chunk, L.krow, L.vrow, L.krow / 64, L.Vp / 16, L.rows, L.ns};
+        if (L.NT == 64) launch_attn_decode<T, 64>(a, st);
+        else if (L.NT == 128) launch_attn_decode<T, 128>(a, st);
+        else launch_attn_decode<T, 256>(a, st);
+
+        p = SeqGemv{};
+        p.input = kInVector;
+        p.xin = s->o;
+        p.w_s = (const char*)d.w_o;
+        p.pitch_s = (int)pitch_of(d.heads * d.vdim, s->esize);
+        p.units_s = width;
+        p.yf = s->dy;
+        gemv<T, kEpiF32, true>(s, p, st);
+        launches += 3;
+        pending = d.norm1;
+        if (d.ff_kind == CFPP_SEQ_FF_NONE) {
+            pending_copy = copy;
+            continue;
+        }
+        const bool moe = d.ff_kind == CFPP_SEQ_FF_TABLE_EXPERTS;
+        const int hp = (int)pitch_of(d.ff, s->esize), sp = moe ? (int)pitch_of(d.shared_ff, s->esize) : hp;
+        p = SeqGemv{};
+        input(p);
+        p.yt = s->h;
+        p.seg_y = hp;
+        p.pitch_s = xp;
+        if (moe) {
+            p.table = d.table;
+            p.top = d.top;
+            p.w_e = (const char*)d.w_up;
+            p.pitch_e = xp;
+            p.e_stride = (size_t)2 * d.ff * xp;
+            p.units_e = d.ff;
+            p.w_s = (const char*)d.w_shared_up;
+            p.units_s = d.shared_ff;
+            gemv<T, kEpiGated, false>(s, p, st);
+        } else {
+            p.w_s = (const char*)d.w_up;
+            p.units_s = d.ff;
+            gemv<T, kEpiRelu2, false>(s, p, st);
+        }
+        p = SeqGemv{};
+        p.input = kInVector;
+        p.state = s->state;
+        p.xin = s->h;
+        p.seg_e = hp;
+        p.units_s = width;
+        p.yf = s->dy;
+        if (moe) {
+            p.table = d.table;
+            p.top = d.top;
+            p.w_e = (const char*)d.w_down;
+            p.pitch_e = hp;
+            p.e_stride = (size_t)width * hp;
+            p.w_s = (const char*)d.w_shared_down;
+            p.pitch_s = d.shared_ff > 0 ? sp : 0;
+        } else {
+            p.w_s = (const char*)d.w_down;
+            p.pitch_s = hp;
+        }
+        gemv<T, kEpiF32, true>(s, p, st);
+        launches += 2;
+        pending = d.norm2;
+        pending_copy = copy;
+    }
+    if (head || residuals != nullptr) {
+        SeqGemv p{};
+        input(p);
+        p.nw2 = s->d.final_norm;
+        p.w_s = (const char*)s->d.head;
+        p.pitch_s = xp;
+        p.units_s = s->d.vocab;
+        p.yf = s->logits;
+        p.cap = s->d.softcap;
+        p.best_v = s->best_v;
+        p.best_i = s->best_i;
+        s->head_grid = gemv<T, kEpiHead, false>(s, p, st);
+        ++launches;
+        if (pick) {
+            hipLaunchKernelGGL(k_seq_pick, dim3(1), dim3(kSeqThreads), 0, st, s->best_v, s->best_i, s->head_grid, s->state, s->history, s->history_cap);
+            ++launches;
+        }
+    }
+    if (pick) s->launches = launches;
+    return last_error();
+}
+
+int step(cfpp_seq* s, bool head, bool pick, float* residuals, hipStream_t st) {
+    return s->d.dtype == CFPP_SEQ_BF16 ? run_step<bf16_t>(s, head, pick, residuals, st) : run_step<float>(s, head, pick, residuals, st);
+}
+
+int check_layer(const cfpp_seq_desc& D, const cfpp_seq_layer& d, int esize) {
+    if (d.heads < 1 || d.kv_heads < 1 || d.heads % d.kv_heads || d.dim < 1 || d.vdim < 1 || d.dim > 256 || d.vdim > 256 || d.chunk < 0)
+        return CFPP_ERR_DIMS;
+    if (d.rot_dims < 0 || d.rot_dims > d.dim || d.rot_dims % 2) return CFPP_ERR_DIMS;
+    const void* need[] = {d.w_qkv, d.b_qkv, d.q_norm, d.k_norm, d.sink, d.w_o, d.norm1};
+    for (const void* p : need)
+        if (p == nullptr) return CFPP_ERR_NULL;
+    if (d.ff_kind < CFPP_SEQ_FF_NONE || d.ff_kind > CFPP_SEQ_FF_TABLE_EXPERTS) return CFPP_ERR_MODE;
+    size_t lds = std::max(pitch_of(D.width, esize) + 1024 + (size_t)D.width * 4, pitch_of(d.heads * d.vdim, esize) + 1024);
+    if (d.ff_kind != CFPP_SEQ_FF_NONE) {
+        if (d.ff < 1 || d.w_up == nullptr || d.w_down == nullptr || d.norm2 == nullptr) return CFPP_ERR_NULL;
+        const size_t one = pitch_of(d.ff, esize) + 1024;
+        if (d.ff_kind == CFPP_SEQ_FF_TABLE_EXPERTS) {
+            if (d.experts < 1 || d.experts > 8192 || d.top < 1 || d.top > kWave || d.top > d.experts || d.shared_ff < 0) return CFPP_ERR_DIMS;
+            if (d.table == nullptr || (d.shared_ff > 0 && (d.w_shared_up == nullptr || d.w_shared_down == nullptr))) return CFPP_ERR_NULL;
+            lds = std::max(lds, d.top * one + (d.shared_ff > 0 ? pitch_of(d.shared_ff, esize) + 1024 : 0));
+        } else {
+            lds = std::max(lds, one);
+        }
+    }
+    // the input of a matrix-vector product sits in LDS
+    return lds > 150 * 1024 ? CFPP_ERR_DIMS : CFPP_OK;
+}
+
+}  // namespace
+
+extern "C" {
+
+size_t cfpp_seq_row_pitch(int32_t K, int32_t dtype) { return pitch_of(K, dtype == CFPP_SEQ_F32 ? 4 : 2); }
+const char* cfpp_seq_version(void) { return "cfpp_seq 0.1 (gfx950)"; }
+
+int cfpp_seq_create(const cfpp_seq_desc* desc, cfpp_seq** out) {
+    if (desc == nullptr || out == nullptr) return CFPP_ERR_NULL;
+    *out = nullptr;
+    const cfpp_seq_desc& D = *desc;
+    if (D.layers == nullptr || D.embed == nullptr || D.final_norm == nullptr || D.head == nullptr) return CFPP_ERR_NULL;
+    if (D.dtype != CFPP_SEQ_BF16 && D.dtype != CFPP_SEQ_F32) return CFPP_ERR_MODE;
+    if (D.n_layers < 1 || D.width < 1 || D.width > 16384 || D.vocab < 1 || D.vocab > 524288 || D.slots < 1 || D.capacity < 1 || D.max_portion < 1)
+        return CFPP_ERR_DIMS;
+    const int esize = D.dtype == CFPP_SEQ_BF16 ? 2 : 4;
+    int first_mix = -1;
+    for (int i = 0; i < D.n_layers; ++i) {
+        const int rc = check_layer(D, D.layers[i], esize);
+        if (rc) return rc;
+        if (D.layers[i].v_mix) {
+            if (first_mix < 0) first_mix = i;
+            // the mixed values are those of the first such layer, element by element
+            else if (D.layers[i].kv_heads * D.layers[i].vdim != D.layers[first_mix].kv_heads * D.layers[first_mix].vdim) return CFPP_ERR_DIMS;
+        }
+    }
+    cfpp_seq* s = new (std::nothrow) cfpp_seq();
+    if (s == nullptr) return CFPP_ERR_NULL;
+    s->d = D;
+    s->esize = esize;
+    s->xpitch = (int)pitch_of(D.width, esize);
+    s->portion = std::min(D.max_portion, D.capacity);
+    (void)hipGetDevice(&s->device);
+    if (hipDeviceGetAttribute(&s->cus, hipDeviceAttributeMultiprocessorCount, s->device) != hipSuccess || s->cus < 1) s->cus = 256;
+    const size_t P = (size_t)s->portion;
+    size_t n_qkv = 0, o_bytes = 0, h_bytes = 0, hs_bytes = 0, q_el = 0, k_el = 0, v_el = 0, vf = 0, ys = 0, part = 0, items = 0, dec_h = 0;
+    std::map<std::pair<float, int>, float2*> tables;
+    for (int i = 0; i < D.n_layers; ++i) {
+        LayerPlan L{};
+        L.d = D.layers[i];
+        const cfpp_seq_layer& d = L.d;
+        L.R = d.heads / d.kv_heads;
+        L.nct = ceil_div(L.R, kAttnCols);
+        L.Dp = up_to(d.dim, 64 / esize);
+        L.Vp = up_to(d.vdim, 16);
+        L.krow = L.Dp * esize;
+        L.vrow = L.Vp * esize;
+        L.NT = std::max(L.Dp, L.Vp) <= 64 ? 64 : std::max(L.Dp, L.Vp) <= 128 ? 128 : 256;
+        L.rows = d.chunk > 0 ? std::min(d.chunk, D.capacity) : D.capacity;
+        L.n_qkv = d.heads * d.dim + d.kv_heads * (d.dim + d.vdim);
+        L.v_role = !d.v_mix ? 0 : i == first_mix ? 1 : 2;
+        const int kt = esize == 2 ? 32 : (L.NT <= 128 ? 32 : 16);
+        L.ns = std::max(1, std::min({kMaxSeqSplit, ceil_div(s->cus, d.kv_heads * L.nct), ceil_div(L.rows, kt * kSeqWaves)}));
+        L.kc = s->alloc<char>((size_t)D.slots * d.kv_heads * L.rows * L.krow);
+        L.vc = s->alloc<char>((size_t)D.slots * d.kv_heads * L.rows * L.vrow);
+        L.cs = nullptr;
+        if (d.rot_dims > 0) {
+            float2*& t = tables[{d.rot_base, d.rot_dims}];
+            if (t == nullptr) {
+                const int half = d.rot_dims / 2;
+                t = s->alloc<float2>((size_t)D.capacity * half);
+                std::vector<double> freq(half);
+                for (int j = 0; j < half; ++j) freq[j] = pow((double)d.rot_base, -2.0 * j / d.rot_dims);
+                double* df = s->alloc<double>(half);
+                if (!s->failed) {
+                    (void)hipDeviceSynchronize();        // the zero fill of the table comes before its copy
+                    if (hipMemcpy(df, freq.data(), half * sizeof(double), hipMemcpyHostToDevice) != hipSuccess) s->failed = true;
+                    hipLaunchKernelGGL(k_seq_rope_table, dim3(1024), dim3(256), 0, nullptr, t, df, half, D.capacity);
+                }
+            }
+            L.cs = t;
+        }
+        n_qkv = std::max(n_qkv, (size_t)L.n_qkv);
+        o_bytes = std::max(o_bytes, pitch_of(d.heads * d.vdim, esize));
+        q_el = std::max(q_el, (size_t)d.heads * L.krow);
+        k_el = std::max(k_el, (size_t)d.kv_heads * L.krow);
+        v_el = std::max(v_el, (size_t)d.kv_heads * L.vrow);
+        if (d.v_mix) vf = std::max(vf, (size_t)d.kv_heads * d.vdim);
+        items = std::max(items, (size_t)d.kv_heads * L.nct);
+        part = std::max(part, (size_t)d.kv_heads * L.nct * L.ns * kAttnCols * (L.Vp + 2));
+        L.route = -1;
+        if (d.ff_kind == CFPP_SEQ_FF_RELU2) {
+            h_bytes = std::max(h_bytes, pitch_of(d.ff, esize));
+        } else if (d.ff_kind == CFPP_SEQ_FF_TABLE_EXPERTS) {
+            h_bytes = std::max(h_bytes, d.top * pitch_of(d.ff, esize));
+            hs_bytes = std::max(hs_bytes, pitch_of(d.shared_ff, esize));
+            ys = std::max(ys, (size_t)d.top * D.width);
+            dec_h = std::max(dec_h, d.top * pitch_of(d.ff, esize) + pitch_of(d.shared_ff, esize));
+            SeqRoute r{d.table, s->alloc<int>(d.experts + 1), s->alloc<int>(d.experts + 1), s->alloc<int>(P * d.top), d.experts, d.top};
+            L.route = (int)s->host_routes.size();
+            s->host_routes.push_back(r);
+            s->max_experts = std::max(s->max_experts, d.experts);
+        }
+        s->layers.push_back(L);
+    }
+    s->ld_qkv = up_to((int)n_qkv, 4);
+    s->tokens = s->alloc<int>(2 * P);
+    s->want = s->tokens != nullptr ? s->tokens + P : nullptr;
+    s->x = s->alloc<float>(P * D.width);
+    s->y = s->alloc<float>(P * D.width);
+    s->ys = s->alloc<float>(P * ys);
+    s->qkv = s->alloc<float>(P * s->ld_qkv);
+    s->v_first = s->alloc<float>(P * vf);
+    s->xb = s->alloc<char>(P * s->xpitch);
+    s->wb = s->alloc<char>(P * s->xpitch);
+    s->q = s->alloc<char>(P * q_el);
+    s->k = s->alloc<char>(P * k_el);
+    s->v = s->alloc<char>(P * v_el);
+    s->o = s->alloc<char>(P * o_bytes);
+    s->h = s->alloc<char>(std::max(P * h_bytes, dec_h));
+    s->hs = s->alloc<char>(P * hs_bytes);
+    s->routes = s->alloc<SeqRoute>(s->host_routes.size());
+    s->state = s->alloc<int>(4);
+    s->history_cap = D.capacity;
+    s->history = s->alloc<int>(s->history_cap);
+    s->cnt = s->alloc<int>(items * kHeadCntStride);
+    s->part = s->alloc<float>(part);
+    s->dx[0] = s->alloc<float>(D.width);
+    s->dx[1] = s->alloc<float>(D.width);
+    s->dy = s->alloc<float>(D.width);
+    s->dres = s->alloc<float>((size_t)D.n_layers * D.width);
+    s->logits = s->alloc<float>(D.vocab);
+    s->best_v = s->alloc<float>(2 * s->cus);
+    s->best_i = s->alloc<int>(2 * s->cus);
+    if (!s->failed && hipDeviceSynchronize() != hipSuccess) s->failed = true;
+    if (!s->failed && !s->host_routes.empty() &&
+        hipMemcpy(s->routes, s->host_routes.data(), s->host_routes.size() * sizeof(SeqRoute), hipMemcpyHostToDevice) != hipSuccess)
+        s->failed = true;
+    if (s->failed) {
+        const int e = (int)hipGetLastError();
+        cfpp_seq_destroy(s);
+        return e > 0 ? e : (int)hipErrorOutOfMemory;
+    }
+    *out = s;
+    return CFPP_OK;
+}
+
+int cfpp_seq_destroy(cfpp_seq* s) {
+    if (s == nullptr) return CFPP_OK;
+    (void)hipDeviceSynchronize();
+    if (s->graph != nullptr) (void)hipGraphExecDestroy(s->graph);
+    if (s->capture != nullptr) (void)hipStreamDestroy(s->capture);
+    for (void* p : s->owned) (void)hipFree(p);
+    delete s;
+    return CFPP_OK;
+}
+
+size_t cfpp_seq_bytes(const cfpp_seq* s) { return s != nullptr ? s->bytes : 0; }
+
+int cfpp_seq_forward(cfpp_seq* s, int32_t slot, const int32_t* tokens, int32_t n, int32_t pos, const int32_t* want, int32_t n_want,
+                     float* logits, float* residuals, void* stream) {
+    if (s == nullptr || tokens == nullptr || n_want < 0 || (n_want > 0 && (want == nullptr || logits == nullptr))) return CFPP_ERR_NULL;
+    if (slot < 0 || slot >= s->d.slots) return CFPP_ERR_CONTEXT;
+    if (n < 1 || pos < 0 || n > s->d.capacity - pos) return CFPP_ERR_SEQ;
+    for (int i = 0; i < n; ++i)
+        if (tokens[i] < 0 || tokens[i] >= s->d.vocab) return CFPP_ERR_DIMS;
+    for (int i = 0; i < n_want; ++i)
+        if (want[i] < 0 || want[i] >= n || (i > 0 && want[i] <= want[i - 1])) return CFPP_ERR_DIMS;
+    hipStream_t st = (hipStream_t)stream;
+    const int width = s->d.width, V = s->d.vocab;
+    int w = 0;
+    for (int off = 0; off < n;) {
+        const int T = std::min(n - off, s->portion);
+        int w1 = w;
+        while (w1 < n_want && want[w1] < off + T) ++w1;
+        const int nw = w1 - w;
+        int rc;
+        if (T == 1) {
+            hipLaunchKernelGGL(k_seq_set_state, dim3(1), dim3(64), 0, st, s->state, slot, tokens[off], pos + off, -1);
+            // (a single token's residual rows are written one layer after the other; with other tokens they lie n rows apart)
+            float* res = residuals == nullptr || n == 1 ? residuals : s->dres;
+            rc = step(s, nw > 0, false, res, st);
+            if (res != residuals)
+                for (int l = 0; l < s->d.n_layers; ++l)
+                    (void)hipMemcpyAsync(residuals + ((size_t)l * n + off) * width, res + (size_t)l * width, (size_t)width * 4, hipMemcpyDeviceToDevice, st);
+            if (rc == CFPP_OK && nw > 0) {
+                const hipError_t e = hipMemcpyAsync(logits + (size_t)w * V, s->logits, (size_t)V * 4, hipMemcpyDeviceToDevice, st);
+                if (e != hipSuccess) rc = (int)e;
+            }
+        } else {
+            std::vector<int> places(nw);
+            for (int i = 0; i < nw; ++i) places[i] = want[w + i] - off;
+            hipError_t e = hipMemcpyAsync(s->tokens, tokens + off, (size_t)T * 4, hipMemcpyHostToDevice, st);
+            if (e == hipSuccess && nw > 0) e = hipMemcpyAsync(s->want, places.data(), (size_t)nw * 4, hipMemcpyHostToDevice, st);
+            if (e == hipSuccess) e = hipStreamSynchronize(st);           // the host arrays are the caller's and this frame's
+            if (e != hipSuccess) return (int)e;
+            float* res = residuals != nullptr ? residuals + (size_t)off * width : nullptr;
+            float* lg = nw > 0 ? logits + (size_t)w * V : nullptr;
+            const size_t rs = (size_t)n * width;
+            rc = s->d.dtype == CFPP_SEQ_BF16 ? run_portion<bf16_t>(s, slot, T, pos + off, nw, lg, res, rs, st)
+                                             : run_portion<float>(s, slot, T, pos + off, nw, lg, res, rs, st);
+        }
+        if (rc != CFPP_OK) return rc;
+        off += T;
+        w = w1;
+    }
+    return CFPP_OK;
+}
+
+int cfpp_seq_set_state(cfpp_seq* s, int32_t slot, int32_t token, int32_t pos, void* stream) {
+    if (s == nullptr) return CFPP_ERR_NULL;
+    if (slot < 0 || slot >= s->d.slots) return CFPP_ERR_CONTEXT;
+    if (token < 0 || token >= s->d.vocab) return CFPP_ERR_DIMS;
+    if (pos < 0 || pos >= s->d.capacity) return CFPP_ERR_SEQ;
+    hipLaunchKernelGGL(k_seq_set_state, dim3(1), dim3(64), 0, (hipStream_t)stream, s->state, slot, token, pos, 0);
+    s->pos = pos;
+    return last_error();
+}
+
+int cfpp_seq_steps(cfpp_seq* s, int32_t n, void* stream) {
+    if (s == nullptr) return CFPP_ERR_NULL;
+    if (n < 0 || n > s->d.capacity - s->pos) return CFPP_ERR_SEQ;
+    for (int i = 0; i < n; ++i) {
+        const int rc = step(s, true, true, nullptr, (hipStream_t)stream);
+        if (rc != CFPP_OK) return rc;
+        ++s->pos;
+    }
+    return CFPP_OK;
+}
+
+int cfpp_seq_graph_steps(cfpp_seq* s, int32_t n, void* stream) {
+    if (s == nullptr) return CFPP_ERR_NULL;
+    if (n < 0 || n > s->d.capacity - s->pos) return CFPP_ERR_SEQ;
+    if (s->graph == nullptr) {
+        hipGraph_t g = nullptr;
+        hipError_t e = s->capture != nullptr ? hipSuccess : hipStreamCreateWithFlags(&s->capture, hipStreamNonBlocking);
+        if (e == hipSuccess) e = hipStreamBeginCapture(s->capture, hipStreamCaptureModeThreadLocal);
+        if (e != hipSuccess) return (int)e;
+        const int rc = step(s, true, true, nullptr, s->capture);
+        e = hipStreamEndCapture(s->capture, &g);
+        if (rc != CFPP_OK || e != hipSuccess) {
+            if (g != nullptr) (void)hipGraphDestroy(g);
+            return rc != CFPP_OK ? rc : (int)e;
+        }
+        e = hipGraphInstantiate(&s->graph, g, nullptr, nullptr, 0);
+        (void)hipGraphDestroy(g);
+        if (e != hipSuccess) {
+            s->graph = nullptr;
+            return (int)e;
+        }
+    }
+    for (int i = 0; i < n; ++i) {
+        const hipError_t e = hipGraphLaunch(s->graph, (hipStream_t)stream);
+        if (e != hipSuccess) return (int)e;
+        ++s->pos;
+    }
+    return CFPP_OK;
+}
+
+int cfpp_seq_launches_per_step(const cfpp_seq* s) { return s != nullptr ? s->launches : 0; }
+
+int cfpp_seq_buffers(cfpp_seq* s, float** logits, int32_t** state, int32_t** history, int32_t* history_capacity) {
+    if (s == nullptr) return CFPP_ERR_NULL;
+    if (logits) *logits = s->logits;
+    if (state) *state = s->state;
+    if (history) *history = s->history;
+    if (history_capacity) *history_capacity = s->history_cap;
+    return CFPP_OK;
+}
+
+}  // extern "C"

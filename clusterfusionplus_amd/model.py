@@ -222,3 +222,62 @@ class NeoxDecoder:
         self.check()
         n = int(self.state[2].item())
         return self._stack.history()[:n].tolist()
+
+
+# ---- serving: the decoder behind the engine's interface -----------------------------------------------------------
+
+_hf_names = {"ln_w": "input_layernorm.weight", "ln_b": "input_layernorm.bias",
+             "w_qkv": "attention.query_key_value.weight", "b_qkv": "attention.query_key_value.bias",
+             "w_o": "attention.dense.weight", "b_o": "attention.dense.bias",
+             "post_ln_w": "post_attention_layernorm.weight", "post_ln_b": "post_attention_layernorm.bias",
+             "w_up": "mlp.dense_h_to_4h.weight", "b_up": "mlp.dense_h_to_4h.bias",
+             "w_down": "mlp.dense_4h_to_h.weight", "b_down": "mlp.dense_4h_to_h.bias"}
+
+
+class NeoxSequence:
+    """A GPT-NeoX model as the engine drives it (`forward`, `decode`), over NeoxDecoder.  One slot.  The library has decode
+    kernels only for this family, so a prompt is run token by token through the captured step."""
+
+    architecture = "GPTNeoXForCausalLM"
+    slots = 1
+
+    def __init__(self, decoder: NeoxDecoder, capacity: int):
+        self.decoder, self.vocab, self.capacity = decoder, decoder.cfg.vocab, int(capacity)
+
+    def forward(self, slot: int, tokens: Sequence[int], pos: int, want: Sequence[int] = ()) -> torch.Tensor:
+        wanted, rows = set(want), {}
+        for i, t in enumerate(tokens):
+            self.decoder.set_state(t, pos + i)
+            self.decoder.graph_steps(1)
+            if i in wanted:
+                rows[i] = self.decoder.logits.clone()
+        self.decoder.check()
+        return torch.stack([rows[i] for i in want]) if rows else self.decoder.logits.new_empty((0, self.vocab))
+
+    def decode(self, slot: int, token: int, pos: int, n: int) -> List[int]:
+        self.decoder.set_state(token, pos)
+        self.decoder.graph_steps(n)
+        return self.decoder.generated()
+
+
+def load_neox(path: str, dtype=torch.float16, capacity: int = 4096, slots: int = 1, max_portion: int = 0, device="cuda") -> NeoxSequence:
+    """A HuggingFace GPT-NeoX checkpoint folder (config.json, safetensors) with empty caches of `capacity` rows."""
+    from types import SimpleNamespace
+
+    from .weights import read_config, read_weights
+    if dtype != torch.float16:
+        raise ValueError("the GPT-NeoX kernels run in float16")
+    if slots != 1:
+        raise ValueError("the GPT-NeoX decoder holds one sequence")
+    cfg = config_from_hf(SimpleNamespace(**read_config(path)))
+    w = read_weights(path)
+
+    def get(name):
+        if name not in w:
+            raise ValueError(f"checkpoint: tensor {name} is missing")
+        return w[name].to(device=device, dtype=dtype).contiguous()
+    layers = [{k: get(f"gpt_neox.layers.{i}.{n}") for k, n in _hf_names.items()} for i in range(cfg.n_layers)]
+    caches = [[torch.zeros((capacity, cfg.hidden), dtype=dtype, device=device) for _ in range(cfg.n_layers)] for _ in range(2)]
+    dec = NeoxDecoder(cfg, layers, get("gpt_neox.embed_in.weight"), get("gpt_neox.final_layer_norm.weight"),
+                      get("gpt_neox.final_layer_norm.bias"), get("embed_out.weight"), *caches)
+    return NeoxSequence(dec, capacity)
