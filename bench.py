@@ -513,13 +513,137 @@ def other_workloads(pkg, dev, args):
     return out
 
 
+NIBOTAR_SIZES = {
+    # the layer of Pythia-6.9B: the same matrices (q, k, v, o of 4096 x 4096, up and down of 16384 x 4096), heads and vocabulary
+    "dense_6b9": dict(width=4096, layers=32, heads=32, kv_heads=32, dim=128, vdim=128, chunk=8192, ff=16384, vocab=50432),
+    # grouped heads, a wide feed-forward (the layer sizes of today's 8B models)
+    "dense_8b": dict(width=4096, layers=32, heads=32, kv_heads=8, dim=128, vdim=128, chunk=8192, ff=14336, vocab=128256),
+    # many small experts and a shared one
+    "experts_16b": dict(width=2048, layers=28, heads=16, kv_heads=4, dim=128, vdim=128, chunk=8192, ff=1408, experts=64, top=6, shared=2816,
+                        vocab=102400),
+}
+
+
+def nibotar_model(z, capacity, max_portion, dev, n_layers=None):
+    """A Nibotar model of the given sizes with random bf16 weights on the device, and the bytes and flops it is priced by."""
+    import torch
+    from clusterfusionplus_amd import seq_model as S
+    torch.manual_seed(0)
+    W, H, G, D, Dv, F, V = (z[k] for k in ("width", "heads", "kv_heads", "dim", "vdim", "ff", "vocab"))
+    E, top, sh = z.get("experts", 0), z.get("top", 0), z.get("shared", 0)
+
+    def rn(*shape, std=0.02):
+        return torch.empty(shape, dtype=torch.bfloat16, device=dev).normal_(0, std)
+
+    def vec(n, mean=0.0):
+        return torch.empty(n, dtype=torch.float32, device=dev).normal_(mean, 0.02)
+    layers = []
+    for i in range(n_layers or z["layers"]):
+        ff = dict(ff_kind=S.FF_RELU2, ff=F, w_up=rn(F, W), w_down=rn(W, F))
+        if E and i:                      # (the first layer is a dense one of the active experts' size)
+            ff = dict(ff_kind=S.FF_TABLE_EXPERTS, ff=F, experts=E, top=top, shared_ff=sh, w_up=rn(E, 2 * F, W), w_down=rn(E, W, F),
+                      w_shared_up=rn(2 * sh, W), w_shared_down=rn(W, sh),
+                      table=torch.rand(V, E, device=dev).argsort(1)[:, :top].int().contiguous())
+        elif E:
+            ff = dict(ff_kind=S.FF_RELU2, ff=top * F + sh, w_up=rn(top * F + sh, W), w_down=rn(W, top * F + sh))
+        layers.append(S.SeqLayer(heads=H, kv_heads=G, dim=D, vdim=Dv, scale=D ** -0.5, chunk=z["chunk"], rot_dims=D, v_mix=True, v_lambda=0.5,
+                                 w_qkv=rn(H * D + G * D + G * Dv, W), b_qkv=vec(H * D + G * D + G * Dv), q_norm=vec(H * D, 1.0),
+                                 k_norm=vec(G * D, 1.0), sink=vec(H), w_o=rn(W, H * Dv), norm1=vec(W), norm2=vec(W), **ff))
+    w = S.SeqWeights(dtype=torch.bfloat16, width=W, vocab=V, eps=1e-6, alpha=2.0, softcap=15.0, layers=layers, embed=rn(V, W, std=1.0),
+                     final_norm=vec(W), head=rn(V, W), architecture="Nibotar")
+    m = S.SeqModel(w, capacity=capacity, max_portion=max_portion)
+    per_layer = []
+    for l in layers:
+        n = W * (H * D + G * D + G * Dv) + W * H * Dv
+        n += 3 * W * (top * F + sh) if l.ff_kind == S.FF_TABLE_EXPERTS else 2 * W * l.ff
+        per_layer.append(n)
+    kv_row = G * (D + Dv) * 2
+    return m, dict(layer_params=per_layer, params=sum(per_layer), head=W * V, kv_row=kv_row, attn_flops=2 * H * (D + Dv), n_layers=len(layers))
+
+
+def bench_nibotar(args):
+    """Nibotar at a few sizes (random weights): decode (TPOT of captured-graph replays at --ctx cached tokens) and prefill
+    (whole prompts of several lengths), each against its roofline: decode against the HBM bytes of the weights the token
+    uses and of the visible cache rows, prefill against the dense bf16 matrix peak.  Beside the size that has a Pythia-6.9B
+    layer's matrices: the Pythia-6.9B stack itself, in fused and in split mode."""
+    import torch
+    import clusterfusionplus_amd as pkg
+    dev, peak_tf = "cuda:0", 2500.0
+    sizes = args.size.split(",") if args.size else list(NIBOTAR_SIZES)
+    out = []
+    for name in sizes:
+        z = NIBOTAR_SIZES[name]
+        prompts = [512, 2048, 8192]
+        m, b = nibotar_model(z, max(args.ctx + args.warmup + args.steps + 64, max(prompts)), max(prompts), dev, args.layers or None)
+        g = torch.Generator().manual_seed(1)
+        toks = torch.randint(0, z["vocab"], (max(prompts + [args.ctx]),), generator=g).tolist()
+        e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+        pre = []
+        for n in prompts:
+            for _ in range(2):
+                m.forward(0, toks[:n], 0, [n - 1])
+            torch.cuda.synchronize()
+            reps = max(1, min(5, 16384 // n))
+            e0.record()
+            for _ in range(reps):
+                m.forward(0, toks[:n], 0, [n - 1])
+            e1.record()
+            torch.cuda.synchronize()
+            ms = e0.elapsed_time(e1) / reps
+            flops = 2 * n * b["params"] + 2 * b["head"] + b["n_layers"] * b["attn_flops"] * n * (n + 1) / 2
+            pre.append({"tokens": n, "ms": round(ms, 3), "tokens_per_s": round(n / ms * 1e3), "tflops": round(flops / ms / 1e9, 1),
+                        "frac_of_matrix_peak": round(flops / ms / 1e9 / peak_tf, 4)})
+            log(f"[nibotar {name}] prefill {n}: {ms:.3f} ms, {pre[-1]['tokens_per_s']} tokens/s, {pre[-1]['tflops']} TFLOP/s")
+        m.forward(0, toks[:args.ctx], 0)
+        m.set_state(11, args.ctx)
+        m.graph_steps(args.warmup)
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        m.graph_steps(args.steps)
+        torch.cuda.synchronize()
+        tpot = (time.perf_counter() - t0) * 1e3 / args.steps
+        rows = min(args.ctx + args.warmup + args.steps // 2, z["chunk"])
+        nbytes = 2 * (b["params"] + b["head"]) + b["n_layers"] * rows * b["kv_row"]
+        gbps = nbytes / (tpot * 1e-3) / 1e9
+        log(f"[nibotar {name}] decode at {args.ctx}: {tpot:.4f} ms/token, {gbps / HBM_PEAK_GBPS * 100:.1f} % of the HBM roofline")
+        out.append({"size": name, **z, "layers": b["n_layers"], "prefill": pre, "decode": {
+            "context": args.ctx, "tpot_ms": round(tpot, 4), "tokens_per_s": round(1e3 / tpot, 1), "launches": m.launches_per_step, "bytes": nbytes,
+            "hbm_gbps": round(gbps, 1), "frac_of_peak": round(gbps / HBM_PEAK_GBPS, 4)}})
+        del m
+        torch.cuda.empty_cache()
+    closest = []
+    if args.also and "dense_6b9" in sizes:
+        from dataclasses import replace
+        cfg = replace(pkg.PYTHIA_6B9, n_layers=args.layers or pkg.PYTHIA_6B9.n_layers)
+        for mode in ("fused", "split"):
+            dec = build_model(cfg, args.ctx + args.warmup + args.steps + 40, args.ctx, dev, mode)
+            stream = torch.cuda.Stream()
+            with torch.cuda.stream(stream):
+                tpot = time_tokens(dec, stream, args.ctx, args.steps, args.warmup)
+            dec.check()
+            sb = step_bytes(cfg, args.ctx + args.warmup + args.steps // 2)
+            closest.append({"model": f"pythia_6b9 ({cfg.n_layers} layers)", "mode": mode, "context": args.ctx, "tpot_ms": round(tpot, 4), "bytes": sb,
+                            "frac_of_peak": round(sb / (tpot * 1e-3) / 1e9 / HBM_PEAK_GBPS, 4)})
+            log(f"[closest] pythia_6b9 {mode}: {tpot:.4f} ms/token, {closest[-1]['frac_of_peak'] * 100:.1f} %")
+            del dec
+            torch.cuda.empty_cache()
+    d = out[0]["decode"]
+    print(json.dumps({"metric": "tpot_ms", "value": d["tpot_ms"], "unit": "ms/token", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+                      "ms_per_step": d["tpot_ms"], "higher_is_better": False, "scaling": "weak", "vs_baseline": None, "dtype": "bf16",
+                      "data": "synthetic", "config": {"workload": f"nibotar {out[0]['size']}, batch-1 greedy decode, hipGraph replay", "context": args.ctx},
+                      "roofline": {"bound": "hbm", "achieved": d["hbm_gbps"], "peak": HBM_PEAK_GBPS, "unit": "GB/s", "frac": d["frac_of_peak"]},
+                      "sizes": out, "closest": closest, "cpu_baseline": None}), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=64)
     ap.add_argument("--warmup", type=int, default=8)
-    ap.add_argument("--model", default="pythia_6b9", choices=["pythia_6b9", "pythia_2b8", "llama2_7b_layer", "llama2_7b_batch"])
+    ap.add_argument("--model", default="pythia_6b9", choices=["pythia_6b9", "pythia_2b8", "llama2_7b_layer", "llama2_7b_batch", "nibotar"])
     ap.add_argument("--batch", type=int, default=16, help="sequences per call (llama2_7b_batch only)")
+    ap.add_argument("--size", default="", help=f"sizes to measure, with commas between them (nibotar only): {', '.join(NIBOTAR_SIZES)}")
+    ap.add_argument("--layers", type=int, default=0, help="layers instead of the model's own number (nibotar only)")
     ap.add_argument("--ctx", type=int, default=2048, help="KV-cache rows already filled when the timed region starts")
     ap.add_argument("--mode", default="fused", choices=["fused", "split", "fused_layers"],
                     help="fused: one launch per layer, or one for all layers where the device holds the whole grid; "
@@ -543,6 +667,8 @@ def main():
         if args.ctx == 2048:
             args.ctx = 4096          # the context this workload is quoted at
         return bench_llama_layer(args)
+    if args.model == "nibotar":
+        return bench_nibotar(args)
     if args.model == "llama2_7b_batch":
         if args.ctx == 2048:
             args.ctx = 1024

@@ -93,7 +93,8 @@ size_t cfpp_seq_bytes(const cfpp_seq* s);
 /* Runs the `n` tokens at positions pos .. pos + n - 1 of the sequence in `slot`, whose positions 0 .. pos - 1 earlier calls
  * have run, and writes the logits at the places want[0 .. n_want) among them to `logits` (device fp32 [n_want, vocab]).
  * `tokens` and `want` are host arrays; want must be increasing.  One token runs through the decode kernels, more through
- * the prefill kernels.  pos == 0 starts the slot anew.  `residuals` (may be NULL): device fp32 [n_layers, n, width],
+ * the prefill kernels.  pos == 0 starts the slot anew; a sequence cannot be wound back, since a chunk's cache rows are taken
+ * over by the next chunk.  `residuals` (may be NULL): device fp32 [n_layers, n, width],
  * receives the residual stream after every layer. */
 int cfpp_seq_forward(cfpp_seq* s, int32_t slot, const int32_t* tokens, int32_t n, int32_t pos, const int32_t* want,
                      int32_t n_want, float* logits, float* residuals, void* stream);
