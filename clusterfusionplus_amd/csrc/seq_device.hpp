@@ -23,6 +23,8 @@ constexpr int kRowBytes = 128;                    // matrix rows are padded to t
 constexpr int kSeqThreads = 256;                  // threads of every sequence kernel: four waves
 constexpr int kSeqWaves = kSeqThreads / kWave;
 constexpr float kLog2e = 1.4426950408889634f;
+constexpr float kMasked = -3.0e38f;               // score of a key that is not seen: its exp2 is zero next to any other, and next
+                                                  // to kNegBig, where a column has seen nothing yet
 
 template <typename T> struct Unit;                // elements in 16 bytes
 template <> struct Unit<bf16_t> { static constexpr int n = 8; };
@@ -64,6 +66,13 @@ template <> __device__ __forceinline__ float dot16<float>(u32x4 w, u32x4 x, floa
 __device__ __forceinline__ void copy_to_lds16(const void* g, void* lds) {
     __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(uintptr_t)g,
                                      (__attribute__((address_space(3))) void*)(uintptr_t)lds, 16, 0, 0);
+}
+
+// A barrier of the workgroup behind its LDS accesses only: __syncthreads() would also wait for loads in flight.
+__device__ __forceinline__ void lds_barrier() {
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+    __builtin_amdgcn_s_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
 }
 
 // sum over the workgroup, in every thread, in a fixed order; `red` holds kSeqWaves floats (2 of them: two sums at a time)
@@ -108,42 +117,42 @@ template <typename T, int KT> struct VtTile {
 };
 
 // 4 keys x one unit of value columns per step, transposed on the way into LDS.  `rowp(key)` is the address of a key's
-// value row, for keys 0 .. KT - 1 of the tile; threads tid of nthreads share the tile.
-template <typename T, int KT, int NT, int NTHREADS, typename RowPtr>
-__device__ __forceinline__ void stage_vt(char* vt, int vunits, int tid, RowPtr rowp) {
-    constexpr int UE = Unit<T>::n, KG = KT / 4;
-    constexpr int ITERS = (KG * (NT / UE) + NTHREADS - 1) / NTHREADS;
-    constexpr int BATCH = ITERS < 2 ? ITERS : 2;
+// value row, for keys 0 .. KT - 1 of the tile; threads tid of NTHREADS share the tile.  Steps [FIRST, FIRST + N) of
+// VtSteps: request puts them into registers, store writes them out.
+template <typename T, int KT, int NT, int NTHREADS> struct VtSteps {
+    static constexpr int n = (KT / 4 * (NT / Unit<T>::n) + NTHREADS - 1) / NTHREADS;
+};
+template <typename T, int KT, int NTHREADS, int FIRST, int N, typename RowPtr>
+__device__ __forceinline__ void vt_request(u32x4 (&r)[N][4], int vunits, int tid, RowPtr rowp) {
+    constexpr int KG = KT / 4;
 #pragma unroll
-    for (int it0 = 0; it0 < ITERS; it0 += BATCH) {
-        u32x4 r[BATCH][4];
+    for (int b = 0; b < N; ++b) {
+        const int idx = tid + (FIRST + b) * NTHREADS, kg = idx % KG, vc = min(idx / KG, vunits - 1);
 #pragma unroll
-        for (int b = 0; b < BATCH; ++b) {
-            const int idx = tid + (it0 + b) * NTHREADS, kg = idx % KG, vc = idx / KG;
-            if (vc < vunits) {
+        for (int j = 0; j < 4; ++j) r[b][j] = ld16(rowp(kg * 4 + j) + (size_t)vc * 16);
+    }
+}
+template <typename T, int KT, int NTHREADS, int FIRST, int N>
+__device__ __forceinline__ void vt_store(const u32x4 (&r)[N][4], char* vt, int vunits, int tid) {
+    constexpr int KG = KT / 4;
 #pragma unroll
-                for (int j = 0; j < 4; ++j) r[b][j] = ld16(rowp(kg * 4 + j) + (size_t)vc * 16);
-            }
-        }
+    for (int b = 0; b < N; ++b) {
+        const int idx = tid + (FIRST + b) * NTHREADS, kg = idx % KG, vc = idx / KG;
+        if (vc < vunits) {
+            if constexpr (sizeof(T) == 2) {
 #pragma unroll
-        for (int b = 0; b < BATCH; ++b) {
-            const int idx = tid + (it0 + b) * NTHREADS, kg = idx % KG, vc = idx / KG;
-            if (vc < vunits) {
-                if constexpr (sizeof(T) == 2) {
+                for (int e = 0; e < 8; ++e) {
+                    // halfword e & 1 of word e >> 1 of the four keys
+                    constexpr uint32_t kLow = 0x05040100u, kHigh = 0x07060302u;
+                    const uint32_t sel = (e & 1) ? kHigh : kLow;
+                    u32x2 v = {__builtin_amdgcn_perm(r[b][1][e >> 1], r[b][0][e >> 1], sel), __builtin_amdgcn_perm(r[b][3][e >> 1], r[b][2][e >> 1], sel)};
+                    *reinterpret_cast<u32x2*>(vt + (vc * 8 + e) * VtTile<T, KT>::pitch + kg * 8) = v;
+                }
+            } else {
 #pragma unroll
-                    for (int e = 0; e < 8; ++e) {
-                        const int sh = (e & 1) * 16;
-                        const uint32_t a = (r[b][0][e >> 1] >> sh) & 0xffffu, bb = (r[b][1][e >> 1] >> sh) & 0xffffu;
-                        const uint32_t c = (r[b][2][e >> 1] >> sh) & 0xffffu, d = (r[b][3][e >> 1] >> sh) & 0xffffu;
-                        u32x2 v = {a | (bb << 16), c | (d << 16)};
-                        *reinterpret_cast<u32x2*>(vt + (vc * 8 + e) * VtTile<T, KT>::pitch + kg * 8) = v;
-                    }
-                } else {
-#pragma unroll
-                    for (int e = 0; e < 4; ++e) {
-                        u32x4 v = {r[b][0][e], r[b][1][e], r[b][2][e], r[b][3][e]};
-                        *reinterpret_cast<u32x4*>(vt + (vc * 4 + e) * VtTile<T, KT>::pitch + kg * 16) = v;
-                    }
+                for (int e = 0; e < 4; ++e) {
+                    u32x4 v = {r[b][0][e], r[b][1][e], r[b][2][e], r[b][3][e]};
+                    *reinterpret_cast<u32x4*>(vt + (vc * 4 + e) * VtTile<T, KT>::pitch + kg * 16) = v;
                 }
             }
         }
@@ -163,7 +172,7 @@ __device__ __forceinline__ void attn_reset(AttnState<NT>& st) {
     for (int i = 0; i < NT / 16; ++i) st.acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
 }
 
-// s[kt][r]: scores (already times scale * log2 e; kNegBig and below: not seen) of keys 16 kt + 4 g + r.  Turns them into
+// s[kt][r]: scores (already times scale * log2 e; kMasked: not seen) of keys 16 kt + 4 g + r.  Turns them into
 // weights relative to the new maximum and rescales the state.
 template <int NT, int NKT>
 __device__ __forceinline__ void attn_softmax(AttnState<NT>& st, f32x4 (&s)[NKT], int vtiles) {
@@ -181,8 +190,7 @@ __device__ __forceinline__ void attn_softmax(AttnState<NT>& st, f32x4 (&s)[NKT],
     for (int kt = 0; kt < NKT; ++kt)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            // (a key that is not seen has weight zero also where the column has seen nothing yet and m is kNegBig itself)
-            const float p = s[kt][r] > kNegBig ? fast_exp2(s[kt][r] - m) : 0.0f;
+            const float p = fast_exp2(s[kt][r] - m);
             s[kt][r] = p;
             sum += p;
         }

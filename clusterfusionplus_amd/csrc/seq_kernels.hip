@@ -33,6 +33,7 @@ namespace {
 enum : int { kStToken = 0, kStPos = 1, kStSteps = 2, kStSlot = 3 };
 constexpr int kAttnCols = 16;          // query columns of a decode item (one MFMA column tile)
 constexpr int kMaxSeqSplit = 64;       // KV splits of a decode step
+constexpr int kAttnWgs = 2;            // ... sized for this many workgroups per compute unit
 
 // ------------------------------------------------------------------------------------------------
 // small kernels
@@ -381,23 +382,23 @@ struct SeqAttn {
 };
 template <int UN> __device__ __forceinline__ int swz_key(int row) { return UN == 8 ? (row >> 1) & 7 : row & 15; }
 
+// (the next tile's keys go straight to the other LDS buffer and its values into registers while this one is worked on)
 template <typename T, int NT, int CT>
-__global__ __launch_bounds__(kSeqThreads) void k_seq_attn(SeqAttn a) {
+__global__ __launch_bounds__(kSeqThreads, (NT <= 128 ? 2 : 1)) void k_seq_attn(SeqAttn a) {
     constexpr int KT = sizeof(T) == 2 ? 64 : 32;
     constexpr int NB = NT * (int)sizeof(T), UN = NB / 16, RPC = 1024 / NB;   // bytes and units of a key row in LDS, rows per copy
-    __shared__ __align__(1024) char ks[KT * NB];
+    constexpr int VS = VtSteps<T, KT, NT, kSeqThreads>::n;
+    __shared__ __align__(1024) char ks[2][KT * NB];
     __shared__ __align__(16) char vt[NT * VtTile<T, KT>::pitch];
     const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, col = lane & 15, g = lane >> 4;
     const int gq = blockIdx.y, ncols = a.T * a.R, c0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * 64 * CT;
 
-    int tok[CT], head[CT], pq[CT], first[CT];
-    bool mine[CT];
+    int pq[CT], first[CT], tok[CT], head[CT];
     u32x4 qf[CT][NB / 64];
     AttnState<NT> st[CT];
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
-        const int c = c0 + (wave * CT + ct) * 16 + col, cc = min(c, ncols - 1);
-        mine[ct] = c < ncols;
+        const int cc = min(c0 + (wave * CT + ct) * 16 + col, ncols - 1);
         tok[ct] = cc / a.R;
         head[ct] = gq * a.R + (cc - tok[ct] * a.R);
         pq[ct] = a.pos0 + tok[ct];
@@ -408,28 +409,44 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_attn(SeqAttn a) {
             if (s < a.dsteps) qf[ct][s] = ld16(qr + s * 64);
         attn_reset(st[ct]);
     }
+    // keys the workgroup needs, and those every column of this wave sees / any column sees
     const int t_first = c0 / a.R, t_last = min(a.T - 1, (c0 + 64 * CT - 1) / a.R);
     const int k_first = chunk_start(a.pos0 + t_first, a.chunk), k_end = a.pos0 + t_last + 1;
+    const int w_first = min(c0 + wave * CT * 16, ncols - 1) / a.R, w_last = min(c0 + (wave + 1) * CT * 16 - 1, ncols - 1) / a.R;
+    const int all_lo = chunk_start(a.pos0 + w_last, a.chunk), all_hi = a.pos0 + w_first;
+    const int any_lo = chunk_start(a.pos0 + w_first, a.chunk), any_hi = a.pos0 + w_last;
     const int dunits = a.krow / 16, vunits = a.vrow / 16;
 
-    for (int seg = 0; seg < 2; ++seg) {
-        const int lo = seg == 0 ? k_first : max(k_first, a.pos0), hi = seg == 0 ? min(k_end, a.pos0) : k_end;
-        if (lo >= hi) continue;
-        // row of position p: base + p * row bytes
-        const int base_pos = seg == 0 ? chunk_start(a.pos0, a.chunk) : a.pos0;
-        const size_t row0 = (size_t)gq * (seg == 0 ? a.rows : a.cap);
-        const char* kb = (seg == 0 ? a.kc : a.k) + row0 * a.krow;
-        const char* vb = (seg == 0 ? a.vc : a.v) + row0 * a.vrow;
-        for (int k0 = lo; k0 < hi; k0 += KT) {
-            __syncthreads();
-            for (int i = wave; i < KT / RPC; i += kSeqWaves) {
-                const int r = i * RPC + lane / UN;
-                int u = (lane % UN) ^ swz_key<UN>(r);
-                if (u >= dunits) u = 0;
-                copy_to_lds16(kb + (size_t)(min(k0 + r, hi - 1) - base_pos) * a.krow + u * 16, ks + i * 1024);
-            }
-            stage_vt<T, KT, NT, kSeqThreads>(vt, vunits, tid, [&](int key) { return vb + (size_t)(min(k0 + key, hi - 1) - base_pos) * a.vrow; });
-            __syncthreads();
+    // tiles: [k_first, pos0) in the cache, then [pos0, k_end) in the portion
+    struct Tile { int k0, hi; const char *k, *v; };      // first key, end of its part, row of position 0
+    auto tile_at = [&](int k0) {
+        const bool cached = k0 < a.pos0;
+        const size_t row0 = (size_t)gq * (cached ? a.rows : a.cap) - (cached ? chunk_start(a.pos0, a.chunk) : a.pos0);
+        return Tile{k0, cached ? min(k_end, a.pos0) : k_end, (cached ? a.kc : a.k) + (ptrdiff_t)row0 * a.krow, (cached ? a.vc : a.v) + (ptrdiff_t)row0 * a.vrow};
+    };
+    u32x4 vr[VS][4];
+    auto fetch = [&](const Tile& t, int buf) {
+        for (int i = wave; i < KT / RPC; i += kSeqWaves) {
+            const int r = i * RPC + lane / UN;
+            int u = (lane % UN) ^ swz_key<UN>(r);
+            if (u >= dunits) u = 0;
+            copy_to_lds16(t.k + (ptrdiff_t)min(t.k0 + r, t.hi - 1) * a.krow + u * 16, ks[buf] + i * 1024);
+        }
+        vt_request<T, KT, kSeqThreads, 0, VS>(vr, vunits, tid, [&](int key) { return t.v + (ptrdiff_t)min(t.k0 + key, t.hi - 1) * a.vrow; });
+    };
+    Tile t = tile_at(k_first);
+    fetch(t, 0);
+    for (int buf = 0;; buf ^= 1) {
+        __syncthreads();                                 // the tile's keys are there; nobody reads the last tile's values any more
+        vt_store<T, KT, kSeqThreads, 0, VS>(vr, vt, vunits, tid);
+        const int next = min(t.k0 + KT, t.hi);
+        Tile tn = t;
+        if (next < k_end) {
+            tn = tile_at(next);
+            fetch(tn, buf ^ 1);
+        }
+        lds_barrier();                                   // (waits for the stores to LDS, not for the next tile)
+        if (t.k0 <= any_hi && next > any_lo) {
             f32x4 s[CT][KT / 16];
 #pragma unroll
             for (int kt = 0; kt < KT / 16; ++kt) {
@@ -439,29 +456,37 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_attn(SeqAttn a) {
 #pragma unroll
                 for (int d = 0; d < NB / 64; ++d)
                     if (d < a.dsteps) {
-                        const u32x4 kf = *reinterpret_cast<const u32x4*>(ks + r * NB + ((d * 4 + g) ^ swz_key<UN>(r)) * 16);
+                        const u32x4 kf = *reinterpret_cast<const u32x4*>(ks[buf] + r * NB + ((d * 4 + g) ^ swz_key<UN>(r)) * 16);
 #pragma unroll
                         for (int ct = 0; ct < CT; ++ct) s[ct][kt] = mma16<T>(kf, qf[ct][d], s[ct][kt]);
                     }
             }
+            const bool full = t.k0 + KT <= t.hi && t.k0 >= all_lo && t.k0 + KT - 1 <= all_hi;
 #pragma unroll
             for (int ct = 0; ct < CT; ++ct) {
 #pragma unroll
                 for (int kt = 0; kt < KT / 16; ++kt)
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) {
-                        const int key = k0 + kt * 16 + g * 4 + r;
-                        const bool see = key < hi && key <= pq[ct] && key >= first[ct];
-                        s[ct][kt][r] = see ? s[ct][kt][r] * a.scale_log2 : kNegBig;
-                    }
+                    for (int r = 0; r < 4; ++r) s[ct][kt][r] *= a.scale_log2;
+                if (!full) {
+#pragma unroll
+                    for (int kt = 0; kt < KT / 16; ++kt)
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) {
+                            const int key = t.k0 + kt * 16 + g * 4 + r;
+                            if (key >= t.hi || key > pq[ct] || key < first[ct]) s[ct][kt][r] = kMasked;
+                        }
+                }
                 attn_softmax<NT, KT / 16>(st[ct], s[ct], a.vtiles);
                 attn_pv<T, NT, KT>(st[ct], s[ct], vt, a.vtiles, lane);
             }
         }
+        if (next >= k_end) break;
+        t = tn;
     }
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
-        if (!mine[ct]) continue;
+        if (c0 + (wave * CT + ct) * 16 + col >= ncols) continue;
         const float snk = a.sink[head[ct]] * kLog2e, m = fmaxf(st[ct].m, snk), c = fast_exp2(st[ct].m - m);
         const float f = c / (st[ct].l * c + fast_exp2(snk - m));
         T* o = reinterpret_cast<T*>(a.out + (size_t)tok[ct] * a.ldo) + head[ct] * a.V;
@@ -499,10 +524,27 @@ struct SeqAttnDec {
 };
 template <typename T, int NT> struct DecTile { static constexpr int kt = sizeof(T) == 2 ? 32 : (NT <= 128 ? 32 : 16); };
 
+// sum of squares of n floats over the workgroup's threads (each thread's share)
+__device__ __forceinline__ float share_sq(const float* __restrict__ v, int n, int tid) {
+    float s = 0.0f;
+    int i0 = 0;
+    if (((uintptr_t)v & 15) == 0) {
+        i0 = n & ~3;
+        for (int i = tid; i < n / 4; i += kSeqThreads) {
+            const f32x4 x = reinterpret_cast<const f32x4*>(v)[i];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) s = fmadd(x[j], x[j], s);
+        }
+    }
+    for (int i = i0 + tid; i < n; i += kSeqThreads) s = fmadd(v[i], v[i], s);
+    return s;
+}
+
 template <typename T, int NT>
 __global__ __launch_bounds__(kSeqThreads) void k_seq_attn_decode(SeqAttnDec a) {
     constexpr int KT = DecTile<T, NT>::kt, NB = NT * (int)sizeof(T);
     constexpr int VB = NT * VtTile<T, KT>::pitch, MB = kAttnCols * NT * 4;
+    constexpr int VS = VtSteps<T, KT, NT, kWave>::n, KF = KT / 16;
     __shared__ __align__(16) char buf[kSeqWaves * (VB > MB ? VB : MB)];
     __shared__ __align__(16) char qs[kAttnCols * NB];
     __shared__ float red[kSeqWaves], wm[kSeqWaves][kAttnCols], wl[kSeqWaves][kAttnCols];
@@ -511,21 +553,36 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_attn_decode(SeqAttnDec a) {
     const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, col = lane & 15, g = lane >> 4;
     const int item = blockIdx.y, gq = item / a.nct, cols0 = (item - gq * a.nct) * kAttnCols, ncols = min(kAttnCols, a.R - cols0);
     const int pos = a.state[kStPos], slot = a.state[kStSlot];
-    const int k_first = chunk_start(pos, a.chunk), n = pos - k_first + 1;
-    const int tile = KT * kSeqWaves;
-    const int per = ((n + a.ns - 1) / a.ns + tile - 1) / tile * tile, nsplit = (n + per - 1) / per;
-    const int sp = blockIdx.x;
+    // tiles of KT keys are shared evenly among the splits
+    const int k_first = chunk_start(pos, a.chunk), ntiles = (pos - k_first + KT) / KT, nsplit = min(a.ns, ntiles), sp = blockIdx.x;
     if (sp >= nsplit) return;
-    const int k0 = k_first + sp * per, k1 = min(k0 + per, pos + 1);
+    const int k0 = k_first + mul_div(ntiles, sp, nsplit) * KT, k1 = min(k_first + mul_div(ntiles, sp + 1, nsplit) * KT, pos + 1);
     char* kc = a.kc + slot * a.k_slot + (size_t)gq * a.rows * a.krow;
     char* vc = a.vc + slot * a.v_slot + (size_t)gq * a.rows * a.vrow;
-    const float2* cs = a.cs + (size_t)pos * (a.rot / 2);
+    const int vunits = a.vrow / 16;
 
-    const int nq = a.H * a.D, nk = a.G * a.D, nv = a.G * a.V;
+    u32x4 kf[KF][NB / 64], vr[VS][4];
+    auto fetch = [&](int kb) {
+#pragma unroll
+        for (int kt = 0; kt < KF; ++kt) {
+            const char* kr = kc + (size_t)(min(kb + kt * 16 + col, k1 - 1) - k_first) * a.krow + g * 16;
+#pragma unroll
+            for (int d = 0; d < NB / 64; ++d)
+                if (d < a.dsteps) kf[kt][d] = ld16(kr + d * 64);
+        }
+        vt_request<T, KT, kWave, 0, VS>(vr, vunits, lane, [&](int key) { return vc + (size_t)(min(kb + key, k1 - 1) - k_first) * a.vrow; });
+    };
+    const int nq = a.H * a.D, nk = a.G * a.D;
     const float *q = a.qkv, *k = q + nq, *v = k + nk;
+    const bool newest = k1 == pos + 1;                   // this split makes and appends the newest position's rows
+    const float sq = share_sq(q, nq, tid), sk = newest ? share_sq(k, nk, tid) : 0.0f;
+    // the wave's first tile, unless the newest position, which is not in the cache yet, is in it
+    int kb = k0 + wave * KT;
+    const bool early = kb + KT <= pos && kb < k1;
+    if (early) fetch(kb);
+
+    const float2* cs = a.cs + (size_t)pos * (a.rot / 2);
     {
-        float sq = 0.0f;
-        for (int i = tid; i < nq; i += kSeqThreads) sq = fmadd(q[i], q[i], sq);
         const float iq = inv_rms(block_sum(sq, red), nq, a.eps);
         const int dp = a.krow / (int)sizeof(T);
         for (int i = tid; i < kAttnCols * dp; i += kSeqThreads) {
@@ -535,9 +592,7 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_attn_decode(SeqAttnDec a) {
             reinterpret_cast<T*>(qs)[c * NT + d] = from_f32<T>(x);
         }
     }
-    if (k1 == pos + 1) {
-        float sk = 0.0f;
-        for (int i = tid; i < nk; i += kSeqThreads) sk = fmadd(k[i], k[i], sk);
+    if (newest) {
         const float ik = inv_rms(block_sum(sk, red), nk, a.eps);
         T* ko = reinterpret_cast<T*>(kc + (size_t)(pos - k_first) * a.krow);
         T* vo = reinterpret_cast<T*>(vc + (size_t)(pos - k_first) * a.vrow);
@@ -559,26 +614,23 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_attn_decode(SeqAttnDec a) {
     AttnState<NT> st;
     attn_reset(st);
     char* vt = buf + wave * VB;
-    for (int kb = k0 + wave * KT; kb < k1; kb += tile) {
-        f32x4 s[KT / 16];
+    if (!early && kb < k1) fetch(kb);
+    for (; kb < k1; kb += KT * kSeqWaves) {
+        f32x4 s[KF];
 #pragma unroll
-        for (int kt = 0; kt < KT / 16; ++kt) {
-            const char* kr = kc + (size_t)(min(kb + kt * 16 + col, k1 - 1) - k_first) * a.krow + g * 16;
-            u32x4 kf[NB / 64];
-#pragma unroll
-            for (int d = 0; d < NB / 64; ++d)
-                if (d < a.dsteps) kf[d] = ld16(kr + d * 64);
+        for (int kt = 0; kt < KF; ++kt) {
             s[kt] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int d = 0; d < NB / 64; ++d)
-                if (d < a.dsteps) s[kt] = mma16<T>(kf[d], qf[d], s[kt]);
+                if (d < a.dsteps) s[kt] = mma16<T>(kf[kt][d], qf[d], s[kt]);
         }
-        stage_vt<T, KT, NT, kWave>(vt, a.vrow / 16, lane, [&](int key) { return vc + (size_t)(min(kb + key, k1 - 1) - k_first) * a.vrow; });
+        vt_store<T, KT, kWave, 0, VS>(vr, vt, vunits, lane);
+        if (kb + KT * kSeqWaves < k1) fetch(kb + KT * kSeqWaves);
 #pragma unroll
-        for (int kt = 0; kt < KT / 16; ++kt)
+        for (int kt = 0; kt < KF; ++kt)
 #pragma unroll
-            for (int r = 0; r < 4; ++r) s[kt][r] = kb + kt * 16 + g * 4 + r < k1 ? s[kt][r] * a.scale_log2 : kNegBig;
-        attn_softmax<NT, KT / 16>(st, s, a.vtiles);
+            for (int r = 0; r < 4; ++r) s[kt][r] = kb + kt * 16 + g * 4 + r < k1 ? s[kt][r] * a.scale_log2 : kMasked;
+        attn_softmax<NT, KF>(st, s, a.vtiles);
         __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
         __builtin_amdgcn_wave_barrier();                 // the tile in LDS belongs to this wave alone
         attn_pv<T, NT, KT>(st, s, vt, a.vtiles, lane);
@@ -657,8 +709,8 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_attn_decode(SeqAttnDec a) {
 // ------------------------------------------------------------------------------------------------
 // matrix-vector products of one token
 // ------------------------------------------------------------------------------------------------
-// A wave streams whole weight rows: 1 KB per wave-wide load, eight loads per step, two steps in flight, the first two
-// requested before the prologue.  The input sits in LDS.  Rows go to waves in equal contiguous shares.
+// A wave streams its weight rows as one sequence of 1 KB chunks (one wave-wide load each), eight per step, two steps in
+// flight, the first two requested before the prologue.  The input sits in LDS.  Rows go to waves in equal contiguous shares.
 //
 // ROWS: the outputs are the rows of up to `top` chosen matrices and of one that is always there, one after the other.
 // KCAT: every output is the sum of the products with the rows of these matrices (the chosen ones weighted 1 / top); the
@@ -691,9 +743,11 @@ struct SeqGemv {
     float cap;
     float* best_v;           // kEpiHead: best logit of every workgroup and its row
     int* best_i;
+    int park, park_n;        // LDS: offset of the finished outputs, outputs per wave at most
 };
 constexpr int kGemvChunk = 1024;      // bytes of a row per wave-wide load
 constexpr int kGemvLoads = 8;         // loads per step
+constexpr int kGemvWgs = 2;           // workgroups per compute unit
 
 template <typename T, int EPI, bool KCAT>
 __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
@@ -706,74 +760,110 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
 
     const int nch_e = (p.pitch_e + kGemvChunk - 1) / kGemvChunk, nch_s = (p.pitch_s + kGemvChunk - 1) / kGemvChunk;
     const int nch_all_e = KCAT ? p.top * nch_e : 0;      // chunks of the chosen part of a row
-    const int nch = KCAT ? nch_all_e + nch_s : nch_s;
-    const int total = KCAT ? p.units_s : p.top * p.units_e + p.units_s;
+    const int nch = KCAT ? nch_all_e + nch_s : nch_s;    // chunks of a whole row
+    const int outputs = KCAT ? p.units_s : p.top * p.units_e + p.units_s;
     const int nw = gridDim.x * kSeqWaves, gw = blockIdx.x * kSeqWaves + wave;
-    const int u0 = mul_div(total, gw, nw), u1 = mul_div(total, gw + 1, nw);
+    const int u0 = mul_div(outputs, gw, nw), u1 = mul_div(outputs, gw + 1, nw);
     int expert = 0;                                      // lane j: the j-th chosen matrix
     if (p.top > 0) {
         const int tok = p.state[kStToken];
         if (lane < p.top) expert = p.table[(size_t)tok * p.top + lane];
     }
-    const int steps_row = (nch + kGemvLoads - 1) / kGemvLoads, nsteps = (u1 - u0) * UR * steps_row;
 
-    // base of row `r` of output `u` (ROWS), or of segment `seg`'s row (KCAT)
-    auto rows_base = [&](int u, int r) -> const char* {
-        if (u < p.top * p.units_e) {
-            const int b = u / p.units_e;
-            return p.w_e + (size_t)__builtin_amdgcn_readlane(expert, b) * p.e_stride + (size_t)((u - b * p.units_e) * UR + r) * p.pitch_e;
-        }
-        return p.w_s + (size_t)((u - p.top * p.units_e) * UR + r) * p.pitch_s;
+    // ---- the wave's chunks, one after the other.  Requests are never conditional (past the end they repeat the last
+    // chunk), so that the number of loads in flight is known and a step waits for its own loads only.
+    const char* ask_row = nullptr;                       // row (KCAT: of the segment) being requested
+    int ask_lim = 0, ask_n = 0, ask_c = 0;               // offset of its last 16 bytes, its chunks, the next chunk
+    int ask_u = 0, ask_seg = 0;                          // output; matrix: the seg-th chosen one, or p.top: the one that is always there
+    int ask_j = 0, ask_r = 0;                            // ROWS: output inside the matrix, row of the output
+    auto open_row = [&]() __attribute__((always_inline)) {
+        // (both alternatives are read before one is chosen: a choice between two members' addresses would keep the
+        // parameters in memory)
+        const bool e = ask_seg < p.top;
+        const char *we = p.w_e + (size_t)__builtin_amdgcn_readlane(expert, e ? ask_seg : 0) * p.e_stride, *ws = p.w_s;
+        const int pe = p.pitch_e, ps = p.pitch_s, pitch = e ? pe : ps;
+        ask_row = (e ? we : ws) + (size_t)(KCAT ? ask_u : ask_j * UR + ask_r) * pitch;
+        ask_lim = pitch - 16;
+        ask_n = e ? nch_e : nch_s;
     };
-    struct Cursor { int u, r, c; };                      // output, row of it, first chunk of the step
-    auto advance = [&](Cursor& k) {
-        k.c += kGemvLoads;
-        if (k.c >= nch) {
-            k.c = 0;
-            if (++k.r == UR) {
-                k.r = 0;
-                ++k.u;
+    auto next_chunk = [&]() __attribute__((always_inline)) {
+        if (ask_c + 1 < ask_n) {
+            ask_c = ask_c + 1;
+            return;
+        }
+        const bool same = KCAT ? ask_seg + 1 < p.top + (nch_s > 0 ? 1 : 0) : ask_r + 1 < UR;    // the output has another row
+        if (!same && ask_u + 1 >= u1) return;
+        ask_c = 0;
+        const int du = same ? 0 : 1;
+        ask_u = ask_u + du;
+        if constexpr (KCAT) {
+            ask_seg = same ? ask_seg + 1 : 0;
+        } else {
+            ask_r = same ? ask_r + 1 : 0;
+            const int j = ask_j + du;
+            const bool hop = j == p.units_e && ask_seg < p.top;
+            ask_j = hop ? 0 : j;
+            ask_seg = ask_seg + (hop ? 1 : 0);
+        }
+        open_row();
+    };
+    auto request = [&](u32x4 (&b)[kGemvLoads]) __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < kGemvLoads; ++i) {
+            b[i] = ld_stream16(ask_row + min(ask_c * kGemvChunk + lane * 16, ask_lim));
+            next_chunk();
+        }
+    };
+    ask_u = min(u0, outputs - 1);                        // (a wave without rows asks for a valid one and uses nothing)
+    ask_r = ask_c = 0;
+    ask_seg = KCAT || p.top == 0 ? 0 : min(ask_u / p.units_e, p.top);
+    ask_j = ask_u - ask_seg * p.units_e;
+    open_row();
+
+    // ---- prologue: the input into LDS, zeros up to whole chunks.  What it reads is requested before the first weights
+    // (loads return in order), in registers up to kPre units per thread, the rest afterwards.
+    constexpr int kPre = KCAT ? 8 : 4;
+    T* xs = reinterpret_cast<T*>(smem);
+    const int nunits = nch * (kGemvChunk / 16);          // units of the input in LDS
+    auto input_unit = [&](int i) -> u32x4 {
+        const int c = i / (kGemvChunk / 16), o = i - c * (kGemvChunk / 16);
+        const bool e = c < nch_all_e;
+        const int seg = e ? c / nch_e : p.top, off = (e ? c - seg * nch_e : c - nch_all_e) * kGemvChunk + o * 16;
+        const int pe = p.pitch_e, ps = p.pitch_s;
+        u32x4 v = {0, 0, 0, 0};
+        if (off < (e ? pe : ps)) v = ld16(p.xin + (size_t)seg * p.seg_e + off);
+        return v;
+    };
+    const f32x4 *x4 = reinterpret_cast<const f32x4*>(p.x), *y4 = reinterpret_cast<const f32x4*>(p.y), *n4 = reinterpret_cast<const f32x4*>(p.nw);
+    const int w4 = (p.width & 3) ? 0 : p.width / 4;
+    u32x4 pv[kPre];
+    f32x4 px[kPre], py[kPre], pn[kPre];
+    if constexpr (KCAT) {
+#pragma unroll
+        for (int i = 0; i < kPre; ++i)
+            if (tid + i * kSeqThreads < nunits) pv[i] = input_unit(tid + i * kSeqThreads);
+    } else if (p.input == kInNorm) {
+#pragma unroll
+        for (int i = 0; i < kPre; ++i) {
+            const int k = min(tid + i * kSeqThreads, w4 - 1);
+            if (w4 > 0) {
+                px[i] = x4[k];
+                py[i] = y4[k];
+                pn[i] = n4[k];
             }
         }
-    };
-    auto request = [&](const Cursor& k, u32x4 (&b)[kGemvLoads]) {
-        if constexpr (!KCAT) {
-            const char* row = rows_base(k.u, k.r);
-#pragma unroll
-            for (int i = 0; i < kGemvLoads; ++i)
-                if (k.c + i < nch) b[i] = ld_stream16(row + min((k.c + i) * kGemvChunk + lane * 16, p.pitch_s - 16));
-        } else {
-            int seg = k.c < nch_all_e ? k.c / nch_e : p.top, cc = k.c < nch_all_e ? k.c - seg * nch_e : k.c - nch_all_e;
-#pragma unroll
-            for (int i = 0; i < kGemvLoads; ++i)
-                if (k.c + i < nch) {
-                    const bool e = seg < p.top;
-                    const char* row = e ? p.w_e + (size_t)__builtin_amdgcn_readlane(expert, seg) * p.e_stride + (size_t)k.u * p.pitch_e
-                                        : p.w_s + (size_t)k.u * p.pitch_s;
-                    b[i] = ld_stream16(row + min(cc * kGemvChunk + lane * 16, (e ? p.pitch_e : p.pitch_s) - 16));
-                    if (++cc == (e ? nch_e : nch_s)) {
-                        cc = 0;
-                        ++seg;
-                    }
-                }
-        }
-    };
+    }
+    __builtin_amdgcn_sched_barrier(0);
     u32x4 b0[kGemvLoads], b1[kGemvLoads];
-    Cursor ask{u0, 0, 0}, use{u0, 0, 0};
-    if (nsteps > 0) { request(ask, b0); advance(ask); }
-    if (nsteps > 1) { request(ask, b1); advance(ask); }
+    request(b0);
+    request(b1);
+    __builtin_amdgcn_sched_barrier(0);
 
-    // ---- prologue: the input into LDS, zeros up to whole chunks
-    T* xs = reinterpret_cast<T*>(smem);
-    if (p.input == kInVector) {
-        for (int i = tid; i < nch * (kGemvChunk / 16); i += kSeqThreads) {
-            const int c = i / (kGemvChunk / 16), o = i - c * (kGemvChunk / 16);
-            const bool e = c < nch_all_e;
-            const int seg = e ? c / nch_e : p.top, off = (e ? c - seg * nch_e : c - nch_all_e) * kGemvChunk + o * 16;
-            u32x4 v = {0, 0, 0, 0};
-            if (off < (e ? p.pitch_e : p.pitch_s)) v = ld16(p.xin + (size_t)seg * p.seg_e + off);
-            reinterpret_cast<u32x4*>(smem)[i] = v;
-        }
+    if constexpr (KCAT) {
+#pragma unroll
+        for (int i = 0; i < kPre; ++i)
+            if (tid + i * kSeqThreads < nunits) reinterpret_cast<u32x4*>(smem)[tid + i * kSeqThreads] = pv[i];
+        for (int i = tid + kPre * kSeqThreads; i < nunits; i += kSeqThreads) reinterpret_cast<u32x4*>(smem)[i] = input_unit(i);
     } else {
         for (int i = p.width + tid; i < nch * kGemvChunk / (int)sizeof(T); i += kSeqThreads) xs[i] = from_f32<T>(0.0f);
         const bool keep = blockIdx.x == 0;
@@ -786,9 +876,8 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
         } else {
             float* ts = reinterpret_cast<float*>(smem + nch * kGemvChunk);
             float ss = 0.0f;
-            const int w4 = (p.width & 3) ? 0 : p.width / 4;
-            for (int i = tid; i < w4; i += kSeqThreads) {
-                const f32x4 x = reinterpret_cast<const f32x4*>(p.x)[i], y = reinterpret_cast<const f32x4*>(p.y)[i];
+            // (every thread reads back only what it has written)
+            auto sum4 = [&](int i, f32x4 x, f32x4 y) {
                 f32x4 t;
 #pragma unroll
                 for (int j = 0; j < 4; ++j) {
@@ -796,7 +885,11 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
                     ss = fmadd(t[j], t[j], ss);
                 }
                 reinterpret_cast<f32x4*>(ts)[i] = t;
-            }
+            };
+#pragma unroll
+            for (int i = 0; i < kPre; ++i)
+                if (tid + i * kSeqThreads < w4) sum4(tid + i * kSeqThreads, px[i], py[i]);
+            for (int i = tid + kPre * kSeqThreads; i < w4; i += kSeqThreads) sum4(i, x4[i], y4[i]);
             for (int i = w4 * 4 + tid; i < p.width; i += kSeqThreads) {
                 const float t = fmadd(p.alpha, p.x[i], p.y[i]);
                 ss = fmadd(t, t, ss);
@@ -804,15 +897,24 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
             }
             float inv = inv_rms(block_sum(ss, red), p.width, p.eps);
             ss = 0.0f;
-            for (int i = tid; i < p.width; i += kSeqThreads) {
-                const float v = ts[i] * inv * (1.0f + p.nw[i]);
+            auto out1 = [&](int i, float v) {
                 ss = fmadd(v, v, ss);
                 if (keep) {
                     p.x_out[i] = v;
                     if (p.copy != nullptr) p.copy[i] = v;
                 }
                 if (p.nw2 != nullptr) ts[i] = v; else xs[i] = from_f32<T>(v);
-            }
+            };
+            auto out4 = [&](int i, f32x4 w) {
+                const f32x4 t = reinterpret_cast<const f32x4*>(ts)[i];
+#pragma unroll
+                for (int j = 0; j < 4; ++j) out1(i * 4 + j, t[j] * inv * (1.0f + w[j]));
+            };
+#pragma unroll
+            for (int i = 0; i < kPre; ++i)
+                if (tid + i * kSeqThreads < w4) out4(tid + i * kSeqThreads, pn[i]);
+            for (int i = tid + kPre * kSeqThreads; i < w4; i += kSeqThreads) out4(i, n4[i]);
+            for (int i = w4 * 4 + tid; i < p.width; i += kSeqThreads) out1(i, ts[i] * inv * (1.0f + p.nw[i]));
             if (p.nw2 != nullptr) {
                 __syncthreads();
                 inv = inv_rms(block_sum(ss, red), p.width, p.eps);
@@ -822,54 +924,77 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
     }
     __syncthreads();
 
-    // ---- the rows
-    float acc = 0.0f, gate = 0.0f, top_v = -INFINITY;
-    int top_i = 0;
+    // ---- the rows; finished outputs are parked in LDS and stored together at the end
+    const int n_out = u1 - u0;
+    float* park = reinterpret_cast<float*>(smem + p.park) + wave * p.park_n;
+    float acc = 0.0f, gate = 0.0f;
+    int c_use = 0, r_use = 0, done = 0;                  // chunk and row of the output in work, outputs finished
     const float we = p.top > 0 ? 1.0f / (float)p.top : 1.0f;
-    auto consume = [&](const u32x4 (&b)[kGemvLoads]) {
+    auto consume = [&](const u32x4 (&b)[kGemvLoads]) __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < kGemvLoads; ++i)
-            if (use.c + i < nch) {
-                const u32x4 x = *reinterpret_cast<const u32x4*>(smem + (use.c + i) * kGemvChunk + lane * 16);
+            if (done < n_out) {
+                const u32x4 x = *reinterpret_cast<const u32x4*>(smem + c_use * kGemvChunk + lane * 16);
                 if constexpr (KCAT)
-                    acc = use.c + i < nch_all_e ? fmadd(we, dot16<T>(b[i], x, 0.0f), acc) : dot16<T>(b[i], x, acc);
+                    acc = fmadd(c_use < nch_all_e ? we : 1.0f, dot16<T>(b[i], x, 0.0f), acc);
                 else
                     acc = dot16<T>(b[i], x, acc);
-            }
-        if (use.c + kGemvLoads >= nch) {
-            const float v = wave_sum(acc);
-            acc = 0.0f;
-            if constexpr (EPI == kEpiF32) {
-                if (lane == 0) p.yf[use.u] = p.bias != nullptr ? v + p.bias[use.u] : v;
-            } else if constexpr (EPI == kEpiHead) {
-                const float z = soft_cap(v, p.cap);
-                if (lane == 0) p.yf[use.u] = z;
-                if (z > top_v) {
-                    top_v = z;
-                    top_i = use.u;
-                }
-            } else if constexpr (EPI == kEpiRelu2) {
-                if (lane == 0) reinterpret_cast<T*>(p.yt)[use.u] = from_f32<T>(relu2(v));
-            } else {
-                if (use.r == 0) {
-                    gate = v;
-                } else if (lane == 0) {
-                    const int b = use.u < p.top * p.units_e ? use.u / p.units_e : p.top;
-                    reinterpret_cast<T*>(p.yt + (size_t)b * p.seg_y)[use.u - b * p.units_e] = from_f32<T>(silu(gate) * v);
+                if (++c_use == nch) {
+                    c_use = 0;
+                    const float v = wave_sum(acc);
+                    acc = 0.0f;
+                    if (UR == 2 && r_use == 0) {
+                        gate = v;
+                        r_use = 1;
+                    } else {
+                        if (lane == 0) park[done] = UR == 2 ? silu(gate) * v : v;
+                        r_use = 0;
+                        ++done;
+                    }
                 }
             }
-        }
-        advance(use);
     };
-    for (int s = 0; s < nsteps; s += 2) {
+    const int steps = (n_out * UR * nch + kGemvLoads - 1) / kGemvLoads;
+    for (int s = 2; s < steps; s += 2) {                 // the steps before the last two
         consume(b0);
-        if (s + 2 < nsteps) { request(ask, b0); advance(ask); }
-        if (s + 1 < nsteps) {
-            consume(b1);
-            if (s + 3 < nsteps) { request(ask, b1); advance(ask); }
+        request(b0);
+        consume(b1);
+        request(b1);
+    }
+    consume(b0);
+    consume(b1);
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    float top_v = -INFINITY;
+    int top_i = 0;
+    for (int i = lane; i < n_out; i += kWave) {
+        const float v = park[i];
+        const int u = u0 + i;
+        if constexpr (EPI == kEpiF32) {
+            p.yf[u] = p.bias != nullptr ? v + p.bias[u] : v;
+        } else if constexpr (EPI == kEpiHead) {
+            const float z = soft_cap(v, p.cap);
+            p.yf[u] = z;
+            if (z > top_v) {
+                top_v = z;
+                top_i = u;
+            }
+        } else if constexpr (EPI == kEpiRelu2) {
+            reinterpret_cast<T*>(p.yt)[u] = from_f32<T>(relu2(v));
+        } else {
+            const int b = u < p.top * p.units_e ? u / p.units_e : p.top;
+            reinterpret_cast<T*>(p.yt + (size_t)b * p.seg_y)[u - b * p.units_e] = from_f32<T>(v);
         }
     }
     if constexpr (EPI == kEpiHead) {
+        for (int m = 1; m < kWave; m <<= 1) {            // the wave's best; the lowest row on ties
+            const float ov = __shfl_xor(top_v, m, kWave);
+            const int oi = __shfl_xor(top_i, m, kWave);
+            if (ov > top_v || (ov == top_v && oi < top_i)) {
+                top_v = ov;
+                top_i = oi;
+            }
+        }
         if (lane == 0) {
             bv[wave] = top_v;
             bi[wave] = top_i;
@@ -1220,12 +1345,14 @@ int run_portion(cfpp_seq* s, int slot, int n, int pos, int n_want, float* logits
 
 // ---- one token ---------------------------------------------------------------------------------
 template <typename T, int EPI, bool KCAT>
-int gemv(const cfpp_seq* s, const SeqGemv& p, hipStream_t st) {
+int gemv(const cfpp_seq* s, SeqGemv p, hipStream_t st) {
     const int nch_e = ceil_div(p.pitch_e, kGemvChunk), nch_s = ceil_div(p.pitch_s, kGemvChunk);
     const int nch = KCAT ? p.top * nch_e + nch_s : nch_s;
-    const size_t lds = (size_t)nch * kGemvChunk + (p.input == kInNorm ? (size_t)p.width * 4 : 0);
     const int total = KCAT ? p.units_s : p.top * p.units_e + p.units_s;
-    const int grid = std::max(1, std::min(2 * s->cus, ceil_div(total, kSeqWaves)));
+    const int grid = std::max(1, std::min(kGemvWgs * s->cus, ceil_div(total, kSeqWaves)));
+    p.park = nch * kGemvChunk + (p.input == kInNorm ? up_to(p.width * 4, 16) : 0);
+    p.park_n = ceil_div(total, grid * kSeqWaves);
+    const size_t lds = (size_t)p.park + (size_t)p.park_n * kSeqWaves * 4;
     allow_lds(k_seq_gemv<T, EPI, KCAT>, lds);
     hipLaunchKernelGGL((k_seq_gemv<T, EPI, KCAT>), dim3(grid), dim3(kSeqThreads), lds, st, p);
     return grid;
@@ -1446,7 +1573,7 @@ int cfpp_seq_create(const cfpp_seq_desc* desc, cfpp_seq** out) {
         L.n_qkv = d.heads * d.dim + d.kv_heads * (d.dim + d.vdim);
         L.v_role = !d.v_mix ? 0 : i == first_mix ? 1 : 2;
         const int kt = esize == 2 ? 32 : (L.NT <= 128 ? 32 : 16);
-        L.ns = std::max(1, std::min({kMaxSeqSplit, ceil_div(s->cus, d.kv_heads * L.nct), ceil_div(L.rows, kt * kSeqWaves)}));
+        L.ns = std::max(1, std::min({kMaxSeqSplit, ceil_div(kAttnWgs * s->cus, d.kv_heads * L.nct), ceil_div(L.rows, kt)}));
         L.kc = s->alloc<char>((size_t)D.slots * d.kv_heads * L.rows * L.krow);
         L.vc = s->alloc<char>((size_t)D.slots * d.kv_heads * L.rows * L.vrow);
         L.cs = nullptr;
@@ -1516,8 +1643,8 @@ int cfpp_seq_create(const cfpp_seq_desc* desc, cfpp_seq** out) {
     s->dy = s->alloc<float>(D.width);
     s->dres = s->alloc<float>((size_t)D.n_layers * D.width);
     s->logits = s->alloc<float>(D.vocab);
-    s->best_v = s->alloc<float>(2 * s->cus);
-    s->best_i = s->alloc<int>(2 * s->cus);
+    s->best_v = s->alloc<float>(kGemvWgs * s->cus);
+    s->best_i = s->alloc<int>(kGemvWgs * s->cus);
     if (!s->failed && hipDeviceSynchronize() != hipSuccess) s->failed = true;
     if (!s->failed && !s->host_routes.empty() &&
         hipMemcpy(s->routes, s->host_routes.data(), s->host_routes.size() * sizeof(SeqRoute), hipMemcpyHostToDevice) != hipSuccess)
