@@ -34,6 +34,11 @@ __device__ __forceinline__ float to_f32(bf16_t v) { return (float)v; }
 __device__ __forceinline__ float to_f32(float v) { return v; }
 template <typename T> __device__ __forceinline__ T from_f32(float v) { return (T)v; }
 
+__device__ __forceinline__ uint32_t pack_bf16(float a, float b) {
+    bf16x2_t v = {(bf16_t)a, (bf16_t)b};
+    return __builtin_bit_cast(uint32_t, v);
+}
+
 template <typename T> __device__ __forceinline__ f32x4 mma16(u32x4 a, u32x4 b, f32x4 c);
 template <> __device__ __forceinline__ f32x4 mma16<bf16_t>(u32x4 a, u32x4 b, f32x4 c) {
     return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), c, 0, 0, 0);
@@ -75,7 +80,7 @@ __device__ __forceinline__ void lds_barrier() {
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
 }
 
-// sum over the workgroup, in every thread, in a fixed order; `red` holds kSeqWaves floats (2 of them: two sums at a time)
+// sum over the workgroup, in every thread, in a fixed order; `red` holds kSeqWaves values
 __device__ __forceinline__ float block_sum(float v, float* red) {
     v = wave_sum(v);
     __syncthreads();
@@ -84,20 +89,82 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
     return (red[0] + red[1]) + (red[2] + red[3]);
 }
 
+__device__ __forceinline__ float2 block_sum2(float a, float b, float2* red) {
+    a = wave_sum(a);
+    b = wave_sum(b);
+    __syncthreads();
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = make_float2(a, b);
+    __syncthreads();
+    return make_float2((red[0].x + red[1].x) + (red[2].x + red[3].x), (red[0].y + red[1].y) + (red[2].y + red[3].y));
+}
+
 __device__ __forceinline__ float inv_rms(float sum_sq, int n, float eps) { return 1.0f / sqrtf(sum_sq / (float)n + eps); }
 __device__ __forceinline__ float relu2(float v) { v = fmaxf(v, 0.0f); return v * v; }
 __device__ __forceinline__ float soft_cap(float v, float cap) { return cap > 0.0f ? cap * tanhf(v / cap) : v; }
 
-// Element d of one head after the norm over the whole projection (inv, w) and the rotation; `row` is the head's slice of
-// the projection, `w` of the norm weight, `cs` the (cos, sin) pairs of the position.
-__device__ __forceinline__ float norm_rotate(const float* __restrict__ row, const float* __restrict__ w, float inv, int d, int rot,
-                                             const float2* __restrict__ cs) {
-    const float a = row[d] * inv * w[d];
-    if (d >= rot) return a;
-    const float b = row[d ^ 1] * inv * w[d ^ 1];
-    const float2 t = cs[d >> 1];
-    return (d & 1) ? a * t.x + b * t.y : a * t.x - b * t.y;
+// sum of squares of n floats over the workgroup's threads (each thread's share)
+__device__ __forceinline__ float share_sq(const float* __restrict__ v, int n, int tid) {
+    float s = 0.0f;
+    int i0 = 0;
+    if (((uintptr_t)v & 15) == 0) {
+        i0 = n & ~3;
+        for (int i = tid; i < n / 4; i += 4 * kSeqThreads) {         // four loads in one round trip
+            f32x4 x[4];
+#pragma unroll
+            for (int b = 0; b < 4; ++b) x[b] = reinterpret_cast<const f32x4*>(v)[min(i + b * kSeqThreads, n / 4 - 1)];
+#pragma unroll
+            for (int b = 0; b < 4; ++b)
+                if (i + b * kSeqThreads < n / 4) {
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) s = fmadd(x[b][j], x[b][j], s);
+                }
+        }
+    }
+    for (int i = i0 + tid; i < n; i += kSeqThreads) s = fmadd(v[i], v[i], s);
+    return s;
 }
+
+// four values to T, 16 or 8 bytes (p aligned to that)
+template <typename T> __device__ __forceinline__ void store4(void* p, f32x4 v) {
+    if constexpr (sizeof(T) == 4) {
+        *reinterpret_cast<f32x4*>(p) = v;
+    } else {
+        *reinterpret_cast<u32x2*>(p) = u32x2{pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3])};
+    }
+}
+// N = 4: one access of 16 (T: 8) bytes; N = 1: one element
+template <int N> __device__ __forceinline__ void add_n(float (&s)[N], const float* __restrict__ p) {
+    if constexpr (N == 4) {
+        const f32x4 v = *reinterpret_cast<const f32x4*>(p);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) s[j] += v[j];
+    } else {
+        s[0] += *p;
+    }
+}
+template <typename T, int N> __device__ __forceinline__ void put_n(T* p, const float (&v)[N]) {
+    if constexpr (N == 4) store4<T>(p, f32x4{v[0], v[1], v[2], v[3]});
+    else *p = from_f32<T>(v[0]);
+}
+
+// Element d of head h of a run of heads (D elements each) after the norm over the whole projection and the rotation: the
+// element and its partner with their norm weights, and (cos, sin) of the pair.  `row` is the run in the projection, `w` in
+// the norm weight, `cs` the pairs of the position.
+struct RotIn { float a, b, c, s; };
+__device__ __forceinline__ RotIn rotate_request(const float* __restrict__ row, const float* __restrict__ w, int h, int d, int D, int rot,
+                                                const float2* __restrict__ cs) {
+    const int e = h * D + d;
+    RotIn r = {row[e] * w[e], 0.0f, 1.0f, 0.0f};
+    if (d < rot) {
+        const int o = e + ((d & 1) ? -1 : 1);
+        const float2 t = cs[d >> 1];
+        r.b = row[o] * w[o];
+        r.c = t.x;
+        r.s = (d & 1) ? t.y : -t.y;
+    }
+    return r;
+}
+__device__ __forceinline__ float rotate_finish(const RotIn& r, float inv) { return (r.a * inv) * r.c + (r.b * inv) * r.s; }
 
 // First position of position p's chunk (chunk 0: the whole past).
 __device__ __forceinline__ int chunk_start(int p, int chunk) { return chunk > 0 ? (p / chunk) * chunk : 0; }
@@ -201,11 +268,6 @@ __device__ __forceinline__ void attn_softmax(AttnState<NT>& st, f32x4 (&s)[NKT],
 #pragma unroll
     for (int i = 0; i < NT / 16; ++i)
         if (i < vtiles) st.acc[i] *= c;
-}
-
-__device__ __forceinline__ uint32_t pack_bf16(float a, float b) {
-    bf16x2_t v = {(bf16_t)a, (bf16_t)b};
-    return __builtin_bit_cast(uint32_t, v);
 }
 
 // acc += V^T p for the keys of one tile

@@ -20,6 +20,7 @@
 #include <algorithm>
 #include <map>
 #include <new>
+#include <type_traits>
 #include <utility>
 #include <vector>
 
@@ -33,7 +34,7 @@ namespace {
 enum : int { kStToken = 0, kStPos = 1, kStSteps = 2, kStSlot = 3 };
 constexpr int kAttnCols = 16;          // query columns of a decode item (one MFMA column tile)
 constexpr int kMaxSeqSplit = 64;       // KV splits of a decode step
-constexpr int kAttnWgs = 2;            // ... sized for this many workgroups per compute unit
+constexpr int kAttnWgs = 1;            // ... sized for this many workgroups per compute unit
 
 // ------------------------------------------------------------------------------------------------
 // small kernels
@@ -87,29 +88,52 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_postnorm(SeqPostNorm a) {
     extern __shared__ __align__(16) float ts[];
     const int t = a.rows != nullptr ? a.rows[blockIdx.x] : (int)blockIdx.x;
     const float* x = a.x + (size_t)t * a.width;
+    char* xb = a.xb + (size_t)blockIdx.x * a.pitch;
     float ss = 0.0f;
-    for (int i = threadIdx.x; i < a.width; i += kSeqThreads) {
-        float s = 0.0f;
+    // N elements at a time (4 where the rows allow it); every thread reads back only what it has written
+    auto sum = [&](auto n, int i) {
+        constexpr int N = decltype(n)::value;
+        float s[N];
+#pragma unroll
+        for (int j = 0; j < N; ++j) s[j] = 0.0f;
         if (a.ys != nullptr) {
             const float* ys = a.ys + (size_t)t * a.top * a.width + i;
-            for (int j = 0; j < a.top; ++j) s += ys[(size_t)j * a.width];
-            s *= a.slot_weight;
+            for (int e = 0; e < a.top; ++e) add_n<N>(s, ys + (size_t)e * a.width);
+#pragma unroll
+            for (int j = 0; j < N; ++j) s[j] *= a.slot_weight;
         }
-        if (a.y != nullptr) s += a.y[(size_t)t * a.width + i];
-        const float v = a.rows != nullptr ? x[i] : fmadd(a.alpha, x[i], s);
-        ts[i] = v;
-        ss = fmadd(v, v, ss);
-    }
-    const float inv = inv_rms(block_sum(ss, red), a.width, a.eps);
-    T* xb = reinterpret_cast<T*>(a.xb + (size_t)blockIdx.x * a.pitch);
-    for (int i = threadIdx.x; i < a.width; i += kSeqThreads) {
-        const float v = ts[i] * inv * (1.0f + a.w[i]);
+        if (a.y != nullptr) add_n<N>(s, a.y + (size_t)t * a.width + i);
+        float v[N];
+#pragma unroll
+        for (int j = 0; j < N; ++j) v[j] = 0.0f;
+        add_n<N>(v, x + i);
+#pragma unroll
+        for (int j = 0; j < N; ++j) {
+            if (a.rows == nullptr) v[j] = fmadd(a.alpha, v[j], s[j]);
+            ts[i + j] = v[j];
+            ss = fmadd(v[j], v[j], ss);
+        }
+    };
+    auto out = [&](auto n, int i, float inv) {
+        constexpr int N = decltype(n)::value;
+        float w[N], v[N];
+#pragma unroll
+        for (int j = 0; j < N; ++j) w[j] = 1.0f;
+        add_n<N>(w, a.w + i);
+#pragma unroll
+        for (int j = 0; j < N; ++j) v[j] = ts[i + j] * inv * w[j];
         if (a.rows == nullptr) {
-            a.x_out[(size_t)t * a.width + i] = v;
-            if (a.copy != nullptr) a.copy[(size_t)t * a.width + i] = v;
+            put_n<float, N>(a.x_out + (size_t)t * a.width + i, v);
+            if (a.copy != nullptr) put_n<float, N>(a.copy + (size_t)t * a.width + i, v);
         }
-        xb[i] = from_f32<T>(v);
-    }
+        put_n<T, N>(reinterpret_cast<T*>(xb) + i, v);
+    };
+    const int w4 = (a.width & 3) ? 0 : a.width;
+    for (int i = threadIdx.x * 4; i < w4; i += kSeqThreads * 4) sum(std::integral_constant<int, 4>{}, i);
+    for (int i = w4 + threadIdx.x; i < a.width; i += kSeqThreads) sum(std::integral_constant<int, 1>{}, i);
+    const float inv = inv_rms(block_sum(ss, red), a.width, a.eps);
+    for (int i = threadIdx.x * 4; i < w4; i += kSeqThreads * 4) out(std::integral_constant<int, 4>{}, i, inv);
+    for (int i = w4 + threadIdx.x; i < a.width; i += kSeqThreads) out(std::integral_constant<int, 1>{}, i, inv);
 }
 
 // One workgroup per token: raw q | k | v rows (fp32, biases included) -> norm over all of q and all of k, rotation, value
@@ -127,37 +151,62 @@ struct SeqQkv {
 };
 template <typename T>
 __global__ __launch_bounds__(kSeqThreads) void k_seq_qkv_finish(SeqQkv a) {
-    __shared__ float red[kSeqWaves];
+    __shared__ float2 red[kSeqWaves];
     const int t = blockIdx.x, nq = a.H * a.D, nk = a.G * a.D, nv = a.G * a.V;
     const float* q = a.qkv + (size_t)t * a.ld;
     const float *k = q + nq, *v = k + nk;
-    float sq = 0.0f, sk = 0.0f;
-    for (int i = threadIdx.x; i < nq; i += kSeqThreads) sq = fmadd(q[i], q[i], sq);
-    for (int i = threadIdx.x; i < nk; i += kSeqThreads) sk = fmadd(k[i], k[i], sk);
-    const float iq = inv_rms(block_sum(sq, red), nq, a.eps), ik = inv_rms(block_sum(sk, red), nk, a.eps);
+    const float2 sums = block_sum2(share_sq(q, nq, threadIdx.x), share_sq(k, nk, threadIdx.x), red);
+    const float iq = inv_rms(sums.x, nq, a.eps), ik = inv_rms(sums.y, nk, a.eps);
     const float2* cs = a.cs + (size_t)(a.pos0 + t) * (a.rot / 2);
-    T* qo = reinterpret_cast<T*>(a.q) + (size_t)t * a.H * a.Dp;
-    T* ko = reinterpret_cast<T*>(a.k) + (size_t)t * a.Dp;
-    T* vo = reinterpret_cast<T*>(a.v) + (size_t)t * a.Vp;
-    // (the padding of a row is written too: layers of other sizes share these buffers)
-    for (int i = threadIdx.x; i < a.H * a.Dp; i += kSeqThreads) {
-        const int h = i / a.Dp, d = i - h * a.Dp;
-        qo[i] = from_f32<T>(d < a.D ? norm_rotate(q + h * a.D, a.qn + h * a.D, iq, d, a.rot, cs) : 0.0f);
-    }
-    for (int i = threadIdx.x; i < a.G * a.Dp; i += kSeqThreads) {
-        const int g = i / a.Dp, d = i - g * a.Dp;
-        ko[(size_t)g * a.cap * a.Dp + d] = from_f32<T>(d < a.D ? norm_rotate(k + g * a.D, a.kn + g * a.D, ik, d, a.rot, cs) : 0.0f);
-    }
-    for (int i = threadIdx.x; i < a.G * a.Vp; i += kSeqThreads) {
-        const int g = i / a.Vp, d = i - g * a.Vp;
-        float x = 0.0f;
-        if (d < a.V) {
-            float* first = a.v_first + (size_t)t * nv + g * a.V + d;
-            x = v[g * a.V + d];
-            if (a.v_role == 1) *first = x;
-            if (a.v_role == 2) x = (1.0f - a.lambda) * x + a.lambda * *first;
+    char* qo = a.q + (size_t)t * a.H * a.Dp * sizeof(T);
+    char* ko = a.k + (size_t)t * a.Dp * sizeof(T);
+    char* vo = a.v + (size_t)t * a.Vp * sizeof(T);
+    const size_t khead = (size_t)a.cap * a.Dp * sizeof(T), vhead = (size_t)a.cap * a.Vp * sizeof(T);
+    // four elements at a time: head `h`, elements d .. d + 3 of its padded row (zeros past the end: the padding is written
+    // too, since layers of other sizes share these buffers)
+    auto rotated = [&](const float* row, const float* w, float inv, int d) {
+        f32x4 x, y;
+        const bool whole = d + 3 < a.D && ((uintptr_t)(row + d) & 15) == 0 && ((uintptr_t)(w + d) & 15) == 0;
+        if (whole) {
+            const f32x4 xr = *reinterpret_cast<const f32x4*>(row + d), wr = *reinterpret_cast<const f32x4*>(w + d);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) x[j] = xr[j] * wr[j];
+        } else {
+#pragma unroll
+            for (int j = 0; j < 4; ++j) x[j] = d + j < a.D ? row[d + j] * w[d + j] : 0.0f;
         }
-        vo[(size_t)g * a.cap * a.Vp + d] = from_f32<T>(x);
+#pragma unroll
+        for (int j = 0; j < 4; j += 2) {
+            const bool r = d + j < a.rot;
+            const float2 cc = r ? cs[(d + j) / 2] : make_float2(1.0f, 0.0f);
+            y[j] = rotate_finish(RotIn{x[j], x[j + 1], cc.x, -cc.y}, inv);
+            y[j + 1] = rotate_finish(RotIn{x[j + 1], x[j], cc.x, cc.y}, inv);
+        }
+        return y;
+    };
+    const int q4 = a.Dp / 4, v4 = a.Vp / 4;
+    for (int i = threadIdx.x; i < a.H * q4; i += kSeqThreads) {
+        const int h = i / q4, d = (i - h * q4) * 4;
+        store4<T>(qo + ((size_t)h * a.Dp + d) * sizeof(T), rotated(q + h * a.D, a.qn + h * a.D, iq, d));
+    }
+    for (int i = threadIdx.x; i < a.G * q4; i += kSeqThreads) {
+        const int g = i / q4, d = (i - g * q4) * 4;
+        store4<T>(ko + g * khead + d * sizeof(T), rotated(k + g * a.D, a.kn + g * a.D, ik, d));
+    }
+    for (int i = threadIdx.x; i < a.G * v4; i += kSeqThreads) {
+        const int g = i / v4, d = (i - g * v4) * 4;
+        f32x4 x;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            x[j] = 0.0f;
+            if (d + j < a.V) {
+                float* first = a.v_first + (size_t)t * nv + g * a.V + d + j;
+                x[j] = v[g * a.V + d + j];
+                if (a.v_role == 1) *first = x[j];
+                if (a.v_role == 2) x[j] = (1.0f - a.lambda) * x[j] + a.lambda * *first;
+            }
+        }
+        store4<T>(vo + g * vhead + d * sizeof(T), x);
     }
 }
 
@@ -524,22 +573,6 @@ struct SeqAttnDec {
 };
 template <typename T, int NT> struct DecTile { static constexpr int kt = sizeof(T) == 2 ? 32 : (NT <= 128 ? 32 : 16); };
 
-// sum of squares of n floats over the workgroup's threads (each thread's share)
-__device__ __forceinline__ float share_sq(const float* __restrict__ v, int n, int tid) {
-    float s = 0.0f;
-    int i0 = 0;
-    if (((uintptr_t)v & 15) == 0) {
-        i0 = n & ~3;
-        for (int i = tid; i < n / 4; i += kSeqThreads) {
-            const f32x4 x = reinterpret_cast<const f32x4*>(v)[i];
-#pragma unroll
-            for (int j = 0; j < 4; ++j) s = fmadd(x[j], x[j], s);
-        }
-    }
-    for (int i = i0 + tid; i < n; i += kSeqThreads) s = fmadd(v[i], v[i], s);
-    return s;
-}
-
 template <typename T, int NT>
 __global__ __launch_bounds__(kSeqThreads) void k_seq_attn_decode(SeqAttnDec a) {
     constexpr int KT = DecTile<T, NT>::kt, NB = NT * (int)sizeof(T);
@@ -547,14 +580,16 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_attn_decode(SeqAttnDec a) {
     constexpr int VS = VtSteps<T, KT, NT, kWave>::n, KF = KT / 16;
     __shared__ __align__(16) char buf[kSeqWaves * (VB > MB ? VB : MB)];
     __shared__ __align__(16) char qs[kAttnCols * NB];
-    __shared__ float red[kSeqWaves], wm[kSeqWaves][kAttnCols], wl[kSeqWaves][kAttnCols];
+    __shared__ float2 red2[kSeqWaves];
+    __shared__ float wm[kSeqWaves][kAttnCols], wl[kSeqWaves][kAttnCols];
     __shared__ float sm[kMaxSeqSplit][kAttnCols], sl[kMaxSeqSplit][kAttnCols];
     __shared__ int last;
     const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, col = lane & 15, g = lane >> 4;
     const int item = blockIdx.y, gq = item / a.nct, cols0 = (item - gq * a.nct) * kAttnCols, ncols = min(kAttnCols, a.R - cols0);
     const int pos = a.state[kStPos], slot = a.state[kStSlot];
-    // tiles of KT keys are shared evenly among the splits
-    const int k_first = chunk_start(pos, a.chunk), ntiles = (pos - k_first + KT) / KT, nsplit = min(a.ns, ntiles), sp = blockIdx.x;
+    // tiles of KT keys are shared evenly among the splits, no more of them than give every wave a tile
+    const int k_first = chunk_start(pos, a.chunk), ntiles = (pos - k_first + KT) / KT;
+    const int nsplit = min(a.ns, (ntiles + kSeqWaves - 1) / kSeqWaves), sp = blockIdx.x;
     if (sp >= nsplit) return;
     const int k0 = k_first + mul_div(ntiles, sp, nsplit) * KT, k1 = min(k_first + mul_div(ntiles, sp + 1, nsplit) * KT, pos + 1);
     char* kc = a.kc + slot * a.k_slot + (size_t)gq * a.rows * a.krow;
@@ -572,37 +607,47 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_attn_decode(SeqAttnDec a) {
         }
         vt_request<T, KT, kWave, 0, VS>(vr, vunits, lane, [&](int key) { return vc + (size_t)(min(kb + key, k1 - 1) - k_first) * a.vrow; });
     };
+    // everything the prologue reads is requested up front: one round trip instead of one per use
     const int nq = a.H * a.D, nk = a.G * a.D;
     const float *q = a.qkv, *k = q + nq, *v = k + nk;
+    const float2* cs = a.cs + (size_t)pos * (a.rot / 2);
     const bool newest = k1 == pos + 1;                   // this split makes and appends the newest position's rows
+    // NT threads per head; the first kQ passes are held in registers, more query heads go through a loop
+    constexpr int kQ = 2, kHeads = kSeqThreads / NT;
+    const int own0 = (gq * a.R + cols0) * a.D, qd = tid % NT, qc = tid / NT;
+    RotIn rq[kQ], rk;
+    float vn = 0.0f, vm = 0.0f;
+#pragma unroll
+    for (int i = 0; i < kQ; ++i)
+        if (qc + i * kHeads < ncols && qd < a.D) rq[i] = rotate_request(q + own0, a.qn + own0, qc + i * kHeads, qd, a.D, a.rot, cs);
+    if (newest && tid < a.D) rk = rotate_request(k, a.kn, gq, tid, a.D, a.rot, cs);
+    if (newest && tid < a.V) {
+        vn = v[gq * a.V + tid];
+        if (a.v_role == 2) vm = a.v_first[gq * a.V + tid];
+    }
     const float sq = share_sq(q, nq, tid), sk = newest ? share_sq(k, nk, tid) : 0.0f;
     // the wave's first tile, unless the newest position, which is not in the cache yet, is in it
     int kb = k0 + wave * KT;
     const bool early = kb + KT <= pos && kb < k1;
     if (early) fetch(kb);
 
-    const float2* cs = a.cs + (size_t)pos * (a.rot / 2);
-    {
-        const float iq = inv_rms(block_sum(sq, red), nq, a.eps);
-        const int dp = a.krow / (int)sizeof(T);
-        for (int i = tid; i < kAttnCols * dp; i += kSeqThreads) {
-            const int c = i / dp, d = i - c * dp, h = gq * a.R + cols0 + c;
-            float x = 0.0f;
-            if (c < ncols && d < a.D) x = norm_rotate(q + (size_t)h * a.D, a.qn + (size_t)h * a.D, iq, d, a.rot, cs);
-            reinterpret_cast<T*>(qs)[c * NT + d] = from_f32<T>(x);
-        }
-    }
+    for (int i = tid; i < kAttnCols * NB / 16; i += kSeqThreads) reinterpret_cast<u32x4*>(qs)[i] = u32x4{0, 0, 0, 0};
+    const float2 sums = block_sum2(sq, sk, red2);        // (its barriers also separate the zeros from what follows)
+    const float iq = inv_rms(sums.x, nq, a.eps);
+    T* qt = reinterpret_cast<T*>(qs);
+#pragma unroll
+    for (int i = 0; i < kQ; ++i)
+        if (qc + i * kHeads < ncols && qd < a.D) qt[(qc + i * kHeads) * NT + qd] = from_f32<T>(rotate_finish(rq[i], iq));
+#pragma unroll 1
+    for (int c = qc + kQ * kHeads; c < ncols; c += kHeads)
+        if (qd < a.D) qt[c * NT + qd] = from_f32<T>(rotate_finish(rotate_request(q + own0, a.qn + own0, c, qd, a.D, a.rot, cs), iq));
     if (newest) {
-        const float ik = inv_rms(block_sum(sk, red), nk, a.eps);
-        T* ko = reinterpret_cast<T*>(kc + (size_t)(pos - k_first) * a.krow);
-        T* vo = reinterpret_cast<T*>(vc + (size_t)(pos - k_first) * a.vrow);
-        for (int d = tid; d < a.D; d += kSeqThreads)
-            ko[d] = from_f32<T>(norm_rotate(k + (size_t)gq * a.D, a.kn + (size_t)gq * a.D, ik, d, a.rot, cs));
-        for (int d = tid; d < a.V; d += kSeqThreads) {
-            float x = v[gq * a.V + d];
-            if (a.v_role == 1) a.v_first[gq * a.V + d] = x;
-            if (a.v_role == 2) x = (1.0f - a.lambda) * x + a.lambda * a.v_first[gq * a.V + d];
-            vo[d] = from_f32<T>(x);
+        const float ik = inv_rms(sums.y, nk, a.eps);
+        if (tid < a.D) reinterpret_cast<T*>(kc + (size_t)(pos - k_first) * a.krow)[tid] = from_f32<T>(rotate_finish(rk, ik));
+        if (tid < a.V) {
+            if (a.v_role == 1) a.v_first[gq * a.V + tid] = vn;
+            if (a.v_role == 2) vn = (1.0f - a.lambda) * vn + a.lambda * vm;
+            reinterpret_cast<T*>(vc + (size_t)(pos - k_first) * a.vrow)[tid] = from_f32<T>(vn);
         }
     }
     __syncthreads();
@@ -683,33 +728,56 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_attn_decode(SeqAttnDec a) {
     }
     __syncthreads();
     if (!last) return;
+    // pairs of value columns, kM splits at a time; the first ones travel together with the maxima
+    constexpr int kM = 8;
+    const int half = vp / 2, pairs = ncols * half, split_stride = kAttnCols * stride;
+    float2 pv[kM];
+    auto request = [&](const float* p0, int s0) {
+#pragma unroll
+        for (int j = 0; j < kM; ++j) ld_agent2(p0 + (size_t)min(s0 + j, nsplit - 1) * split_stride, pv[j].x, pv[j].y);
+    };
     for (int i = tid; i < nsplit * ncols; i += kSeqThreads) {
         const int s = i / ncols, c = i - s * ncols;
-        const float* pr = part + ((size_t)s * kAttnCols + c) * stride;
-        sm[s][c] = ld_agent(pr);
-        sl[s][c] = ld_agent(pr + 1);
+        ld_agent2(part + (size_t)s * split_stride + c * stride, sm[s][c], sl[s][c]);
     }
+    int i = tid, c = i / half, x = (i - c * half) * 2;
+    if (i < pairs) request(part + c * stride + 2 + x, 0);
     __syncthreads();
-    for (int i = tid; i < ncols * vp; i += kSeqThreads) {
-        const int c = i / vp, x = i - c * vp, h = gq * a.R + cols0 + c;
+#pragma unroll 1
+    while (i < pairs) {
+        const int h = gq * a.R + cols0 + c;
         const float snk = a.sink[h] * kLog2e;
         float m = snk;
         for (int s = 0; s < nsplit; ++s) m = fmaxf(m, sm[s][c]);
-        float acc = 0.0f, l = fast_exp2(snk - m);
-#pragma unroll 8
-        for (int s = 0; s < nsplit; ++s) {
-            const float f = fast_exp2(sm[s][c] - m);
-            acc = fmadd(ld_agent(part + ((size_t)s * kAttnCols + c) * stride + 2 + x), f, acc);
-            l = fmadd(sl[s][c], f, l);
+        float ax = 0.0f, ay = 0.0f, l = fast_exp2(snk - m);
+#pragma unroll 1
+        for (int s0 = 0;;) {
+#pragma unroll
+            for (int j = 0; j < kM; ++j)
+                if (s0 + j < nsplit) {
+                    const float f = fast_exp2(sm[s0 + j][c] - m);
+                    ax = fmadd(pv[j].x, f, ax);
+                    ay = fmadd(pv[j].y, f, ay);
+                    l = fmadd(sl[s0 + j][c], f, l);
+                }
+            s0 += kM;
+            if (s0 >= nsplit) break;
+            request(part + c * stride + 2 + x, s0);
         }
-        if (x < a.V) reinterpret_cast<T*>(a.out)[(size_t)h * a.V + x] = from_f32<T>(acc / l);
+        T* o = reinterpret_cast<T*>(a.out) + (size_t)h * a.V + x;
+        if (x < a.V) o[0] = from_f32<T>(ax / l);
+        if (x + 1 < a.V) o[1] = from_f32<T>(ay / l);
+        i += kSeqThreads;
+        c = i / half;
+        x = (i - c * half) * 2;
+        if (i < pairs) request(part + c * stride + 2 + x, 0);
     }
 }
 
 // ------------------------------------------------------------------------------------------------
 // matrix-vector products of one token
 // ------------------------------------------------------------------------------------------------
-// A wave streams its weight rows as one sequence of 1 KB chunks (one wave-wide load each), eight per step, two steps in
+// A wave streams its weight rows as one sequence of 1 KB chunks (one wave-wide load each), four per step, two steps in
 // flight, the first two requested before the prologue.  The input sits in LDS.  Rows go to waves in equal contiguous shares.
 //
 // ROWS: the outputs are the rows of up to `top` chosen matrices and of one that is always there, one after the other.
@@ -746,8 +814,8 @@ struct SeqGemv {
     int park, park_n;        // LDS: offset of the finished outputs, outputs per wave at most
 };
 constexpr int kGemvChunk = 1024;      // bytes of a row per wave-wide load
-constexpr int kGemvLoads = 8;         // loads per step
-constexpr int kGemvWgs = 2;           // workgroups per compute unit
+constexpr int kGemvLoads = 4;         // loads per step
+constexpr int kGemvWgs = 4;           // workgroups per compute unit
 
 template <typename T, int EPI, bool KCAT>
 __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
@@ -1573,7 +1641,7 @@ int cfpp_seq_create(const cfpp_seq_desc* desc, cfpp_seq** out) {
         L.n_qkv = d.heads * d.dim + d.kv_heads * (d.dim + d.vdim);
         L.v_role = !d.v_mix ? 0 : i == first_mix ? 1 : 2;
         const int kt = esize == 2 ? 32 : (L.NT <= 128 ? 32 : 16);
-        L.ns = std::max(1, std::min({kMaxSeqSplit, ceil_div(kAttnWgs * s->cus, d.kv_heads * L.nct), ceil_div(L.rows, kt)}));
+        L.ns = std::max(1, std::min({kMaxSeqSplit, ceil_div(kAttnWgs * s->cus, d.kv_heads * L.nct), ceil_div(L.rows, kt * kSeqWaves)}));
         L.kc = s->alloc<char>((size_t)D.slots * d.kv_heads * L.rows * L.krow);
         L.vc = s->alloc<char>((size_t)D.slots * d.kv_heads * L.rows * L.vrow);
         L.cs = nullptr;
