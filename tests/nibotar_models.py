@@ -86,6 +86,8 @@ CASES = {
     "rotation_whole": model(64, 51, [(attn(2, 1, 48, 64, base=1e6), None)]),
     "chunks": model(64, 51, [(attn(4, 2, 32, 40, chunk=13), None), (attn(3, 3, 16, 16, chunk=5), None)]),
     "many_heads_per_group": model(72, 51, [(attn(20, 1, 16, 8, chunk=50), None), (attn(34, 2, 8, 24), None)]),
+    "tiny_chunks": model(64, 51, [(attn(2, 1, 16, 16, chunk=1), None), (attn(4, 2, 24, 8, chunk=2), dense(40)), (attn(2, 2, 16, 16, chunk=3), None)]),
+    "more_experts_than_tokens": model(64, 51, [(attn(2, 2, 16, 16), moe(16, 300, 5, shared=24)), (attn(2, 2, 16, 16), moe(24, 2, 2))]),
     "value_mixing": model(64, 51, [(attn(2, 1, 16, 32), None), (attn(4, 2, 24, 20, v_mix=True), None), (attn(2, 2, 16, 20, chunk=9), None),
                                    (attn(8, 4, 16, 10, v_mix=True), None)]),
     "relu_squared": model(100, 51, [(attn(2, 2, 16, 16), dense(77)), (attn(2, 2, 16, 16), dense(260))]),
