@@ -67,6 +67,20 @@ template <> __device__ __forceinline__ float dot16<float>(u32x4 w, u32x4 x, floa
     return acc;
 }
 
+// the elements of a 16-byte unit
+template <typename T> __device__ __forceinline__ void unpack16(u32x4 b, float (&v)[Unit<T>::n]);
+template <> __device__ __forceinline__ void unpack16<bf16_t>(u32x4 b, float (&v)[8]) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        v[2 * j] = __uint_as_float(b[j] << 16);
+        v[2 * j + 1] = __uint_as_float(b[j] & 0xffff0000u);
+    }
+}
+template <> __device__ __forceinline__ void unpack16<float>(u32x4 b, float (&v)[4]) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = __uint_as_float(b[j]);
+}
+
 // 64 lanes copy 64 units from memory straight to LDS; the lanes' units land next to each other from `lds` (wave-uniform) on
 __device__ __forceinline__ void copy_to_lds16(const void* g, void* lds) {
     __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(uintptr_t)g,
@@ -78,6 +92,12 @@ __device__ __forceinline__ void lds_barrier() {
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
     __builtin_amdgcn_s_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
+}
+
+__device__ __forceinline__ float wave_max(float v) {
+#pragma unroll
+    for (int m = 1; m < kWave; m <<= 1) v = fmaxf(v, xor_shfl(v, m));
+    return v;
 }
 
 // sum over the workgroup, in every thread, in a fixed order; `red` holds kSeqWaves values
@@ -99,6 +119,7 @@ __device__ __forceinline__ float2 block_sum2(float a, float b, float2* red) {
 }
 
 __device__ __forceinline__ float inv_rms(float sum_sq, int n, float eps) { return 1.0f / sqrtf(sum_sq / (float)n + eps); }
+__device__ __forceinline__ float sigmoid(float v) { return 1.0f / (1.0f + fast_exp2(-v * kLog2e)); }
 __device__ __forceinline__ float relu2(float v) { v = fmaxf(v, 0.0f); return v * v; }
 __device__ __forceinline__ float soft_cap(float v, float cap) { return cap > 0.0f ? cap * tanhf(v / cap) : v; }
 

@@ -11,6 +11,9 @@
 //   k_seq_gemv (output rows)
 //   k_seq_gemv (residual sum + norm | up rows of the chosen and the shared experts | activation)
 //   k_seq_gemv (down rows of all of them, weighted and summed)
+// Latent mixers: k_seq_latent_finish, a product that makes keys and values of all heads, k_seq_attn in portions; k_seq_latent_q,
+// k_seq_latent_attn, k_seq_latent_out in decode (seq_latent.hpp).  Residual streams: k_seq_streams after every product that
+// ends a sublayer of a portion; in decode the output rows' own launch updates them.
 // then k_seq_gemv over the vocabulary (both last norms | head rows | soft cap | best logit per workgroup) and k_seq_pick.
 #include <hip/hip_runtime.h>
 #include <math.h>
@@ -20,12 +23,14 @@
 #include <algorithm>
 #include <map>
 #include <new>
+#include <tuple>
 #include <type_traits>
 #include <utility>
 #include <vector>
 
 #include "cfpp_seq.h"
 #include "seq_device.hpp"
+#include "seq_latent.hpp"
 
 using namespace cfpp;
 
@@ -75,7 +80,7 @@ struct SeqPostNorm {
     int top;
     float slot_weight;
     const float* w;
-    float alpha, eps;
+    float alpha, eps, noff;  // noff: the norm weight is noff + w
     int width;
     char* xb;
     int pitch;
@@ -118,7 +123,7 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_postnorm(SeqPostNorm a) {
         constexpr int N = decltype(n)::value;
         float w[N], v[N];
 #pragma unroll
-        for (int j = 0; j < N; ++j) w[j] = 1.0f;
+        for (int j = 0; j < N; ++j) w[j] = a.noff;
         add_n<N>(w, a.w + i);
 #pragma unroll
         for (int j = 0; j < N; ++j) v[j] = ts[i + j] * inv * w[j];
@@ -227,17 +232,22 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_append(SeqAppend a) {
 // ------------------------------------------------------------------------------------------------
 // matrix products of a portion: out[token][row] = W[row] . a[token]
 // ------------------------------------------------------------------------------------------------
-enum : int { kEpiF32 = 0, kEpiRelu2 = 1, kEpiGated = 2, kEpiHead = 3 };
+// kEpiHeads: rows of keys of all heads, then rows of values of all heads, each head's rows [position] in a buffer of its own.
+// kEpiStreams (one token): the output row goes into the residual streams.
+enum : int { kEpiF32 = 0, kEpiRelu2 = 1, kEpiGated = 2, kEpiHead = 3, kEpiHeads = 4, kEpiStreams = 5 };
 struct SeqGemm {
     const char* w;           // [n rows][kbytes]
     const char* a;           // [tokens][lda bytes]
     int n, m, kbytes, lda;
-    const float* bias;       // nullable (kEpiF32)
+    const float* bias;       // nullable (kEpiF32, kEpiGated)
     float* yf;               // kEpiF32 / kEpiHead: [tokens][ldy]
     int ldy;
-    char* yt;                // kEpiRelu2 / kEpiGated: T, [tokens][ldyt bytes]
+    char* yt;                // kEpiRelu2 / kEpiGated: T, [tokens][ldyt bytes]; kEpiHeads: keys
     int ldyt;
-    float cap;
+    float mul, cap;          // kEpiHead
+    char* yv;                // kEpiHeads: values; key rows of kd elements, kp bytes apart, heads kh bytes apart; values alike
+    int nk, kd, kp, vd, vp;  // ... nk: rows of keys
+    size_t kh, vh;
     // tiles of tokens sorted by expert (tile_off null: a plain product)
     const int* tile_off;     // [experts + 1] prefix sums of tiles
     const int* row_off;      // [experts + 1] prefix sums of sorted slots
@@ -358,7 +368,7 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemm(SeqGemm p) {
                 }
                 if (EPI == kEpiHead) {
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) o[r] = soft_cap(o[r], p.cap);
+                    for (int r = 0; r < 4; ++r) o[r] = soft_cap(o[r] * p.mul, p.cap);
                 }
                 if (n0 + 3 < p.n && (p.ldy & 3) == 0) {
                     *reinterpret_cast<f32x4*>(y) = o;
@@ -372,11 +382,31 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemm(SeqGemm p) {
 #pragma unroll
                 for (int r = 0; r < 4; ++r)
                     if (n0 + r < p.n) y[r] = from_f32<T>(relu2(v[r]));
+            } else if constexpr (EPI == kEpiHeads) {
+                const bool keys = n0 < p.nk;
+                const int d = keys ? p.kd : p.vd, n = keys ? n0 : n0 - p.nk, h = n / d, e = n - h * d;
+                char* base = (keys ? p.yt : p.yv) + (size_t)row * (keys ? p.kp : p.vp);
+                const size_t hs = keys ? p.kh : p.vh;
+                if (e + 3 < d && (e & 3) == 0 && n0 + 3 < (keys ? p.nk : p.n)) {
+                    store4<T>(base + h * hs + e * sizeof(T), v);
+                } else {
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) {
+                        if (n0 + r >= p.n) break;
+                        const bool k = n0 + r < p.nk;
+                        const int dd = k ? p.kd : p.vd, nn = k ? n0 + r : n0 + r - p.nk, hh = nn / dd;
+                        char* b = k ? p.yt + (size_t)row * p.kp + hh * p.kh : p.yv + (size_t)row * p.vp + hh * p.vh;
+                        reinterpret_cast<T*>(b)[nn - hh * dd] = from_f32<T>(v[r]);
+                    }
+                }
             } else {
                 T* y = reinterpret_cast<T*>(p.yt + (size_t)row * p.ldyt) + n0 / 2;
 #pragma unroll
                 for (int r = 0; r < 4; r += 2)
-                    if (n0 + r < p.n) y[r / 2] = from_f32<T>(silu(v[r]) * v[r + 1]);
+                    if (n0 + r < p.n) {
+                        const float bg = p.bias != nullptr ? p.bias[n0 + r] : 0.0f, bu = p.bias != nullptr ? p.bias[n0 + r + 1] : 0.0f;
+                        y[r / 2] = from_f32<T>(silu(v[r] + bg) * (v[r + 1] + bu));
+                    }
             }
         }
     }
@@ -420,22 +450,26 @@ __global__ __launch_bounds__(1024) void k_seq_route(const SeqRoute* layers, cons
 // attention of a portion
 // ------------------------------------------------------------------------------------------------
 // The query columns of one key / value head are (token, head of the group), head fastest; a workgroup takes 64 CT of them
-// and walks the keys its tokens can see, first the cached ones, then the portion's own.  The softmax is online, the sink is
-// added to the denominator at the end.
+// and walks the keys its tokens can see, first the cached ones (positions before k_split), then those in the buffer.  Behind a
+// key's own row comes the part that all heads share, if there is one.  The softmax is online, the sink is added to the
+// denominator at the end.
 struct SeqAttn {
     const char *q, *k, *v, *kc, *vc;
+    const char* kr;          // rows of the shared part, of position 0 on
     char* out;
-    const float* sink;
-    int T, H, R, dsteps, krow, vrow, V, vtiles, pos0, chunk, cap, rows, ldo;
+    const float* sink;       // nullable
+    const float* gate;       // nullable: [T][ldg], the outputs are multiplied by its sigmoid
+    int T, H, R, dsteps, qrow, krow, vrow, V, vtiles, pos0, chunk, cap, rows, ldo, k_split, runits, rrow, ldg;
     float scale_log2;
 };
-template <int UN> __device__ __forceinline__ int swz_key(int row) { return UN == 8 ? (row >> 1) & 7 : row & 15; }
+template <int UN> __device__ __forceinline__ int swz_key(int row) { return UN % 16 ? (row >> 1) & 7 : row & 15; }
 
 // (the next tile's keys go straight to the other LDS buffer and its values into registers while this one is worked on)
-template <typename T, int NT, int CT>
+// (NK: elements of a key row in LDS, NT: value columns)
+template <typename T, int NK, int NT, int CT>
 __global__ __launch_bounds__(kSeqThreads, (NT <= 128 ? 2 : 1)) void k_seq_attn(SeqAttn a) {
     constexpr int KT = sizeof(T) == 2 ? 64 : 32;
-    constexpr int NB = NT * (int)sizeof(T), UN = NB / 16, RPC = 1024 / NB;   // bytes and units of a key row in LDS, rows per copy
+    constexpr int NB = NK * (int)sizeof(T), UN = NB / 16;                    // bytes and units of a key row in LDS
     constexpr int VS = VtSteps<T, KT, NT, kSeqThreads>::n;
     __shared__ __align__(1024) char ks[2][KT * NB];
     __shared__ __align__(16) char vt[NT * VtTile<T, KT>::pitch];
@@ -452,7 +486,7 @@ __global__ __launch_bounds__(kSeqThreads, (NT <= 128 ? 2 : 1)) void k_seq_attn(S
         head[ct] = gq * a.R + (cc - tok[ct] * a.R);
         pq[ct] = a.pos0 + tok[ct];
         first[ct] = chunk_start(pq[ct], a.chunk);
-        const char* qr = a.q + ((size_t)tok[ct] * a.H + head[ct]) * a.krow + g * 16;
+        const char* qr = a.q + ((size_t)tok[ct] * a.H + head[ct]) * a.qrow + g * 16;
 #pragma unroll
         for (int s = 0; s < NB / 64; ++s)
             if (s < a.dsteps) qf[ct][s] = ld16(qr + s * 64);
@@ -466,20 +500,20 @@ __global__ __launch_bounds__(kSeqThreads, (NT <= 128 ? 2 : 1)) void k_seq_attn(S
     const int any_lo = chunk_start(a.pos0 + w_first, a.chunk), any_hi = a.pos0 + w_last;
     const int dunits = a.krow / 16, vunits = a.vrow / 16;
 
-    // tiles: [k_first, pos0) in the cache, then [pos0, k_end) in the portion
+    // tiles: [k_first, k_split) in the cache, then [k_split, k_end) in the buffer
     struct Tile { int k0, hi; const char *k, *v; };      // first key, end of its part, row of position 0
     auto tile_at = [&](int k0) {
-        const bool cached = k0 < a.pos0;
-        const size_t row0 = (size_t)gq * (cached ? a.rows : a.cap) - (cached ? chunk_start(a.pos0, a.chunk) : a.pos0);
-        return Tile{k0, cached ? min(k_end, a.pos0) : k_end, (cached ? a.kc : a.k) + (ptrdiff_t)row0 * a.krow, (cached ? a.vc : a.v) + (ptrdiff_t)row0 * a.vrow};
+        const bool cached = k0 < a.k_split;
+        const size_t row0 = (size_t)gq * (cached ? a.rows : a.cap) - (cached ? chunk_start(a.pos0, a.chunk) : a.k_split);
+        return Tile{k0, cached ? min(k_end, a.k_split) : k_end, (cached ? a.kc : a.k) + (ptrdiff_t)row0 * a.krow, (cached ? a.vc : a.v) + (ptrdiff_t)row0 * a.vrow};
     };
     u32x4 vr[VS][4];
     auto fetch = [&](const Tile& t, int buf) {
-        for (int i = wave; i < KT / RPC; i += kSeqWaves) {
-            const int r = i * RPC + lane / UN;
-            int u = (lane % UN) ^ swz_key<UN>(r);
-            if (u >= dunits) u = 0;
-            copy_to_lds16(t.k + (ptrdiff_t)min(t.k0 + r, t.hi - 1) * a.krow + u * 16, ks[buf] + i * 1024);
+        for (int i = wave; i < KT * NB / 1024; i += kSeqWaves) {
+            const int r = (i * 64 + lane) / UN, u = ((i * 64 + lane) % UN) ^ swz_key<UN>(r), key = min(t.k0 + r, t.hi - 1);
+            const char* src = t.k + (ptrdiff_t)key * a.krow + (u < dunits ? u : 0) * 16;
+            if (u >= dunits && u < dunits + a.runits) src = a.kr + (ptrdiff_t)key * a.rrow + (u - dunits) * 16;
+            copy_to_lds16(src, ks[buf] + i * 1024);
         }
         vt_request<T, KT, kSeqThreads, 0, VS>(vr, vunits, tid, [&](int key) { return t.v + (ptrdiff_t)min(t.k0 + key, t.hi - 1) * a.vrow; });
     };
@@ -536,16 +570,17 @@ __global__ __launch_bounds__(kSeqThreads, (NT <= 128 ? 2 : 1)) void k_seq_attn(S
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
         if (c0 + (wave * CT + ct) * 16 + col >= ncols) continue;
-        const float snk = a.sink[head[ct]] * kLog2e, m = fmaxf(st[ct].m, snk), c = fast_exp2(st[ct].m - m);
-        const float f = c / (st[ct].l * c + fast_exp2(snk - m));
+        const float snk = a.sink != nullptr ? a.sink[head[ct]] * kLog2e : kNegBig, m = fmaxf(st[ct].m, snk), c = fast_exp2(st[ct].m - m);
+        const float f = c / (st[ct].l * c + fast_exp2(snk - m));       // (no sink: the last term is zero)
         T* o = reinterpret_cast<T*>(a.out + (size_t)tok[ct] * a.ldo) + head[ct] * a.V;
+        const float* gate = a.gate + (size_t)tok[ct] * a.ldg + head[ct] * a.V;
 #pragma unroll
         for (int i = 0; i < NT / 16; ++i)
             if (i < a.vtiles) {
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
                     const int v = i * 16 + g * 4 + r;
-                    if (v < a.V) o[v] = from_f32<T>(st[ct].acc[i][r] * f);
+                    if (v < a.V) o[v] = from_f32<T>(a.gate != nullptr ? st[ct].acc[i][r] * f * sigmoid(gate[v]) : st[ct].acc[i][r] * f);
                 }
             }
     }
@@ -786,11 +821,11 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_attn_decode(SeqAttnDec a) {
 enum : int { kInVector = 0, kInNorm = 1, kInEmbed = 2 };
 struct SeqGemv {
     int input;
-    const float *x, *y;      // kInNorm: the residual row and the sublayer's output that is still to be added
-    float* x_out;            // ... where the new residual row goes (not x)
+    const float *x, *y;      // kInNorm: the residual row and the sublayer's output that is still to be added (nullable)
+    float* x_out;            // ... where the new residual row goes (not x); nullable
     float* copy;             // nullable: a second copy
     const float *nw, *nw2;   // norm weights; nw2 (nullable): a second norm follows
-    float alpha, eps;
+    float alpha, eps, noff;  // noff: the norms' weights are noff + nw
     int width;
     const char* embed;
     int embed_pitch;
@@ -808,7 +843,11 @@ struct SeqGemv {
     float* yf;
     char* yt;                // T; ROWS: a chosen matrix' outputs at multiples of seg_y bytes
     int seg_y;
-    float cap;
+    float mul, cap;          // kEpiHead
+    float* xs;               // kEpiStreams: the streams [streams][width], updated in place
+    const float *mix, *out, *in;          // ... in: of the next sublayer, null: all one
+    int streams;
+    float *u, *sum;          // ... its input before the norm; the sum of the streams (nullable)
     float* best_v;           // kEpiHead: best logit of every workgroup and its row
     int* best_i;
     int park, park_n;        // LDS: offset of the finished outputs, outputs per wave at most
@@ -916,7 +955,7 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
             const int k = min(tid + i * kSeqThreads, w4 - 1);
             if (w4 > 0) {
                 px[i] = x4[k];
-                py[i] = y4[k];
+                py[i] = p.y != nullptr ? y4[k] : f32x4{0.f, 0.f, 0.f, 0.f};
                 pn[i] = n4[k];
             }
         }
@@ -934,7 +973,7 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
         for (int i = tid + kPre * kSeqThreads; i < nunits; i += kSeqThreads) reinterpret_cast<u32x4*>(smem)[i] = input_unit(i);
     } else {
         for (int i = p.width + tid; i < nch * kGemvChunk / (int)sizeof(T); i += kSeqThreads) xs[i] = from_f32<T>(0.0f);
-        const bool keep = blockIdx.x == 0;
+        const bool keep = blockIdx.x == 0 && p.x_out != nullptr;
         if (p.input == kInEmbed) {
             const T* e = reinterpret_cast<const T*>(p.embed + (size_t)p.state[kStToken] * p.embed_pitch);
             for (int i = tid; i < p.width; i += kSeqThreads) {
@@ -957,9 +996,9 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
 #pragma unroll
             for (int i = 0; i < kPre; ++i)
                 if (tid + i * kSeqThreads < w4) sum4(tid + i * kSeqThreads, px[i], py[i]);
-            for (int i = tid + kPre * kSeqThreads; i < w4; i += kSeqThreads) sum4(i, x4[i], y4[i]);
+            for (int i = tid + kPre * kSeqThreads; i < w4; i += kSeqThreads) sum4(i, x4[i], p.y != nullptr ? y4[i] : f32x4{0.f, 0.f, 0.f, 0.f});
             for (int i = w4 * 4 + tid; i < p.width; i += kSeqThreads) {
-                const float t = fmadd(p.alpha, p.x[i], p.y[i]);
+                const float t = fmadd(p.alpha, p.x[i], p.y != nullptr ? p.y[i] : 0.0f);
                 ss = fmadd(t, t, ss);
                 ts[i] = t;
             }
@@ -976,17 +1015,17 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
             auto out4 = [&](int i, f32x4 w) {
                 const f32x4 t = reinterpret_cast<const f32x4*>(ts)[i];
 #pragma unroll
-                for (int j = 0; j < 4; ++j) out1(i * 4 + j, t[j] * inv * (1.0f + w[j]));
+                for (int j = 0; j < 4; ++j) out1(i * 4 + j, t[j] * inv * (p.noff + w[j]));
             };
 #pragma unroll
             for (int i = 0; i < kPre; ++i)
                 if (tid + i * kSeqThreads < w4) out4(tid + i * kSeqThreads, pn[i]);
             for (int i = tid + kPre * kSeqThreads; i < w4; i += kSeqThreads) out4(i, n4[i]);
-            for (int i = w4 * 4 + tid; i < p.width; i += kSeqThreads) out1(i, ts[i] * inv * (1.0f + p.nw[i]));
+            for (int i = w4 * 4 + tid; i < p.width; i += kSeqThreads) out1(i, ts[i] * inv * (p.noff + p.nw[i]));
             if (p.nw2 != nullptr) {
                 __syncthreads();
                 inv = inv_rms(block_sum(ss, red), p.width, p.eps);
-                for (int i = tid; i < p.width; i += kSeqThreads) xs[i] = from_f32<T>(ts[i] * inv * (1.0f + p.nw2[i]));
+                for (int i = tid; i < p.width; i += kSeqThreads) xs[i] = from_f32<T>(ts[i] * inv * (p.noff + p.nw2[i]));
             }
         }
     }
@@ -994,8 +1033,8 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
 
     // ---- the rows; finished outputs are parked in LDS and stored together at the end
     const int n_out = u1 - u0;
-    float* park = reinterpret_cast<float*>(smem + p.park) + wave * p.park_n;
-    float acc = 0.0f, gate = 0.0f;
+    float* park = reinterpret_cast<float*>(smem + p.park) + wave * p.park_n * UR;
+    float acc = 0.0f;
     int c_use = 0, r_use = 0, done = 0;                  // chunk and row of the output in work, outputs finished
     const float we = p.top > 0 ? 1.0f / (float)p.top : 1.0f;
     auto consume = [&](const u32x4 (&b)[kGemvLoads]) __attribute__((always_inline)) {
@@ -1011,11 +1050,10 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
                     c_use = 0;
                     const float v = wave_sum(acc);
                     acc = 0.0f;
+                    if (lane == 0) park[done * UR + r_use] = v;
                     if (UR == 2 && r_use == 0) {
-                        gate = v;
                         r_use = 1;
                     } else {
-                        if (lane == 0) park[done] = UR == 2 ? silu(gate) * v : v;
                         r_use = 0;
                         ++done;
                     }
@@ -1036,12 +1074,12 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
     float top_v = -INFINITY;
     int top_i = 0;
     for (int i = lane; i < n_out; i += kWave) {
-        const float v = park[i];
+        const float v = park[i * UR];
         const int u = u0 + i;
         if constexpr (EPI == kEpiF32) {
             p.yf[u] = p.bias != nullptr ? v + p.bias[u] : v;
         } else if constexpr (EPI == kEpiHead) {
-            const float z = soft_cap(v, p.cap);
+            const float z = soft_cap(v * p.mul, p.cap);
             p.yf[u] = z;
             if (z > top_v) {
                 top_v = z;
@@ -1049,9 +1087,28 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
             }
         } else if constexpr (EPI == kEpiRelu2) {
             reinterpret_cast<T*>(p.yt)[u] = from_f32<T>(relu2(v));
+        } else if constexpr (EPI == kEpiStreams) {
+            const float y = p.bias != nullptr ? v + p.bias[u] : v;
+            float o[CFPP_SEQ_MAX_STREAMS], next = 0.0f, all = 0.0f;
+#pragma unroll
+            for (int s = 0; s < CFPP_SEQ_MAX_STREAMS; ++s) o[s] = s < p.streams ? p.xs[(size_t)s * p.width + u] : 0.0f;
+#pragma unroll
+            for (int t = 0; t < CFPP_SEQ_MAX_STREAMS; ++t)
+                if (t < p.streams) {
+                    float z = p.out[t] * y;
+#pragma unroll
+                    for (int s = 0; s < CFPP_SEQ_MAX_STREAMS; ++s)
+                        if (s < p.streams) z = fmadd(p.mix[s * p.streams + t], o[s], z);
+                    p.xs[(size_t)t * p.width + u] = z;
+                    next = fmadd(p.in != nullptr ? p.in[t] : 1.0f, z, next);
+                    all += z;
+                }
+            p.u[u] = next;
+            if (p.sum != nullptr) p.sum[u] = all;
         } else {
             const int b = u < p.top * p.units_e ? u / p.units_e : p.top;
-            reinterpret_cast<T*>(p.yt + (size_t)b * p.seg_y)[u - b * p.units_e] = from_f32<T>(v);
+            const float bg = p.bias != nullptr ? p.bias[2 * u] : 0.0f, bu = p.bias != nullptr ? p.bias[2 * u + 1] : 0.0f;
+            reinterpret_cast<T*>(p.yt + (size_t)b * p.seg_y)[u - b * p.units_e] = from_f32<T>(silu(v + bg) * (park[i * UR + 1] + bu));
         }
     }
     if constexpr (EPI == kEpiHead) {
@@ -1112,12 +1169,12 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_pick(const float* best_v, c
     }
 }
 
-// angle = position * base^(-2i / dims), evaluated in double and rounded once
-__global__ void k_seq_rope_table(float2* t, const double* freq, int half, int positions) {
+// angle = position * frequency, evaluated in double; cos and sin times `mul`, rounded once
+__global__ void k_seq_rope_table(float2* t, const double* freq, double mul, int half, int positions) {
     const size_t n = (size_t)positions * half;
     for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
         const double a = (double)(i / half) * freq[i % half];
-        t[i] = make_float2((float)cos(a), (float)sin(a));
+        t[i] = make_float2((float)(mul * cos(a)), (float)(mul * sin(a)));
     }
 }
 
@@ -1134,6 +1191,12 @@ struct LayerPlan {
     float2* cs;
     char *kc, *vc;
     int ns;
+    // latent mixers: the cache rows are kc's, in bytes
+    bool latent, own;
+    int lpitch, crow;        // latent part (a padded weight row), whole cache row
+    int plain, shared, qrow; // plain and rotated part of a key, whole query row
+    int rp;                  // latent columns of the partial results of a decode step
+    int gate_at;             // first gate row of the projection
     int route;               // index among the layers with table experts, -1: none
 };
 
@@ -1158,6 +1221,7 @@ struct cfpp_seq {
     int* state;
     int *history, *cnt, *best_i;
     float *dx[2], *dy, *dres, *logits, *part, *best_v;
+    float *du;               // residual streams: the next sublayer's input before its norm
     int history_cap, pos = 0, launches = 0, head_grid = 0;
     hipGraphExec_t graph = nullptr;
     hipStream_t capture = nullptr;
@@ -1220,13 +1284,22 @@ void expert_gemm(const cfpp_seq* s, const LayerPlan& L, SeqGemm g, int n, hipStr
     launch_gemm<T, EPI>(g, slots / bt + std::min(L.d.experts, slots), bt == 128, st);
 }
 
-template <typename T, int NT>
+template <typename T, int NK, int NT>
 void launch_attn(const SeqAttn& a, int G, int cus, hipStream_t st) {
     const int cols = a.T * a.R;
     if (ceil_div(cols, 128) * G >= 2 * cus)
-        hipLaunchKernelGGL((k_seq_attn<T, NT, 2>), dim3(ceil_div(cols, 128), G), dim3(kSeqThreads), 0, st, a);
+        hipLaunchKernelGGL((k_seq_attn<T, NK, NT, 2>), dim3(ceil_div(cols, 128), G), dim3(kSeqThreads), 0, st, a);
     else
-        hipLaunchKernelGGL((k_seq_attn<T, NT, 1>), dim3(ceil_div(cols, 64), G), dim3(kSeqThreads), 0, st, a);
+        hipLaunchKernelGGL((k_seq_attn<T, NK, NT, 1>), dim3(ceil_div(cols, 64), G), dim3(kSeqThreads), 0, st, a);
+}
+
+template <typename T>
+void attn(const cfpp_seq* s, const SeqAttn& a, int G, hipStream_t st) {
+    const int nk = a.qrow / (int)sizeof(T), nv = a.vtiles * 16;
+    if (nk <= 64 && nv <= 64) launch_attn<T, 64, 64>(a, G, s->cus, st);
+    else if (nk <= 128 && nv <= 128) launch_attn<T, 128, 128>(a, G, s->cus, st);
+    else if (nk <= 192 && nv <= 128) launch_attn<T, 192, 128>(a, G, s->cus, st);
+    else launch_attn<T, 256, 256>(a, G, s->cus, st);
 }
 
 template <typename T>
@@ -1236,11 +1309,151 @@ void postnorm(const cfpp_seq* s, const SeqPostNorm& n, int rows, hipStream_t st)
     hipLaunchKernelGGL(k_seq_postnorm<T>, dim3(rows), dim3(kSeqThreads), lds, st, n);
 }
 
+template <typename T>
+void streams(const cfpp_seq* s, SeqStreams a, int rows, hipStream_t st) {
+    const size_t lds = (size_t)s->d.width * 4;
+    a.streams = s->d.streams;
+    a.width = s->d.width;
+    a.pitch = s->xpitch;
+    a.eps = s->d.eps;
+    a.noff = s->d.norm_offset;
+    auto go = [&](auto n) {
+        constexpr int S = decltype(n)::value;
+        allow_lds(k_seq_streams<T, S>, lds);
+        hipLaunchKernelGGL((k_seq_streams<T, S>), dim3(rows), dim3(kSeqThreads), lds, st, a);
+    };
+    if (a.streams == 1) go(std::integral_constant<int, 1>{});
+    else if (a.streams == 2) go(std::integral_constant<int, 2>{});
+    else if (a.streams <= 4) go(std::integral_constant<int, 4>{});
+    else go(std::integral_constant<int, CFPP_SEQ_MAX_STREAMS>{});
+}
+
+// What reads the sum after sublayer `q` (0: mixer, 1: feed-forward) of layer `li`; both null after the last one.
+struct NextInput { const float *norm, *in; };
+NextInput next_input(const cfpp_seq* s, size_t li, int q) {
+    const cfpp_seq_layer& d = s->layers[li].d;
+    if (q == 0 && d.ff_kind != CFPP_SEQ_FF_NONE) return {d.norm2, d.hc2.in};
+    if (li + 1 < s->layers.size()) return {s->layers[li + 1].d.norm1, s->layers[li + 1].d.hc1.in};
+    return {nullptr, nullptr};
+}
+
+// The mixer of a portion, from s->xb to s->y.
+template <typename T>
+void portion_grouped(cfpp_seq* s, const LayerPlan& L, int slot, int n, int pos, hipStream_t st) {
+    const cfpp_seq_layer& d = L.d;
+    const int cap = s->portion;
+    SeqQkv f{s->qkv, s->ld_qkv, d.q_norm, d.k_norm, L.cs, s->d.eps, d.v_lambda, d.heads, d.kv_heads, d.dim, L.Dp, d.vdim, L.Vp,
+             d.rot_dims, pos, cap, L.v_role, s->v_first, s->q, s->k, s->v};
+    hipLaunchKernelGGL(k_seq_qkv_finish<T>, dim3(n), dim3(kSeqThreads), 0, st, f);
+
+    char* kc = L.kc + (size_t)slot * d.kv_heads * L.rows * L.krow;
+    char* vc = L.vc + (size_t)slot * d.kv_heads * L.rows * L.vrow;
+    SeqAttn a{};
+    a.q = s->q;
+    a.k = s->k;
+    a.v = s->v;
+    a.kc = kc;
+    a.vc = vc;
+    a.out = s->o;
+    a.sink = d.sink;
+    a.T = n;
+    a.H = d.heads;
+    a.R = L.R;
+    a.dsteps = L.krow / 64;
+    a.qrow = a.krow = L.krow;
+    a.vrow = L.vrow;
+    a.V = d.vdim;
+    a.vtiles = L.Vp / 16;
+    a.pos0 = a.k_split = pos;
+    a.chunk = d.chunk;
+    a.cap = cap;
+    a.rows = L.rows;
+    a.ldo = (int)pitch_of(d.heads * d.vdim, s->esize);
+    a.scale_log2 = d.scale * kLog2e;
+    attn<T>(s, a, d.kv_heads, st);
+
+    const int last = pos + n - 1, cs0 = d.chunk > 0 ? last / d.chunk * d.chunk : 0, first = std::max(pos, cs0) - pos;
+    SeqAppend ap{s->k, s->v, kc, vc, d.kv_heads, L.krow, L.vrow, cap, L.rows, first, pos + first - cs0};
+    hipLaunchKernelGGL(k_seq_append, dim3(n - first), dim3(kSeqThreads), 0, st, ap);
+}
+
+template <typename T>
+LatentRow latent_row_of(const cfpp_seq* s, const LayerPlan& L) {
+    return LatentRow{L.d.kv_norm, L.d.kv_rank, L.d.rot_dims, L.lpitch, L.crow, L.d.rot_half, s->d.eps};
+}
+
+template <typename T>
+void portion_latent(cfpp_seq* s, const LayerPlan& L, int slot, int n, int pos, hipStream_t st) {
+    const cfpp_seq_layer& d = L.d;
+    char* kc = L.kc + (size_t)slot * s->d.capacity * L.crow;
+    SeqLatentFinish f{s->qkv, s->ld_qkv, L.own, latent_row_of<T>(s, L), L.cs, d.heads, d.dim, d.rot_dims, pos, L.plain, L.qrow, s->q, kc};
+    hipLaunchKernelGGL(k_seq_latent_finish<T>, dim3(n), dim3(kSeqThreads), 0, st, f);
+
+    const int ctx = pos + n, cap = s->d.capacity;
+    SeqGemm g{};
+    g.w = (const char*)d.w_ukv;
+    g.a = kc;
+    g.n = d.heads * (d.dim + d.vdim);
+    g.m = ctx;
+    g.kbytes = L.lpitch;
+    g.lda = L.crow;
+    g.yt = s->k;
+    g.yv = s->v;
+    g.nk = d.heads * d.dim;
+    g.kd = d.dim;
+    g.kp = L.plain;
+    g.kh = (size_t)cap * L.plain;
+    g.vd = d.vdim;
+    g.vp = L.vrow;
+    g.vh = (size_t)cap * L.vrow;
+    gemm<T, kEpiHeads>(s, g, st);
+
+    SeqAttn a{};
+    a.q = s->q;
+    a.k = s->k;
+    a.v = s->v;
+    a.kr = kc + L.lpitch;
+    a.out = s->o;
+    a.sink = d.sink;
+    a.gate = d.gated ? s->qkv + L.gate_at : nullptr;
+    a.ldg = s->ld_qkv;
+    a.T = n;
+    a.H = d.heads;
+    a.R = 1;
+    a.dsteps = L.qrow / 64;
+    a.qrow = L.qrow;
+    a.krow = L.plain;
+    a.runits = L.shared / 16;
+    a.rrow = L.crow;
+    a.vrow = L.vrow;
+    a.V = d.vdim;
+    a.vtiles = L.Vp / 16;
+    a.pos0 = pos;
+    a.cap = cap;
+    a.ldo = (int)pitch_of(d.heads * d.vdim, s->esize);
+    a.scale_log2 = d.scale * kLog2e;
+    attn<T>(s, a, d.heads, st);
+}
+
 // One portion: n tokens (device, s->tokens) at positions pos .. pos + n - 1.  want: device places (n_want of them), logits rows.
 template <typename T>
 int run_portion(cfpp_seq* s, int slot, int n, int pos, int n_want, float* logits, float* residuals, size_t residual_stride, hipStream_t st) {
     const int width = s->d.width, xp = s->xpitch;
-    hipLaunchKernelGGL(k_seq_embed<T>, dim3(n), dim3(kSeqThreads), 0, st, s->tokens, (const char*)s->d.embed, xp, width, s->x, s->xb);
+    if (s->d.streams > 0) {
+        SeqStreams e{};
+        e.x = s->x;
+        e.in = s->layers[0].d.hc1.in;
+        e.w = s->layers[0].d.norm1;
+        e.xb = s->xb;
+        e.tokens = s->tokens;
+        e.embed = (const char*)s->d.embed;
+        e.pos = (const char*)s->d.pos;
+        e.embed_pitch = xp;
+        e.pos0 = pos;
+        streams<T>(s, e, n, st);
+    } else {
+        hipLaunchKernelGGL(k_seq_embed<T>, dim3(n), dim3(kSeqThreads), 0, st, s->tokens, (const char*)s->d.embed, xp, width, s->x, s->xb);
+    }
     if (!s->host_routes.empty()) {
         // (one tile size for every layer of the launch: the layers share it when they share top and the expert count)
         for (size_t i = 0; i < s->layers.size(); ++i) {
@@ -1274,68 +1487,88 @@ int run_portion(cfpp_seq* s, int slot, int n, int pos, int n_want, float* logits
         g.ldy = s->ld_qkv;
         gemm<T, kEpiF32>(s, g, st);
 
-        const int cap = s->portion;
-        SeqQkv f{s->qkv, s->ld_qkv, d.q_norm, d.k_norm, L.cs, s->d.eps, d.v_lambda, d.heads, d.kv_heads, d.dim, L.Dp, d.vdim, L.Vp,
-                 d.rot_dims, pos, cap, L.v_role, s->v_first, s->q, s->k, s->v};
-        hipLaunchKernelGGL(k_seq_qkv_finish<T>, dim3(n), dim3(kSeqThreads), 0, st, f);
-
-        char* kc = L.kc + (size_t)slot * d.kv_heads * L.rows * L.krow;
-        char* vc = L.vc + (size_t)slot * d.kv_heads * L.rows * L.vrow;
-        const int op = (int)pitch_of(d.heads * d.vdim, s->esize);
-        SeqAttn a{s->q, s->k, s->v, kc, vc, s->o, d.sink, n, d.heads, L.R, L.krow / 64, L.krow, L.vrow, d.vdim, L.Vp / 16, pos, d.chunk, cap,
-                  L.rows, op, d.scale * kLog2e};
-        if (L.NT == 64) launch_attn<T, 64>(a, d.kv_heads, s->cus, st);
-        else if (L.NT == 128) launch_attn<T, 128>(a, d.kv_heads, s->cus, st);
-        else launch_attn<T, 256>(a, d.kv_heads, s->cus, st);
-
-        const int last = pos + n - 1, cs0 = d.chunk > 0 ? last / d.chunk * d.chunk : 0, first = std::max(pos, cs0) - pos;
-        SeqAppend ap{s->k, s->v, kc, vc, d.kv_heads, L.krow, L.vrow, cap, L.rows, first, pos + first - cs0};
-        hipLaunchKernelGGL(k_seq_append, dim3(n - first), dim3(kSeqThreads), 0, st, ap);
+        if (L.latent) portion_latent<T>(s, L, slot, n, pos, st);
+        else portion_grouped<T>(s, L, slot, n, pos, st);
 
         g = SeqGemm{};
         g.w = (const char*)d.w_o;
         g.a = s->o;
         g.n = width;
         g.m = n;
-        g.kbytes = g.lda = op;
+        g.kbytes = g.lda = (int)pitch_of(d.heads * d.vdim, s->esize);
         g.yf = s->y;
         g.ldy = width;
         gemm<T, kEpiF32>(s, g, st);
-        SeqPostNorm pn{};
-        pn.x = pn.x_out = s->x;
-        pn.y = s->y;
-        pn.w = d.norm1;
-        pn.alpha = s->d.alpha;
-        pn.eps = s->d.eps;
-        pn.width = width;
-        pn.xb = s->xb;
-        pn.pitch = xp;
-        pn.copy = d.ff_kind == CFPP_SEQ_FF_NONE ? copy : nullptr;
-        postnorm<T>(s, pn, n, st);
+        // the residual sum of a sublayer: y (nullable) and the chosen experts' outputs (`top` 0: none)
+        auto close = [&](int q, const float* y, int top) {
+            float* c = q == 1 || d.ff_kind == CFPP_SEQ_FF_NONE ? copy : nullptr;
+            const float* ys = top > 0 ? s->ys : nullptr;
+            const float share = top > 0 ? 1.0f / (float)top : 0.0f;
+            if (s->d.streams > 0) {
+                const cfpp_seq_streams& hc = q == 0 ? d.hc1 : d.hc2;
+                const NextInput next = next_input(s, li, q);
+                SeqStreams a{};
+                a.x = s->x;
+                a.y = y;
+                a.ys = ys;
+                a.top = top;
+                a.slot_weight = share;
+                a.mix = hc.mix;
+                a.out = hc.out;
+                a.in = next.in;
+                a.w = next.norm;
+                a.xb = s->xb;
+                a.copy = c;
+                streams<T>(s, a, n, st);
+            } else {
+                SeqPostNorm pn{};
+                pn.x = pn.x_out = s->x;
+                pn.y = y;
+                pn.ys = ys;
+                pn.top = top;
+                pn.slot_weight = share;
+                pn.w = q == 0 ? d.norm1 : d.norm2;
+                pn.alpha = s->d.alpha;
+                pn.eps = s->d.eps;
+                pn.noff = s->d.norm_offset;
+                pn.width = width;
+                pn.xb = s->xb;
+                pn.pitch = xp;
+                pn.copy = c;
+                postnorm<T>(s, pn, n, st);
+            }
+        };
+        close(0, s->y, 0);
         if (d.ff_kind == CFPP_SEQ_FF_NONE) continue;
-        pn.w = d.norm2;
-        pn.copy = copy;
 
-        if (d.ff_kind == CFPP_SEQ_FF_RELU2) {
+        if (d.ff_kind != CFPP_SEQ_FF_TABLE_EXPERTS) {
             const int hp = (int)pitch_of(d.ff, s->esize);
             g = SeqGemm{};
             g.w = (const char*)d.w_up;
             g.a = s->xb;
-            g.n = d.ff;
             g.m = n;
             g.kbytes = g.lda = xp;
             g.yt = s->h;
             g.ldyt = hp;
-            gemm<T, kEpiRelu2>(s, g, st);
+            if (d.ff_kind == CFPP_SEQ_FF_RELU2) {
+                g.n = d.ff;
+                gemm<T, kEpiRelu2>(s, g, st);
+            } else {
+                g.n = 2 * d.ff;
+                g.bias = d.b_up;
+                gemm<T, kEpiGated>(s, g, st);
+            }
             g = SeqGemm{};
             g.w = (const char*)d.w_down;
             g.a = s->h;
             g.n = width;
             g.m = n;
             g.kbytes = g.lda = hp;
+            g.bias = d.b_down;
             g.yf = s->y;
             g.ldy = width;
             gemm<T, kEpiF32>(s, g, st);
+            close(1, s->y, 0);
         } else {
             const int hp = (int)pitch_of(d.ff, s->esize);
             g = SeqGemm{};
@@ -1358,10 +1591,6 @@ int run_portion(cfpp_seq* s, int slot, int n, int pos, int n_want, float* logits
             g.ldy = width;
             g.slot_div = 1;
             expert_gemm<T, kEpiF32>(s, L, g, n, st);
-            pn.ys = s->ys;
-            pn.top = d.top;
-            pn.slot_weight = 1.0f / (float)d.top;
-            pn.y = nullptr;
             if (d.shared_ff > 0) {
                 const int sp = (int)pitch_of(d.shared_ff, s->esize);
                 g = SeqGemm{};
@@ -1382,21 +1611,30 @@ int run_portion(cfpp_seq* s, int slot, int n, int pos, int n_want, float* logits
                 g.yf = s->y;
                 g.ldy = width;
                 gemm<T, kEpiF32>(s, g, st);
-                pn.y = s->y;
             }
+            close(1, d.shared_ff > 0 ? s->y : nullptr, d.top);
         }
-        postnorm<T>(s, pn, n, st);
     }
     if (n_want > 0) {
-        SeqPostNorm pn{};
-        pn.x = s->x;
-        pn.w = s->d.final_norm;
-        pn.eps = s->d.eps;
-        pn.width = width;
-        pn.xb = s->wb;
-        pn.pitch = xp;
-        pn.rows = s->want;
-        postnorm<T>(s, pn, n_want, st);
+        if (s->d.streams > 0) {
+            SeqStreams a{};
+            a.x = s->x;
+            a.w = s->d.final_norm;
+            a.xb = s->wb;
+            a.rows = s->want;
+            streams<T>(s, a, n_want, st);
+        } else {
+            SeqPostNorm pn{};
+            pn.x = s->x;
+            pn.w = s->d.final_norm;
+            pn.eps = s->d.eps;
+            pn.noff = s->d.norm_offset;
+            pn.width = width;
+            pn.xb = s->wb;
+            pn.pitch = xp;
+            pn.rows = s->want;
+            postnorm<T>(s, pn, n_want, st);
+        }
         SeqGemm g{};
         g.w = (const char*)s->d.head;
         g.a = s->wb;
@@ -1405,6 +1643,7 @@ int run_portion(cfpp_seq* s, int slot, int n, int pos, int n_want, float* logits
         g.kbytes = g.lda = xp;
         g.yf = logits;
         g.ldy = s->d.vocab;
+        g.mul = s->d.logit_scale;
         g.cap = s->d.softcap;
         gemm<T, kEpiHead>(s, g, st);
     }
@@ -1420,7 +1659,7 @@ int gemv(const cfpp_seq* s, SeqGemv p, hipStream_t st) {
     const int grid = std::max(1, std::min(kGemvWgs * s->cus, ceil_div(total, kSeqWaves)));
     p.park = nch * kGemvChunk + (p.input == kInNorm ? up_to(p.width * 4, 16) : 0);
     p.park_n = ceil_div(total, grid * kSeqWaves);
-    const size_t lds = (size_t)p.park + (size_t)p.park_n * kSeqWaves * 4;
+    const size_t lds = (size_t)p.park + (size_t)p.park_n * (EPI == kEpiGated ? 2 : 1) * kSeqWaves * 4;
     allow_lds(k_seq_gemv<T, EPI, KCAT>, lds);
     hipLaunchKernelGGL((k_seq_gemv<T, EPI, KCAT>), dim3(grid), dim3(kSeqThreads), lds, st, p);
     return grid;
@@ -1431,17 +1670,78 @@ void launch_attn_decode(const SeqAttnDec& a, hipStream_t st) {
     hipLaunchKernelGGL((k_seq_attn_decode<T, NT>), dim3(a.ns, a.G * a.nct), dim3(kSeqThreads), 0, st, a);
 }
 
+// The mixer of one token between its projection (s->qkv) and its output rows (s->o); the number of launches.
+template <typename T>
+int step_grouped(cfpp_seq* s, const LayerPlan& L, hipStream_t st) {
+    const cfpp_seq_layer& d = L.d;
+    SeqAttnDec a{s->qkv, d.q_norm, d.k_norm, d.sink, L.cs, s->state, L.kc, L.vc, (size_t)d.kv_heads * L.rows * L.krow,
+                 (size_t)d.kv_heads * L.rows * L.vrow, s->v_first, s->o, s->part, s->cnt, s->d.eps, d.v_lambda, d.scale * kLog2e, L.v_role,
+                 d.heads, d.kv_heads, L.R, L.nct, d.dim, d.vdim, d.rot_dims, d.chunk, L.krow, L.vrow, L.krow / 64, L.Vp / 16, L.rows, L.ns};
+    if (L.NT == 64) launch_attn_decode<T, 64>(a, st);
+    else if (L.NT == 128) launch_attn_decode<T, 128>(a, st);
+    else launch_attn_decode<T, 256>(a, st);
+    return 1;
+}
+
+// sets of 16 heads of a workgroup of k_seq_latent_attn
+int latent_sets(int heads) { return heads <= 16 ? 1 : heads <= 32 ? 2 : 4; }
+
+template <typename T, int NR>
+void launch_latent_attn(const SeqLatentAttn& a, hipStream_t st) {
+    const int sets = latent_sets(a.H);
+    const size_t lds = 2 * (size_t)a.tile_bytes;
+    const dim3 grid(a.ns, ceil_div(a.H, 16 * sets));
+    auto go = [&](auto n) {
+        constexpr int RW = decltype(n)::value;
+        allow_lds(k_seq_latent_attn<T, NR, RW>, lds);
+        hipLaunchKernelGGL((k_seq_latent_attn<T, NR, RW>), grid, dim3(kSeqThreads), lds, st, a);
+    };
+    if (sets == 1) go(std::integral_constant<int, 4>{});
+    else if (sets == 2) go(std::integral_constant<int, 2>{});
+    else go(std::integral_constant<int, 1>{});
+}
+
+template <typename T>
+int step_latent(cfpp_seq* s, const LayerPlan& L, hipStream_t st) {
+    const cfpp_seq_layer& d = L.d;
+    const size_t slot = (size_t)s->d.capacity * L.crow;
+    SeqLatentQ q{s->qkv, s->state, L.cs, (const char*)d.w_ukv, L.lpitch, d.heads, d.dim, d.rot_dims, L.lpitch / 128, L.own, latent_row_of<T>(s, L),
+                 s->q, L.kc, slot};
+    hipLaunchKernelGGL(k_seq_latent_q<T>, dim3(d.heads * q.nrb + (L.own ? 1 : 0)), dim3(kSeqThreads), 0, st, q);
+
+    float* ml = s->part + (size_t)L.ns * d.heads * L.rp;
+    const int tile = up_to(LatentTile<T>::keys * ((L.crow / 16) | 1) * 16, 1024);
+    SeqLatentAttn a{s->q, L.kc, slot, s->state, s->part, ml, d.scale * kLog2e, d.heads, L.crow, L.ns, L.rp, tile};
+    if (L.rp <= 128) launch_latent_attn<T, 128>(a, st);
+    else launch_latent_attn<T, 512>(a, st);
+
+    SeqLatentOut o{s->part, ml, s->state, d.sink, d.gated ? s->qkv + L.gate_at : nullptr, (const char*)d.w_ukv + (size_t)d.heads * d.dim * L.lpitch, s->o,
+                   d.heads, d.vdim, L.lpitch, L.ns, L.rp};
+    hipLaunchKernelGGL(k_seq_latent_out<T>, dim3(ceil_div(d.vdim, kLatentOut), d.heads), dim3(kSeqThreads), 0, st, o);
+    return 3;
+}
+
 // Enqueues one step for the device-side state.  pick: also choose the next token.
 template <typename T>
 int run_step(cfpp_seq* s, bool head, bool pick, float* residuals, hipStream_t st) {
     const int width = s->d.width, xp = s->xpitch;
+    const bool multi = s->d.streams > 0;
     int cur = 0, launches = 0;             // dx[cur]: the residual row before the sum that is still pending
     const float* pending = nullptr;        // norm weight of that sum
     float* pending_copy = nullptr;
-    auto input = [&](SeqGemv& p) {
+    // The input of a sublayer: the streams' weighted sum and its norm, or the pending residual sum and its norm.
+    auto input = [&](SeqGemv& p, const float* norm) {
         p.state = s->state;
         p.width = width;
         p.eps = s->d.eps;
+        p.noff = s->d.norm_offset;
+        if (multi) {
+            p.input = kInNorm;
+            p.x = s->du;
+            p.alpha = 1.0f;
+            p.nw = norm;
+            return;
+        }
         p.alpha = s->d.alpha;
         if (pending == nullptr) {
             p.input = kInEmbed;
@@ -1459,44 +1759,74 @@ int run_step(cfpp_seq* s, bool head, bool pick, float* residuals, hipStream_t st
         }
         pending_copy = nullptr;
     };
+    // The rows that end sublayer `q`: into the streams, or to dy for the sum that the next launch makes.
+    auto output = [&](SeqGemv& p, size_t li, int q, float* copy) {
+        const cfpp_seq_layer& d = s->layers[li].d;
+        p.units_s = width;
+        if (multi) {
+            const cfpp_seq_streams& hc = q == 0 ? d.hc1 : d.hc2;
+            p.width = width;
+            p.xs = s->dx[0];
+            p.mix = hc.mix;
+            p.out = hc.out;
+            p.in = next_input(s, li, q).in;
+            p.streams = s->d.streams;
+            p.u = s->du;
+            p.sum = copy;
+            gemv<T, kEpiStreams, true>(s, p, st);
+        } else {
+            p.yf = s->dy;
+            gemv<T, kEpiF32, true>(s, p, st);
+            pending = q == 0 ? d.norm1 : d.norm2;
+            pending_copy = copy;
+        }
+    };
+    if (multi) {
+        SeqStreams e{};
+        e.x = s->dx[0];
+        e.in = s->layers[0].d.hc1.in;
+        e.w = s->layers[0].d.norm1;
+        e.xb = s->xb;
+        e.tokens = s->state + kStToken;
+        e.state = s->state;
+        e.embed = (const char*)s->d.embed;
+        e.pos = (const char*)s->d.pos;
+        e.embed_pitch = xp;
+        streams<T>(s, e, 1, st);
+        ++launches;
+    }
     for (size_t li = 0; li < s->layers.size(); ++li) {
         const LayerPlan& L = s->layers[li];
         const cfpp_seq_layer& d = L.d;
         float* copy = residuals != nullptr ? residuals + li * width : nullptr;
         SeqGemv p{};
-        input(p);
         p.w_s = (const char*)d.w_qkv;
         p.pitch_s = xp;
         p.units_s = L.n_qkv;
         p.bias = d.b_qkv;
         p.yf = s->qkv;
-        gemv<T, kEpiF32, false>(s, p, st);
-
-        SeqAttnDec a{s->qkv, d.q_norm, d.k_norm, d.sink, L.cs, s->state, L.kc, L.vc, (size_t)d.kv_heads * L.rows * L.krow,
-                     (size_t)d.kv_heads * L.rows * L.vrow, s->v_first, s->o, s->part, s->cnt, s->d.eps, d.v_lambda, d.scale * kLog2e, L.v_role,
-                     d.heads, d.kv_heads, L.R, L.nct, d.dim, d.vdim, d.rot_dims, d.chunk, L.krow, L.vrow, L.krow / 64, L.Vp / 16, L.rows, L.ns};
-        if (L.NT == 64) launch_attn_decode<T, 64>(a, st);
-        else if (L.NT == 128) launch_attn_decode<T, 128>(a, st);
-        else launch_attn_decode<T, 256>(a, st);
+        if (multi && li == 0) {
+            p.input = kInVector;
+            p.xin = s->xb;
+            gemv<T, kEpiF32, true>(s, p, st);
+        } else {
+            input(p, d.norm1);
+            gemv<T, kEpiF32, false>(s, p, st);
+        }
+        launches += L.latent ? step_latent<T>(s, L, st) : step_grouped<T>(s, L, st);
 
         p = SeqGemv{};
         p.input = kInVector;
         p.xin = s->o;
         p.w_s = (const char*)d.w_o;
         p.pitch_s = (int)pitch_of(d.heads * d.vdim, s->esize);
-        p.units_s = width;
-        p.yf = s->dy;
-        gemv<T, kEpiF32, true>(s, p, st);
-        launches += 3;
-        pending = d.norm1;
-        if (d.ff_kind == CFPP_SEQ_FF_NONE) {
-            pending_copy = copy;
-            continue;
-        }
+        output(p, li, 0, d.ff_kind == CFPP_SEQ_FF_NONE ? copy : nullptr);
+        launches += 2;
+        if (d.ff_kind == CFPP_SEQ_FF_NONE) continue;
         const bool moe = d.ff_kind == CFPP_SEQ_FF_TABLE_EXPERTS;
         const int hp = (int)pitch_of(d.ff, s->esize), sp = moe ? (int)pitch_of(d.shared_ff, s->esize) : hp;
         p = SeqGemv{};
-        input(p);
+        input(p, d.norm2);
         p.yt = s->h;
         p.seg_y = hp;
         p.pitch_s = xp;
@@ -1513,15 +1843,15 @@ int run_step(cfpp_seq* s, bool head, bool pick, float* residuals, hipStream_t st
         } else {
             p.w_s = (const char*)d.w_up;
             p.units_s = d.ff;
-            gemv<T, kEpiRelu2, false>(s, p, st);
+            p.bias = d.b_up;
+            if (d.ff_kind == CFPP_SEQ_FF_GATED) gemv<T, kEpiGated, false>(s, p, st);
+            else gemv<T, kEpiRelu2, false>(s, p, st);
         }
         p = SeqGemv{};
         p.input = kInVector;
         p.state = s->state;
         p.xin = s->h;
         p.seg_e = hp;
-        p.units_s = width;
-        p.yf = s->dy;
         if (moe) {
             p.table = d.table;
             p.top = d.top;
@@ -1533,20 +1863,20 @@ int run_step(cfpp_seq* s, bool head, bool pick, float* residuals, hipStream_t st
         } else {
             p.w_s = (const char*)d.w_down;
             p.pitch_s = hp;
+            p.bias = d.b_down;
         }
-        gemv<T, kEpiF32, true>(s, p, st);
+        output(p, li, 1, copy);
         launches += 2;
-        pending = d.norm2;
-        pending_copy = copy;
     }
-    if (head || residuals != nullptr) {
+    if (head || (residuals != nullptr && !multi)) {
         SeqGemv p{};
-        input(p);
-        p.nw2 = s->d.final_norm;
+        input(p, s->d.final_norm);
+        if (!multi) p.nw2 = s->d.final_norm;
         p.w_s = (const char*)s->d.head;
         p.pitch_s = xp;
         p.units_s = s->d.vocab;
         p.yf = s->logits;
+        p.mul = s->d.logit_scale;
         p.cap = s->d.softcap;
         p.best_v = s->best_v;
         p.best_i = s->best_i;
@@ -1565,17 +1895,39 @@ int step(cfpp_seq* s, bool head, bool pick, float* residuals, hipStream_t st) {
     return s->d.dtype == CFPP_SEQ_BF16 ? run_step<bf16_t>(s, head, pick, residuals, st) : run_step<float>(s, head, pick, residuals, st);
 }
 
-int check_layer(const cfpp_seq_desc& D, const cfpp_seq_layer& d, int esize) {
-    if (d.heads < 1 || d.kv_heads < 1 || d.heads % d.kv_heads || d.dim < 1 || d.vdim < 1 || d.dim > 256 || d.vdim > 256 || d.chunk < 0)
-        return CFPP_ERR_DIMS;
-    if (d.rot_dims < 0 || d.rot_dims > d.dim || d.rot_dims % 2) return CFPP_ERR_DIMS;
-    const void* need[] = {d.w_qkv, d.b_qkv, d.q_norm, d.k_norm, d.sink, d.w_o, d.norm1};
-    for (const void* p : need)
-        if (p == nullptr) return CFPP_ERR_NULL;
-    if (d.ff_kind < CFPP_SEQ_FF_NONE || d.ff_kind > CFPP_SEQ_FF_TABLE_EXPERTS) return CFPP_ERR_MODE;
+bool connected(const cfpp_seq_streams& c) { return c.in != nullptr && c.mix != nullptr && c.out != nullptr; }
+
+int check_mixer(const cfpp_seq_desc& D, int li, int esize) {
+    const cfpp_seq_layer& d = D.layers[li];
+    if (d.heads < 1 || d.dim < 1 || d.vdim < 1 || d.dim > 256 || d.vdim > 256 || d.rot_dims < 0 || d.rot_dims % 2) return CFPP_ERR_DIMS;
+    if (d.rot_factor != 0.0 && !(d.rot_factor > 0.0 && d.rot_original > 0.0 && d.rot_fast > 0.0 && d.rot_slow > 0.0 && d.rot_base > 1.0)) return CFPP_ERR_DIMS;
+    if (d.rot_dims > 0 && !(d.rot_base > 0.0)) return CFPP_ERR_DIMS;
+    if (d.w_qkv == nullptr || d.w_o == nullptr || d.norm1 == nullptr) return CFPP_ERR_NULL;
+    if (D.streams > 0 && !connected(d.hc1)) return CFPP_ERR_NULL;
+    if (d.mixer == CFPP_SEQ_MIX_GROUPED) {
+        if (d.kv_heads < 1 || d.heads % d.kv_heads || d.chunk < 0 || d.rot_dims > d.dim) return CFPP_ERR_DIMS;
+        if (d.rot_half || d.gated) return CFPP_ERR_MODE;
+        if (d.b_qkv == nullptr || d.q_norm == nullptr || d.k_norm == nullptr || d.sink == nullptr) return CFPP_ERR_NULL;
+        return CFPP_OK;
+    }
+    if (d.mixer != CFPP_SEQ_MIX_LATENT || d.v_mix || d.chunk != 0) return CFPP_ERR_MODE;
+    if (d.heads > 4096 || d.kv_rank < 1 || d.kv_rank > 512 || d.rot_dims > 128 || up_to(d.dim * esize, 16) + up_to(d.rot_dims * esize, 16) > 256 * esize) return CFPP_ERR_DIMS;
+    if (d.w_ukv == nullptr) return CFPP_ERR_NULL;
+    if (d.kv_from < 0) return d.kv_norm != nullptr ? CFPP_OK : CFPP_ERR_NULL;
+    if (d.kv_from >= li) return CFPP_ERR_DIMS;
+    const cfpp_seq_layer& o = D.layers[d.kv_from];
+    return o.mixer == CFPP_SEQ_MIX_LATENT && o.kv_from < 0 && o.kv_rank == d.kv_rank && o.rot_dims == d.rot_dims ? CFPP_OK : CFPP_ERR_DIMS;
+}
+
+int check_layer(const cfpp_seq_desc& D, int li, int esize) {
+    const cfpp_seq_layer& d = D.layers[li];
+    const int rc = check_mixer(D, li, esize);
+    if (rc) return rc;
+    if (d.ff_kind < CFPP_SEQ_FF_NONE || d.ff_kind > CFPP_SEQ_FF_GATED) return CFPP_ERR_MODE;
     size_t lds = std::max(pitch_of(D.width, esize) + 1024 + (size_t)D.width * 4, pitch_of(d.heads * d.vdim, esize) + 1024);
     if (d.ff_kind != CFPP_SEQ_FF_NONE) {
         if (d.ff < 1 || d.w_up == nullptr || d.w_down == nullptr || d.norm2 == nullptr) return CFPP_ERR_NULL;
+        if (D.streams > 0 && !connected(d.hc2)) return CFPP_ERR_NULL;
         const size_t one = pitch_of(d.ff, esize) + 1024;
         if (d.ff_kind == CFPP_SEQ_FF_TABLE_EXPERTS) {
             if (d.experts < 1 || d.experts > 8192 || d.top < 1 || d.top > kWave || d.top > d.experts || d.shared_ff < 0) return CFPP_ERR_DIMS;
@@ -1587,6 +1939,24 @@ int check_layer(const cfpp_seq_desc& D, const cfpp_seq_layer& d, int esize) {
     }
     // the input of a matrix-vector product sits in LDS
     return lds > 150 * 1024 ? CFPP_ERR_DIMS : CFPP_OK;
+}
+
+// Angles per position of the layer's rotary pairs; the factor on cos and sin.  With scaling, pairs that make more than
+// rot_fast turns over rot_original positions keep their angle, those with fewer than rot_slow have it divided by rot_factor,
+// and the ones between are blended linearly in the pair index.
+double angles(const cfpp_seq_layer& d, double* freq) {
+    const int half = d.rot_dims / 2;
+    const double base = d.rot_base;
+    for (int j = 0; j < half; ++j) freq[j] = pow(base, -2.0 * j / d.rot_dims);
+    if (!(d.rot_factor > 0.0)) return 1.0;
+    const double two_pi = 6.283185307179586476925, factor = d.rot_factor;
+    auto index_of = [&](double turns) { return d.rot_dims * log(d.rot_original / (two_pi * turns)) / (2.0 * log(base)); };
+    const double lo = std::max(floor(index_of(d.rot_fast)), 0.0), hi = std::min(ceil(index_of(d.rot_slow)), (double)(d.rot_dims - 1));
+    for (int j = 0; j < half; ++j) {
+        const double r = std::min(std::max((j - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+        freq[j] = freq[j] / factor * r + freq[j] * (1.0 - r);
+    }
+    return 0.1 * log(factor) + 1.0;
 }
 
 }  // namespace
@@ -1604,10 +1974,11 @@ int cfpp_seq_create(const cfpp_seq_desc* desc, cfpp_seq** out) {
     if (D.dtype != CFPP_SEQ_BF16 && D.dtype != CFPP_SEQ_F32) return CFPP_ERR_MODE;
     if (D.n_layers < 1 || D.width < 1 || D.width > 16384 || D.vocab < 1 || D.vocab > 524288 || D.slots < 1 || D.capacity < 1 || D.max_portion < 1)
         return CFPP_ERR_DIMS;
+    if (D.streams < 0 || D.streams > CFPP_SEQ_MAX_STREAMS || (D.pos != nullptr && (D.streams == 0 || D.positions < D.capacity))) return CFPP_ERR_DIMS;
     const int esize = D.dtype == CFPP_SEQ_BF16 ? 2 : 4;
     int first_mix = -1;
     for (int i = 0; i < D.n_layers; ++i) {
-        const int rc = check_layer(D, D.layers[i], esize);
+        const int rc = check_layer(D, i, esize);
         if (rc) return rc;
         if (D.layers[i].v_mix) {
             if (first_mix < 0) first_mix = i;
@@ -1623,54 +1994,79 @@ int cfpp_seq_create(const cfpp_seq_desc* desc, cfpp_seq** out) {
     s->portion = std::min(D.max_portion, D.capacity);
     (void)hipGetDevice(&s->device);
     if (hipDeviceGetAttribute(&s->cus, hipDeviceAttributeMultiprocessorCount, s->device) != hipSuccess || s->cus < 1) s->cus = 256;
-    const size_t P = (size_t)s->portion;
-    size_t n_qkv = 0, o_bytes = 0, h_bytes = 0, hs_bytes = 0, q_el = 0, k_el = 0, v_el = 0, vf = 0, ys = 0, part = 0, items = 0, dec_h = 0;
-    std::map<std::pair<float, int>, float2*> tables;
+    const size_t P = (size_t)s->portion, C = (size_t)D.capacity;
+    size_t n_qkv = 0, o_bytes = 0, h_bytes = 0, hs_bytes = 0, q_bytes = 0, k_bytes = 0, v_bytes = 0, vf = 0, ys = 0, part = 0, items = 0, dec_h = 0;
+    std::map<std::tuple<double, int, double, double, double, double>, float2*> tables;
     for (int i = 0; i < D.n_layers; ++i) {
         LayerPlan L{};
         L.d = D.layers[i];
         const cfpp_seq_layer& d = L.d;
-        L.R = d.heads / d.kv_heads;
-        L.nct = ceil_div(L.R, kAttnCols);
-        L.Dp = up_to(d.dim, 64 / esize);
-        L.Vp = up_to(d.vdim, 16);
-        L.krow = L.Dp * esize;
-        L.vrow = L.Vp * esize;
-        L.NT = std::max(L.Dp, L.Vp) <= 64 ? 64 : std::max(L.Dp, L.Vp) <= 128 ? 128 : 256;
-        L.rows = d.chunk > 0 ? std::min(d.chunk, D.capacity) : D.capacity;
-        L.n_qkv = d.heads * d.dim + d.kv_heads * (d.dim + d.vdim);
-        L.v_role = !d.v_mix ? 0 : i == first_mix ? 1 : 2;
-        const int kt = esize == 2 ? 32 : (L.NT <= 128 ? 32 : 16);
-        L.ns = std::max(1, std::min({kMaxSeqSplit, ceil_div(kAttnWgs * s->cus, d.kv_heads * L.nct), ceil_div(L.rows, kt * kSeqWaves)}));
-        L.kc = s->alloc<char>((size_t)D.slots * d.kv_heads * L.rows * L.krow);
-        L.vc = s->alloc<char>((size_t)D.slots * d.kv_heads * L.rows * L.vrow);
+        L.latent = d.mixer == CFPP_SEQ_MIX_LATENT;
+        if (L.latent) {
+            L.own = d.kv_from < 0;
+            L.Vp = up_to(d.vdim, 16);
+            L.vrow = L.Vp * esize;
+            L.rp = up_to(d.kv_rank, 16);
+            L.lpitch = (int)pitch_of(d.kv_rank, esize);
+            L.plain = up_to(d.dim * esize, 16);
+            L.shared = up_to(d.rot_dims * esize, 16);
+            L.crow = up_to(L.lpitch + L.shared, 64);
+            L.qrow = up_to(L.plain + L.shared, 64);
+            L.n_qkv = d.heads * (d.dim + d.rot_dims);
+            if (L.own) L.n_qkv += d.kv_rank + d.rot_dims;
+            L.gate_at = L.n_qkv;
+            if (d.gated) L.n_qkv += d.heads * d.vdim;
+            const int groups = ceil_div(d.heads, 16 * latent_sets(d.heads)), keys = esize == 2 ? LatentTile<bf16_t>::keys : LatentTile<float>::keys;
+            L.ns = std::max(1, std::min({kLatentSplits, ceil_div(s->cus, groups), ceil_div(D.capacity, keys)}));
+            L.kc = L.own ? s->alloc<char>((size_t)D.slots * C * L.crow) : s->layers[d.kv_from].kc;
+            q_bytes = std::max({q_bytes, P * d.heads * L.qrow, (size_t)d.heads * L.crow});
+            k_bytes = std::max(k_bytes, C * d.heads * L.plain);
+            v_bytes = std::max(v_bytes, C * d.heads * L.vrow);
+            part = std::max(part, (size_t)L.ns * d.heads * (L.rp + 2));
+        } else {
+            L.R = d.heads / d.kv_heads;
+            L.nct = ceil_div(L.R, kAttnCols);
+            L.Dp = up_to(d.dim, 64 / esize);
+            L.Vp = up_to(d.vdim, 16);
+            L.krow = L.Dp * esize;
+            L.vrow = L.Vp * esize;
+            L.NT = std::max(L.Dp, L.Vp) <= 64 ? 64 : std::max(L.Dp, L.Vp) <= 128 ? 128 : 256;
+            L.rows = d.chunk > 0 ? std::min(d.chunk, D.capacity) : D.capacity;
+            L.n_qkv = d.heads * d.dim + d.kv_heads * (d.dim + d.vdim);
+            L.v_role = !d.v_mix ? 0 : i == first_mix ? 1 : 2;
+            const int kt = esize == 2 ? 32 : (L.NT <= 128 ? 32 : 16);
+            L.ns = std::max(1, std::min({kMaxSeqSplit, ceil_div(kAttnWgs * s->cus, d.kv_heads * L.nct), ceil_div(L.rows, kt * kSeqWaves)}));
+            L.kc = s->alloc<char>((size_t)D.slots * d.kv_heads * L.rows * L.krow);
+            L.vc = s->alloc<char>((size_t)D.slots * d.kv_heads * L.rows * L.vrow);
+            q_bytes = std::max(q_bytes, P * d.heads * L.krow);
+            k_bytes = std::max(k_bytes, P * d.kv_heads * L.krow);
+            v_bytes = std::max(v_bytes, P * d.kv_heads * L.vrow);
+            if (d.v_mix) vf = std::max(vf, (size_t)d.kv_heads * d.vdim);
+            items = std::max(items, (size_t)d.kv_heads * L.nct);
+            part = std::max(part, (size_t)d.kv_heads * L.nct * L.ns * kAttnCols * (L.Vp + 2));
+        }
         L.cs = nullptr;
         if (d.rot_dims > 0) {
-            float2*& t = tables[{d.rot_base, d.rot_dims}];
+            const double f = d.rot_factor;
+            float2*& t = tables[{d.rot_base, d.rot_dims, f, f > 0 ? d.rot_original : 0.0, f > 0 ? d.rot_fast : 0.0, f > 0 ? d.rot_slow : 0.0}];
             if (t == nullptr) {
                 const int half = d.rot_dims / 2;
                 t = s->alloc<float2>((size_t)D.capacity * half);
                 std::vector<double> freq(half);
-                for (int j = 0; j < half; ++j) freq[j] = pow((double)d.rot_base, -2.0 * j / d.rot_dims);
+                const double mul = angles(d, freq.data());
                 double* df = s->alloc<double>(half);
                 if (!s->failed) {
                     (void)hipDeviceSynchronize();        // the zero fill of the table comes before its copy
                     if (hipMemcpy(df, freq.data(), half * sizeof(double), hipMemcpyHostToDevice) != hipSuccess) s->failed = true;
-                    hipLaunchKernelGGL(k_seq_rope_table, dim3(1024), dim3(256), 0, nullptr, t, df, half, D.capacity);
+                    hipLaunchKernelGGL(k_seq_rope_table, dim3(1024), dim3(256), 0, nullptr, t, df, mul, half, D.capacity);
                 }
             }
             L.cs = t;
         }
         n_qkv = std::max(n_qkv, (size_t)L.n_qkv);
         o_bytes = std::max(o_bytes, pitch_of(d.heads * d.vdim, esize));
-        q_el = std::max(q_el, (size_t)d.heads * L.krow);
-        k_el = std::max(k_el, (size_t)d.kv_heads * L.krow);
-        v_el = std::max(v_el, (size_t)d.kv_heads * L.vrow);
-        if (d.v_mix) vf = std::max(vf, (size_t)d.kv_heads * d.vdim);
-        items = std::max(items, (size_t)d.kv_heads * L.nct);
-        part = std::max(part, (size_t)d.kv_heads * L.nct * L.ns * kAttnCols * (L.Vp + 2));
         L.route = -1;
-        if (d.ff_kind == CFPP_SEQ_FF_RELU2) {
+        if (d.ff_kind == CFPP_SEQ_FF_RELU2 || d.ff_kind == CFPP_SEQ_FF_GATED) {
             h_bytes = std::max(h_bytes, pitch_of(d.ff, esize));
         } else if (d.ff_kind == CFPP_SEQ_FF_TABLE_EXPERTS) {
             h_bytes = std::max(h_bytes, d.top * pitch_of(d.ff, esize));
@@ -1687,16 +2083,17 @@ int cfpp_seq_create(const cfpp_seq_desc* desc, cfpp_seq** out) {
     s->ld_qkv = up_to((int)n_qkv, 4);
     s->tokens = s->alloc<int>(2 * P);
     s->want = s->tokens != nullptr ? s->tokens + P : nullptr;
-    s->x = s->alloc<float>(P * D.width);
+    const size_t rows_of_x = std::max(1, D.streams);
+    s->x = s->alloc<float>(P * rows_of_x * D.width);
     s->y = s->alloc<float>(P * D.width);
     s->ys = s->alloc<float>(P * ys);
     s->qkv = s->alloc<float>(P * s->ld_qkv);
     s->v_first = s->alloc<float>(P * vf);
     s->xb = s->alloc<char>(P * s->xpitch);
     s->wb = s->alloc<char>(P * s->xpitch);
-    s->q = s->alloc<char>(P * q_el);
-    s->k = s->alloc<char>(P * k_el);
-    s->v = s->alloc<char>(P * v_el);
+    s->q = s->alloc<char>(q_bytes);
+    s->k = s->alloc<char>(k_bytes);
+    s->v = s->alloc<char>(v_bytes);
     s->o = s->alloc<char>(P * o_bytes);
     s->h = s->alloc<char>(std::max(P * h_bytes, dec_h));
     s->hs = s->alloc<char>(P * hs_bytes);
@@ -1706,7 +2103,8 @@ int cfpp_seq_create(const cfpp_seq_desc* desc, cfpp_seq** out) {
     s->history = s->alloc<int>(s->history_cap);
     s->cnt = s->alloc<int>(items * kHeadCntStride);
     s->part = s->alloc<float>(part);
-    s->dx[0] = s->alloc<float>(D.width);
+    s->dx[0] = s->alloc<float>(rows_of_x * D.width);
+    s->du = s->alloc<float>(D.width);
     s->dx[1] = s->alloc<float>(D.width);
     s->dy = s->alloc<float>(D.width);
     s->dres = s->alloc<float>((size_t)D.n_layers * D.width);

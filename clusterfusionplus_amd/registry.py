@@ -19,6 +19,11 @@ def _nibotar(*args, **kw):
     return nibotar.load(*args, **kw)
 
 
+def _kagapel(*args, **kw):
+    from . import kagapel
+    return kagapel.load(*args, **kw)
+
+
 def _neox(*args, **kw):
     from .build import ensure_neox
     ensure_neox()
@@ -29,6 +34,7 @@ def _neox(*args, **kw):
 # architecture name -> (loader, element types it runs in)
 _REGISTRY: Dict[str, Tuple[Callable, Tuple[str, ...]]] = {
     "Nibotar": (_nibotar, ("bfloat16", "float32")),
+    "Kagapel": (_kagapel, ("bfloat16", "float32")),
     "GPTNeoXForCausalLM": (_neox, ("float16",)),
 }
 

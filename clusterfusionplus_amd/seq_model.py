@@ -13,21 +13,29 @@ import torch
 _HERE = os.path.dirname(os.path.abspath(__file__))
 _DTYPE_CODE = {torch.bfloat16: 0, torch.float32: 1}
 ROW_BYTES = 128
-FF_NONE, FF_RELU2, FF_TABLE_EXPERTS = 0, 1, 2
+FF_NONE, FF_RELU2, FF_TABLE_EXPERTS, FF_GATED = 0, 1, 2, 3
+MIX_GROUPED, MIX_LATENT = 0, 1
+
+
+class _Streams(C.Structure):
+    _fields_ = [(n, C.c_void_p) for n in ("in", "mix", "out")]
 
 
 class _Layer(C.Structure):
-    _fields_ = [(n, C.c_int32) for n in ("heads", "kv_heads", "dim", "vdim", "chunk", "rot_dims", "v_mix")] + \
-        [(n, C.c_float) for n in ("rot_base", "scale", "v_lambda")] + \
-        [(n, C.c_void_p) for n in ("w_qkv", "b_qkv", "q_norm", "k_norm", "sink", "w_o", "norm1")] + \
+    _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "kv_heads", "dim", "vdim", "chunk", "rot_dims", "rot_half", "v_mix", "kv_rank", "kv_from", "gated")] + \
+        [(n, C.c_float) for n in ("scale", "v_lambda")] + \
+        [(n, C.c_double) for n in ("rot_base", "rot_factor", "rot_original", "rot_fast", "rot_slow")] + \
+        [(n, C.c_void_p) for n in ("w_qkv", "b_qkv", "q_norm", "k_norm", "kv_norm", "w_ukv", "sink", "w_o", "norm1")] + \
+        [("hc1", _Streams)] + \
         [(n, C.c_int32) for n in ("ff_kind", "ff", "experts", "top", "shared_ff")] + \
-        [(n, C.c_void_p) for n in ("w_up", "w_down", "w_shared_up", "w_shared_down", "table", "norm2")]
+        [(n, C.c_void_p) for n in ("w_up", "w_down", "b_up", "b_down", "w_shared_up", "w_shared_down", "table", "norm2")] + \
+        [("hc2", _Streams)]
 
 
 class _Desc(C.Structure):
-    _fields_ = [(n, C.c_int32) for n in ("dtype", "n_layers", "width", "vocab")] + \
-        [(n, C.c_float) for n in ("eps", "alpha", "softcap")] + \
-        [("layers", C.POINTER(_Layer)), ("embed", C.c_void_p), ("final_norm", C.c_void_p), ("head", C.c_void_p)] + \
+    _fields_ = [(n, C.c_int32) for n in ("dtype", "n_layers", "width", "vocab", "streams", "positions")] + \
+        [(n, C.c_float) for n in ("eps", "alpha", "norm_offset", "logit_scale", "softcap")] + \
+        [("layers", C.POINTER(_Layer)), ("embed", C.c_void_p), ("pos", C.c_void_p), ("final_norm", C.c_void_p), ("head", C.c_void_p)] + \
         [(n, C.c_int32) for n in ("slots", "capacity", "max_portion")]
 
 
@@ -79,30 +87,58 @@ def interleave(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
     return torch.stack((gate, up), dim=-2).flatten(-3, -2)
 
 
+def _ptr(t: Optional[torch.Tensor]) -> Optional[int]:
+    return t.data_ptr() if t is not None else None
+
+
 def vector(v: torch.Tensor, device) -> torch.Tensor:
     return v.detach().to(device=device, dtype=torch.float32).contiguous()
 
 
 @dataclass
+class Connections:
+    """How a sublayer reads and updates the residual streams (fp32 on the device)."""
+    read: torch.Tensor        # [streams]
+    mix: torch.Tensor         # [streams, streams], indexed [from, to]
+    write: torch.Tensor       # [streams]
+
+
+@dataclass
 class SeqLayer:
-    """One layer: sizes and constants as numbers, tensors on the device (matrices through pad_rows, vectors fp32)."""
+    """One layer: sizes and constants as numbers, tensors on the device (matrices through pad_rows, vectors fp32).  What a
+    mixer or a feed-forward does not use stays at its default; include/cfpp_seq.h says what each one is."""
     heads: int
-    kv_heads: int
     dim: int
     vdim: int
     scale: float
     w_qkv: torch.Tensor
-    b_qkv: torch.Tensor
-    q_norm: torch.Tensor
-    k_norm: torch.Tensor
-    sink: torch.Tensor
     w_o: torch.Tensor
     norm1: torch.Tensor
-    chunk: int = 0
+    mixer: int = MIX_GROUPED
+    sink: Optional[torch.Tensor] = None
     rot_dims: int = 0
+    rot_half: bool = False
     rot_base: float = 10000.0
+    rot_factor: float = 0.0
+    rot_original: float = 0.0
+    rot_fast: float = 0.0
+    rot_slow: float = 0.0
+    hc1: Optional[Connections] = None
+    # grouped heads
+    kv_heads: int = 0
+    chunk: int = 0
     v_mix: bool = False
     v_lambda: float = 0.0
+    b_qkv: Optional[torch.Tensor] = None
+    q_norm: Optional[torch.Tensor] = None
+    k_norm: Optional[torch.Tensor] = None
+    # latent
+    kv_rank: int = 0
+    kv_from: int = -1
+    gated: bool = False
+    kv_norm: Optional[torch.Tensor] = None
+    w_ukv: Optional[torch.Tensor] = None
+    # feed-forward
     ff_kind: int = FF_NONE
     ff: int = 0
     experts: int = 0
@@ -110,10 +146,13 @@ class SeqLayer:
     shared_ff: int = 0
     w_up: Optional[torch.Tensor] = None
     w_down: Optional[torch.Tensor] = None
+    b_up: Optional[torch.Tensor] = None
+    b_down: Optional[torch.Tensor] = None
     w_shared_up: Optional[torch.Tensor] = None
     w_shared_down: Optional[torch.Tensor] = None
     table: Optional[torch.Tensor] = None
     norm2: Optional[torch.Tensor] = None
+    hc2: Optional[Connections] = None
 
 
 @dataclass
@@ -122,11 +161,15 @@ class SeqWeights:
     width: int
     vocab: int
     eps: float
-    alpha: float
     layers: List[SeqLayer]
     embed: torch.Tensor
     final_norm: torch.Tensor
     head: torch.Tensor
+    alpha: float = 1.0
+    streams: int = 0                      # residual streams with norms in front; 0: norms after the sums
+    pos: Optional[torch.Tensor] = None    # learned positions
+    norm_offset: float = 1.0              # norm weight = norm_offset + stored weight
+    logit_scale: float = 1.0
     softcap: float = 0.0
     architecture: str = ""
     extra: dict = field(default_factory=dict)
@@ -150,12 +193,15 @@ class SeqModel:
             for name, kind in _Layer._fields_:
                 v = getattr(l, name)
                 if kind is C.c_void_p:
-                    v = v.data_ptr() if v is not None else None
+                    v = _ptr(v)
                 elif kind is C.c_int32:
                     v = int(v)
+                elif kind is _Streams:
+                    v = _Streams(_ptr(v.read), _ptr(v.mix), _ptr(v.write)) if v is not None else _Streams()
                 setattr(s, name, v)
-        desc = _Desc(_DTYPE_CODE[weights.dtype], self.n_layers, self.width, self.vocab, weights.eps, weights.alpha, weights.softcap,
-                     arr, weights.embed.data_ptr(), weights.final_norm.data_ptr(), weights.head.data_ptr(),
+        desc = _Desc(_DTYPE_CODE[weights.dtype], self.n_layers, self.width, self.vocab, weights.streams,
+                     weights.pos.shape[0] if weights.pos is not None else 0, weights.eps, weights.alpha, weights.norm_offset, weights.logit_scale,
+                     weights.softcap, arr, _ptr(weights.embed), _ptr(weights.pos), _ptr(weights.final_norm), _ptr(weights.head),
                      self.slots, self.capacity, int(max_portion))
         handle = C.c_void_p()
         with torch.cuda.device(self.device):

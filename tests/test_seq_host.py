@@ -9,7 +9,8 @@ import pytest
 import torch
 
 from clusterfusionplus_amd import engine as E
-from clusterfusionplus_amd import nibotar, registry, seq_model, trace, weights
+from clusterfusionplus_amd import kagapel, nibotar, registry, seq_model, trace, weights
+from tests import kagapel_models as KM
 from tests import nibotar_models as M
 
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
@@ -72,6 +73,44 @@ def test_value_mixing_needs_equal_values():
     assert len(sizes) == 1
 
 
+def test_kagapel_config_is_read_in_full():
+    c = kagapel.parse_config(KM.CASES["everything"])
+    assert (c.width, c.vocab, c.eps, c.streams, c.max_positions, c.logit_scale) == (160, 301, 1e-3, 3, 512, 0.7)
+    a, b = c.layers[0].mixer, c.layers[1].mixer
+    assert (a.heads, a.dim, a.rot_dim, a.vdim, a.kv_rank, a.scale, a.rot_base, a.yarn, a.gated, a.sink, a.kv_from) == \
+        (6, 40, 24, 56, 72, 0.2, 5000.0, None, False, True, -1)
+    assert (b.yarn, b.gated, b.sink) == (kagapel.Yarn(3.0, 100.0, 32.0, 1.0), True, False)
+    assert [l.mixer.kv_from for l in c.layers] == [-1, -1, 0, -1, 0] and [l.ff for l in c.layers] == [100, 200, 60, 0, 44]
+
+
+@pytest.mark.parametrize("change", [lambda c: c["layers"][0].update(type="attention"), lambda c: c["layers"][0]["mlp"].update(kind="moe"),
+                                    lambda c: c["layers"][0]["mixer"].update(kv_from=2), lambda c: c["layers"][4]["mixer"].update(kv_from=2),
+                                    lambda c: c["layers"][2]["mixer"].update(kv_rank=71), lambda c: c["layers"][2]["mixer"]["rot"].update(base=1.5),
+                                    lambda c: c["layers"][4]["mixer"].update(kv_from=1), lambda c: c["layers"][1]["mixer"].update(rot_dim=18)])
+def test_kagapel_configs_that_do_not_fit_are_refused(change):
+    cfg = json.loads(json.dumps(KM.CASES["everything"]))
+    change(cfg)
+    with pytest.raises(ValueError):
+        kagapel.parse_config(cfg)
+
+
+def test_kagapel_packed_weights():
+    cfg = KM.CASES["width_not_of_fours"]
+    w = KM.weights(cfg)
+    p = kagapel.pack_weights(kagapel.parse_config(cfg), w, torch.bfloat16, "cpu")
+    l0, l1, l2 = p.layers
+    assert l0.w_qkv.shape == (3 * 24 + 43 + 66, 128) and l1.w_qkv.shape == (5 * 40 + 29, 128) and l2.w_qkv.shape == (2 * 17, 128)
+    assert torch.equal(l0.w_qkv[72:115, :70], w["l0.mix.dkv"]) and torch.equal(l0.w_qkv[115:, :70], w["l0.mix.g"])
+    assert l0.w_ukv.shape == (3 * 40, 64) and torch.equal(l0.w_ukv[54:, :37], w["l0.mix.uv"]) and not l0.w_ukv[:, 37:].any()
+    assert torch.equal(l1.w_up[0::2, :70], w["l1.mlp.gate"]) and torch.equal(l1.b_up[1::2], w["l1.mlp.up.b"].float())
+    assert l0.sink is None and l1.kv_norm.shape == (19,) and l2.kv_norm is None and l2.kv_from == 1 and l2.ff_kind == seq_model.FF_NONE
+    assert torch.equal(l1.hc2.mix, w["l1.hc2.mix"].float()) and l2.hc2 is None and p.norm_offset == 0.0 and p.pos.shape == (512, 128)
+    for name in ("l0.mix.dkv.norm", "l1.hc1.mix", "l1.mlp.down.b", "pos"):
+        bad = {n: (t[:-1] if n == name else t) for n, t in w.items()}
+        with pytest.raises(ValueError, match=re.escape(name)):
+            kagapel.pack_weights(kagapel.parse_config(cfg), bad, torch.bfloat16, "cpu")
+
+
 def test_safetensors_files(tmp_path):
     from safetensors.torch import load_file, save_file
     t = {"a": torch.randn(3, 5), "b": torch.arange(7).int(), "c": torch.randn(2, 3).bfloat16(), "s": torch.tensor(0.5).bfloat16(), "e": torch.zeros(0, 4)}
@@ -90,8 +129,8 @@ def test_safetensors_files(tmp_path):
 
 
 def test_registry(tmp_path):
-    assert registry.architectures() == ["GPTNeoXForCausalLM", "Nibotar"]
-    assert registry.dtypes_of({"architecture": "Nibotar"}) == ("bfloat16", "float32")
+    assert registry.architectures() == ["GPTNeoXForCausalLM", "Kagapel", "Nibotar"]
+    assert registry.dtypes_of({"architecture": "Nibotar"}) == registry.dtypes_of({"architecture": "Kagapel"}) == ("bfloat16", "float32")
     assert registry.architecture_of({"architectures": ["GPTNeoXForCausalLM"]}) == "GPTNeoXForCausalLM"
     with pytest.raises(ValueError):
         registry.architecture_of({"architectures": ["Other"]})
