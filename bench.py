@@ -561,62 +561,113 @@ def nibotar_model(z, capacity, max_portion, dev, n_layers=None):
     return m, dict(layer_params=per_layer, params=sum(per_layer), head=W * V, kv_row=kv_row, attn_flops=2 * H * (D + Dv), n_layers=len(layers))
 
 
-def bench_nibotar(args):
-    """Nibotar at a few sizes (random weights): decode (TPOT of captured-graph replays at --ctx cached tokens) and prefill
-    (whole prompts of several lengths), each against its roofline: decode against the HBM bytes of the weights the token
-    uses and of the visible cache rows, prefill against the dense bf16 matrix peak.  Beside the size that has a Pythia-6.9B
-    layer's matrices: the Pythia-6.9B stack itself, in fused and in split mode."""
+KAGAPEL_SIZES = {
+    # as many parameters per layer as Nibotar's dense_6b9, and its width, heads and vocabulary
+    "latent_6b9": dict(width=4096, layers=32, heads=32, dim=128, rot_dim=64, vdim=128, kv_rank=512, ff=11264, streams=4, vocab=50432),
+    # sixteen heads (the layer sizes of small latent-attention models)
+    "latent_2b": dict(width=2048, layers=27, heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, ff=10944, streams=2, vocab=102400),
+    # as many heads as the largest latent-attention models
+    "latent_wide": dict(width=5120, layers=16, heads=128, dim=128, rot_dim=64, vdim=128, kv_rank=512, ff=12288, streams=4, vocab=102400),
+}
+
+
+def kagapel_model(z, capacity, max_portion, dev, n_layers=None):
+    """A Kagapel model of the given sizes with random bf16 weights on the device: layers with a gate and scaled angles, layers
+    with sinks, and layers that read the latents of the layer before them take turns.  Also what it is priced by."""
+    import torch
+    from clusterfusionplus_amd import seq_model as S
+    torch.manual_seed(0)
+    W, H, D, R, Dv, rank, F, V, n_s = (z[k] for k in ("width", "heads", "dim", "rot_dim", "vdim", "kv_rank", "ff", "vocab", "streams"))
+
+    def rn(*shape, std=0.02):
+        return torch.empty(shape, dtype=torch.bfloat16, device=dev).normal_(0, std)
+
+    def vec(n, mean=0.0):
+        return torch.empty(n, dtype=torch.float32, device=dev).normal_(mean, 0.02)
+
+    def connections():
+        return S.Connections(vec(n_s, 1.0 / n_s), torch.eye(n_s, device=dev) * 0.9 + 0.02, vec(n_s, 1.0))
+    layers, per_layer = [], []
+    for i in range(n_layers or z["layers"]):
+        kind = i % 4                     # 0, 3: gated; 1: sinks; 2: sinks and the latents of the layer before it
+        kw = dict(gated=True, rot_factor=4.0, rot_original=2048.0, rot_fast=32.0, rot_slow=1.0) if kind in (0, 3) else dict(sink=vec(H))
+        kw.update(dict(kv_from=i - 1) if kind == 2 else dict(kv_norm=vec(rank, 1.0)))
+        rows = H * (D + R) + (rank + R if kind != 2 else 0) + (H * Dv if kind in (0, 3) else 0)
+        layers.append(S.SeqLayer(mixer=S.MIX_LATENT, heads=H, dim=D, vdim=Dv, scale=(D + R) ** -0.5, rot_dims=R, rot_half=True, kv_rank=rank,
+                                 w_qkv=rn(rows, W), w_ukv=rn(H * (D + Dv), rank), w_o=rn(W, H * Dv), norm1=vec(W, 1.0), norm2=vec(W, 1.0),
+                                 ff_kind=S.FF_GATED, ff=F, w_up=rn(2 * F, W), b_up=vec(2 * F), w_down=rn(W, F), b_down=vec(W),
+                                 hc1=connections(), hc2=connections(), **kw))
+        per_layer.append(W * rows + H * (D + Dv) * rank + W * H * Dv + 3 * W * F)
+    w = S.SeqWeights(dtype=torch.bfloat16, width=W, vocab=V, eps=1e-6, streams=n_s, norm_offset=0.0, logit_scale=1.5, layers=layers, embed=rn(V, W, std=1.0),
+                     pos=rn(capacity, W, std=0.5), final_norm=vec(W, 1.0), head=rn(V, W), architecture="Kagapel")
+    m = S.SeqModel(w, capacity=capacity, max_portion=max_portion)
+    return m, dict(layer_params=per_layer, params=sum(per_layer), head=W * V, kv_row=(rank + R) * 2, attn_flops=2 * H * (D + R + Dv), n_layers=len(layers))
+
+
+def measure_sequence_model(args, family, name, z, make):
+    """Decode (TPOT of captured-graph replays at --ctx cached tokens) and prefill (whole prompts of several lengths) of one size,
+    each against its roofline: decode against the HBM bytes of the weights the token uses and of the visible cache rows, prefill
+    against the dense bf16 matrix peak."""
+    import torch
+    peak_tf, prompts = 2500.0, [512, 2048, 8192]
+    m, b = make(z, max(args.ctx + args.warmup + args.steps + 64, max(prompts)), max(prompts), "cuda:0", args.layers or None)
+    g = torch.Generator().manual_seed(1)
+    toks = torch.randint(0, z["vocab"], (max(prompts + [args.ctx]),), generator=g).tolist()
+    e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+    pre = []
+    for n in prompts:
+        for _ in range(2):
+            m.forward(0, toks[:n], 0, [n - 1])
+        torch.cuda.synchronize()
+        reps = max(1, min(5, 16384 // n))
+        e0.record()
+        for _ in range(reps):
+            m.forward(0, toks[:n], 0, [n - 1])
+        e1.record()
+        torch.cuda.synchronize()
+        ms = e0.elapsed_time(e1) / reps
+        flops = 2 * n * b["params"] + 2 * b["head"] + b["n_layers"] * b["attn_flops"] * n * (n + 1) / 2
+        pre.append({"tokens": n, "ms": round(ms, 3), "tokens_per_s": round(n / ms * 1e3), "tflops": round(flops / ms / 1e9, 1),
+                    "frac_of_matrix_peak": round(flops / ms / 1e9 / peak_tf, 4)})
+        log(f"[{family} {name}] prefill {n}: {ms:.3f} ms, {pre[-1]['tokens_per_s']} tokens/s, {pre[-1]['tflops']} TFLOP/s")
+    m.forward(0, toks[:args.ctx], 0)
+    m.set_state(11, args.ctx)
+    m.graph_steps(args.warmup)
+    torch.cuda.synchronize()
+    t0 = time.perf_counter()
+    m.graph_steps(args.steps)
+    torch.cuda.synchronize()
+    tpot = (time.perf_counter() - t0) * 1e3 / args.steps
+    rows = args.ctx + args.warmup + args.steps // 2
+    rows = min(rows, z.get("chunk", rows))
+    nbytes = 2 * (b["params"] + b["head"]) + b["n_layers"] * rows * b["kv_row"]
+    gbps = nbytes / (tpot * 1e-3) / 1e9
+    log(f"[{family} {name}] decode at {args.ctx}: {tpot:.4f} ms/token, {gbps / HBM_PEAK_GBPS * 100:.1f} % of the HBM roofline")
+    out = {"model": family, "size": name, **z, "layers": b["n_layers"], "prefill": pre, "decode": {
+        "context": args.ctx, "tpot_ms": round(tpot, 4), "tokens_per_s": round(1e3 / tpot, 1), "launches": m.launches_per_step, "bytes": nbytes,
+        "hbm_gbps": round(gbps, 1), "frac_of_peak": round(gbps / HBM_PEAK_GBPS, 4)}}
+    del m
+    torch.cuda.empty_cache()
+    return out
+
+
+def bench_sequence_models(args):
+    """A design of the sequence-model library at a few sizes (random weights), and the closest model of the framework at equal
+    size in the same run: for Nibotar's dense_6b9 the Pythia-6.9B stack (fused and split mode), for Kagapel's latent_6b9 that
+    Nibotar."""
     import torch
     import clusterfusionplus_amd as pkg
-    dev, peak_tf = "cuda:0", 2500.0
-    sizes = args.size.split(",") if args.size else list(NIBOTAR_SIZES)
-    out = []
-    for name in sizes:
-        z = NIBOTAR_SIZES[name]
-        prompts = [512, 2048, 8192]
-        m, b = nibotar_model(z, max(args.ctx + args.warmup + args.steps + 64, max(prompts)), max(prompts), dev, args.layers or None)
-        g = torch.Generator().manual_seed(1)
-        toks = torch.randint(0, z["vocab"], (max(prompts + [args.ctx]),), generator=g).tolist()
-        e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
-        pre = []
-        for n in prompts:
-            for _ in range(2):
-                m.forward(0, toks[:n], 0, [n - 1])
-            torch.cuda.synchronize()
-            reps = max(1, min(5, 16384 // n))
-            e0.record()
-            for _ in range(reps):
-                m.forward(0, toks[:n], 0, [n - 1])
-            e1.record()
-            torch.cuda.synchronize()
-            ms = e0.elapsed_time(e1) / reps
-            flops = 2 * n * b["params"] + 2 * b["head"] + b["n_layers"] * b["attn_flops"] * n * (n + 1) / 2
-            pre.append({"tokens": n, "ms": round(ms, 3), "tokens_per_s": round(n / ms * 1e3), "tflops": round(flops / ms / 1e9, 1),
-                        "frac_of_matrix_peak": round(flops / ms / 1e9 / peak_tf, 4)})
-            log(f"[nibotar {name}] prefill {n}: {ms:.3f} ms, {pre[-1]['tokens_per_s']} tokens/s, {pre[-1]['tflops']} TFLOP/s")
-        m.forward(0, toks[:args.ctx], 0)
-        m.set_state(11, args.ctx)
-        m.graph_steps(args.warmup)
-        torch.cuda.synchronize()
-        t0 = time.perf_counter()
-        m.graph_steps(args.steps)
-        torch.cuda.synchronize()
-        tpot = (time.perf_counter() - t0) * 1e3 / args.steps
-        rows = min(args.ctx + args.warmup + args.steps // 2, z["chunk"])
-        nbytes = 2 * (b["params"] + b["head"]) + b["n_layers"] * rows * b["kv_row"]
-        gbps = nbytes / (tpot * 1e-3) / 1e9
-        log(f"[nibotar {name}] decode at {args.ctx}: {tpot:.4f} ms/token, {gbps / HBM_PEAK_GBPS * 100:.1f} % of the HBM roofline")
-        out.append({"size": name, **z, "layers": b["n_layers"], "prefill": pre, "decode": {
-            "context": args.ctx, "tpot_ms": round(tpot, 4), "tokens_per_s": round(1e3 / tpot, 1), "launches": m.launches_per_step, "bytes": nbytes,
-            "hbm_gbps": round(gbps, 1), "frac_of_peak": round(gbps / HBM_PEAK_GBPS, 4)}})
-        del m
-        torch.cuda.empty_cache()
+    sizes_of, make = {"nibotar": (NIBOTAR_SIZES, nibotar_model), "kagapel": (KAGAPEL_SIZES, kagapel_model)}[args.model]
+    sizes = args.size.split(",") if args.size else list(sizes_of)
+    out = [measure_sequence_model(args, args.model, name, sizes_of[name], make) for name in sizes]
     closest = []
+    if args.also and "latent_6b9" in sizes:
+        closest.append(measure_sequence_model(args, "nibotar", "dense_6b9", NIBOTAR_SIZES["dense_6b9"], nibotar_model))
     if args.also and "dense_6b9" in sizes:
         from dataclasses import replace
         cfg = replace(pkg.PYTHIA_6B9, n_layers=args.layers or pkg.PYTHIA_6B9.n_layers)
         for mode in ("fused", "split"):
-            dec = build_model(cfg, args.ctx + args.warmup + args.steps + 40, args.ctx, dev, mode)
+            dec = build_model(cfg, args.ctx + args.warmup + args.steps + 40, args.ctx, "cuda:0", mode)
             stream = torch.cuda.Stream()
             with torch.cuda.stream(stream):
                 tpot = time_tokens(dec, stream, args.ctx, args.steps, args.warmup)
@@ -630,7 +681,7 @@ def bench_nibotar(args):
     d = out[0]["decode"]
     print(json.dumps({"metric": "tpot_ms", "value": d["tpot_ms"], "unit": "ms/token", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
                       "ms_per_step": d["tpot_ms"], "higher_is_better": False, "scaling": "weak", "vs_baseline": None, "dtype": "bf16",
-                      "data": "synthetic", "config": {"workload": f"nibotar {out[0]['size']}, batch-1 greedy decode, hipGraph replay", "context": args.ctx},
+                      "data": "synthetic", "config": {"workload": f"{args.model} {out[0]['size']}, batch-1 greedy decode, hipGraph replay", "context": args.ctx},
                       "roofline": {"bound": "hbm", "achieved": d["hbm_gbps"], "peak": HBM_PEAK_GBPS, "unit": "GB/s", "frac": d["frac_of_peak"]},
                       "sizes": out, "closest": closest, "cpu_baseline": None}), flush=True)
 
@@ -640,10 +691,11 @@ def main():
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=64)
     ap.add_argument("--warmup", type=int, default=8)
-    ap.add_argument("--model", default="pythia_6b9", choices=["pythia_6b9", "pythia_2b8", "llama2_7b_layer", "llama2_7b_batch", "nibotar"])
+    ap.add_argument("--model", default="pythia_6b9", choices=["pythia_6b9", "pythia_2b8", "llama2_7b_layer", "llama2_7b_batch", "nibotar", "kagapel"])
     ap.add_argument("--batch", type=int, default=16, help="sequences per call (llama2_7b_batch only)")
-    ap.add_argument("--size", default="", help=f"sizes to measure, with commas between them (nibotar only): {', '.join(NIBOTAR_SIZES)}")
-    ap.add_argument("--layers", type=int, default=0, help="layers instead of the model's own number (nibotar only)")
+    ap.add_argument("--size", default="", help="sizes to measure, with commas between them (nibotar: "
+                    f"{', '.join(NIBOTAR_SIZES)}; kagapel: {', '.join(KAGAPEL_SIZES)})")
+    ap.add_argument("--layers", type=int, default=0, help="layers instead of the model's own number (nibotar, kagapel)")
     ap.add_argument("--ctx", type=int, default=2048, help="KV-cache rows already filled when the timed region starts")
     ap.add_argument("--mode", default="fused", choices=["fused", "split", "fused_layers"],
                     help="fused: one launch per layer, or one for all layers where the device holds the whole grid; "
@@ -667,8 +719,8 @@ def main():
         if args.ctx == 2048:
             args.ctx = 4096          # the context this workload is quoted at
         return bench_llama_layer(args)
-    if args.model == "nibotar":
-        return bench_nibotar(args)
+    if args.model in ("nibotar", "kagapel"):
+        return bench_sequence_models(args)
     if args.model == "llama2_7b_batch":
         if args.ctx == 2048:
             args.ctx = 1024

@@ -87,6 +87,9 @@ __device__ __forceinline__ void copy_to_lds16(const void* g, void* lds) {
                                      (__attribute__((address_space(3))) void*)(uintptr_t)lds, 16, 0, 0);
 }
 
+// waits until at most N of the wave's vector memory operations are still on their way
+template <int N> __device__ __forceinline__ void wait_vm() { asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory"); }
+
 // A barrier of the workgroup behind its LDS accesses only: __syncthreads() would also wait for loads in flight.
 __device__ __forceinline__ void lds_barrier() {
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");

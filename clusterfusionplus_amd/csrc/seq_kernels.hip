@@ -349,6 +349,24 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemm(SeqGemm p) {
                 for (int j = 0; j < NI; ++j) acc[i][j] = mma16<T>(fw[i], fa[j], acc[i][j]);
         }
     }
+    // kEpiHeads: where row n goes at position 0, and the bytes from one position to the next; `whole`: rows n0 .. n0 + 3 lie together
+    auto head_row = [&](int n, int& rp) {
+        const bool k = n < p.nk;
+        const int d = k ? p.kd : p.vd, m = k ? n : n - p.nk, h = m / d;
+        rp = k ? p.kp : p.vp;
+        return (k ? p.yt + h * p.kh : p.yv + h * p.vh) + (m - h * d) * (int)sizeof(T);
+    };
+    char* dst[MI];
+    int pitch[MI];
+    bool whole[MI];
+    if constexpr (EPI == kEpiHeads) {
+#pragma unroll
+        for (int i = 0; i < MI; ++i) {
+            const int n0 = min(tw * BW + wr * (BW / 2) + i * 16 + g * 4, p.n - 1);
+            dst[i] = head_row(n0, pitch[i]);
+            whole[i] = ((p.kd | p.vd) & 3) == 0 && n0 + 3 < p.n;       // (n0, the keys' rows and the heads' rows are multiples of four)
+        }
+    }
 #pragma unroll
     for (int j = 0; j < NI; ++j) {
         const int tl = tt * BT + wc * (BT / 2) + j * 16 + col;
@@ -383,21 +401,16 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemm(SeqGemm p) {
                 for (int r = 0; r < 4; ++r)
                     if (n0 + r < p.n) y[r] = from_f32<T>(relu2(v[r]));
             } else if constexpr (EPI == kEpiHeads) {
-                const bool keys = n0 < p.nk;
-                const int d = keys ? p.kd : p.vd, n = keys ? n0 : n0 - p.nk, h = n / d, e = n - h * d;
-                char* base = (keys ? p.yt : p.yv) + (size_t)row * (keys ? p.kp : p.vp);
-                const size_t hs = keys ? p.kh : p.vh;
-                if (e + 3 < d && (e & 3) == 0 && n0 + 3 < (keys ? p.nk : p.n)) {
-                    store4<T>(base + h * hs + e * sizeof(T), v);
+                if (whole[i]) {
+                    store4<T>(dst[i] + (size_t)row * pitch[i], v);
                 } else {
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) {
-                        if (n0 + r >= p.n) break;
-                        const bool k = n0 + r < p.nk;
-                        const int dd = k ? p.kd : p.vd, nn = k ? n0 + r : n0 + r - p.nk, hh = nn / dd;
-                        char* b = k ? p.yt + (size_t)row * p.kp + hh * p.kh : p.yv + (size_t)row * p.vp + hh * p.vh;
-                        reinterpret_cast<T*>(b)[nn - hh * dd] = from_f32<T>(v[r]);
-                    }
+                    for (int r = 0; r < 4; ++r)
+                        if (n0 + r < p.n) {
+                            int rp;
+                            char* b = head_row(n0 + r, rp);
+                            *reinterpret_cast<T*>(b + (size_t)row * rp) = from_f32<T>(v[r]);
+                        }
                 }
             } else {
                 T* y = reinterpret_cast<T*>(p.yt + (size_t)row * p.ldyt) + n0 / 2;
@@ -960,6 +973,23 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
             }
         }
     }
+    // kEpiStreams: lane (output, stream); the first outputs' streams and the connections
+    constexpr int kS = CFPP_SEQ_MAX_STREAMS;
+    const int st_t = lane % kS, st_o = lane / kS;
+    float so[kS], sm[kS], s_out = 0.0f, s_in = 0.0f, s_bias = 0.0f;
+    auto streams_of = [&](int u) __attribute__((always_inline)) {
+#pragma unroll
+        for (int s = 0; s < kS; ++s) so[s] = p.xs[(size_t)min(s, p.streams - 1) * p.width + u];
+        s_bias = p.bias != nullptr ? p.bias[u] : 0.0f;
+    };
+    if constexpr (EPI == kEpiStreams) {
+        const int t = min(st_t, p.streams - 1);
+#pragma unroll
+        for (int s = 0; s < kS; ++s) sm[s] = s < p.streams ? p.mix[s * p.streams + t] : 0.0f;
+        s_out = p.out[t];
+        s_in = st_t >= p.streams ? 0.0f : p.in != nullptr ? p.in[t] : 1.0f;
+        streams_of(min(u0 + st_o, outputs - 1));
+    }
     __builtin_amdgcn_sched_barrier(0);
     u32x4 b0[kGemvLoads], b1[kGemvLoads];
     request(b0);
@@ -1073,6 +1103,28 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
     __builtin_amdgcn_wave_barrier();
     float top_v = -INFINITY;
     int top_i = 0;
+    if constexpr (EPI == kEpiStreams) {
+        for (int i0 = 0; i0 < n_out; i0 += kWave / kS) {
+            const int i = min(i0 + st_o, n_out - 1), u = u0 + i;
+            if (i0 > 0) streams_of(u);
+            float z = s_out * (park[i] + s_bias);
+#pragma unroll
+            for (int s = 0; s < kS; ++s) z = fmadd(sm[s], so[s], z);
+            const bool live = st_t < p.streams && i0 + st_o < n_out;
+            if (live) p.xs[(size_t)st_t * p.width + u] = z;
+            float next = s_in * z, all = st_t < p.streams ? z : 0.0f;
+#pragma unroll
+            for (int m = 1; m < kS; m <<= 1) {
+                next += xor_shfl(next, m);
+                all += xor_shfl(all, m);
+            }
+            if (live && st_t == 0) {
+                p.u[u] = next;
+                if (p.sum != nullptr) p.sum[u] = all;
+            }
+        }
+        return;
+    }
     for (int i = lane; i < n_out; i += kWave) {
         const float v = park[i * UR];
         const int u = u0 + i;
@@ -1087,24 +1139,6 @@ __global__ __launch_bounds__(kSeqThreads, 2) void k_seq_gemv(SeqGemv p) {
             }
         } else if constexpr (EPI == kEpiRelu2) {
             reinterpret_cast<T*>(p.yt)[u] = from_f32<T>(relu2(v));
-        } else if constexpr (EPI == kEpiStreams) {
-            const float y = p.bias != nullptr ? v + p.bias[u] : v;
-            float o[CFPP_SEQ_MAX_STREAMS], next = 0.0f, all = 0.0f;
-#pragma unroll
-            for (int s = 0; s < CFPP_SEQ_MAX_STREAMS; ++s) o[s] = s < p.streams ? p.xs[(size_t)s * p.width + u] : 0.0f;
-#pragma unroll
-            for (int t = 0; t < CFPP_SEQ_MAX_STREAMS; ++t)
-                if (t < p.streams) {
-                    float z = p.out[t] * y;
-#pragma unroll
-                    for (int s = 0; s < CFPP_SEQ_MAX_STREAMS; ++s)
-                        if (s < p.streams) z = fmadd(p.mix[s * p.streams + t], o[s], z);
-                    p.xs[(size_t)t * p.width + u] = z;
-                    next = fmadd(p.in != nullptr ? p.in[t] : 1.0f, z, next);
-                    all += z;
-                }
-            p.u[u] = next;
-            if (p.sum != nullptr) p.sum[u] = all;
         } else {
             const int b = u < p.top * p.units_e ? u / p.units_e : p.top;
             const float bg = p.bias != nullptr ? p.bias[2 * u] : 0.0f, bu = p.bias != nullptr ? p.bias[2 * u + 1] : 0.0f;
@@ -1195,6 +1229,7 @@ struct LayerPlan {
     bool latent, own;
     int lpitch, crow;        // latent part (a padded weight row), whole cache row
     int plain, shared, qrow; // plain and rotated part of a key, whole query row
+    int least;               // tiles of a split of a decode step at least
     int rp;                  // latent columns of the partial results of a decode step
     int gate_at;             // first gate row of the projection
     int route;               // index among the layers with table experts, -1: none
@@ -1684,12 +1719,12 @@ int step_grouped(cfpp_seq* s, const LayerPlan& L, hipStream_t st) {
 }
 
 // sets of 16 heads of a workgroup of k_seq_latent_attn
-int latent_sets(int heads) { return heads <= 16 ? 1 : heads <= 32 ? 2 : 4; }
+int latent_sets(int heads) { return heads <= 32 ? 1 : 2; }
 
 template <typename T, int NR>
 void launch_latent_attn(const SeqLatentAttn& a, hipStream_t st) {
     const int sets = latent_sets(a.H);
-    const size_t lds = 2 * (size_t)a.tile_bytes;
+    const size_t lds = (size_t)LatentLds<T, NR>::buffers * LatentLds<T, NR>::tile;
     const dim3 grid(a.ns, ceil_div(a.H, 16 * sets));
     auto go = [&](auto n) {
         constexpr int RW = decltype(n)::value;
@@ -1697,8 +1732,7 @@ void launch_latent_attn(const SeqLatentAttn& a, hipStream_t st) {
         hipLaunchKernelGGL((k_seq_latent_attn<T, NR, RW>), grid, dim3(kSeqThreads), lds, st, a);
     };
     if (sets == 1) go(std::integral_constant<int, 4>{});
-    else if (sets == 2) go(std::integral_constant<int, 2>{});
-    else go(std::integral_constant<int, 1>{});
+    else go(std::integral_constant<int, 2>{});
 }
 
 template <typename T>
@@ -1710,14 +1744,13 @@ int step_latent(cfpp_seq* s, const LayerPlan& L, hipStream_t st) {
     hipLaunchKernelGGL(k_seq_latent_q<T>, dim3(d.heads * q.nrb + (L.own ? 1 : 0)), dim3(kSeqThreads), 0, st, q);
 
     float* ml = s->part + (size_t)L.ns * d.heads * L.rp;
-    const int tile = up_to(LatentTile<T>::keys * ((L.crow / 16) | 1) * 16, 1024);
-    SeqLatentAttn a{s->q, L.kc, slot, s->state, s->part, ml, d.scale * kLog2e, d.heads, L.crow, L.ns, L.rp, tile};
+    SeqLatentAttn a{s->q, L.kc, slot, s->state, s->part, ml, d.scale * kLog2e, d.heads, L.crow, L.ns, L.least, L.rp};
     if (L.rp <= 128) launch_latent_attn<T, 128>(a, st);
     else launch_latent_attn<T, 512>(a, st);
 
     SeqLatentOut o{s->part, ml, s->state, d.sink, d.gated ? s->qkv + L.gate_at : nullptr, (const char*)d.w_ukv + (size_t)d.heads * d.dim * L.lpitch, s->o,
-                   d.heads, d.vdim, L.lpitch, L.ns, L.rp};
-    hipLaunchKernelGGL(k_seq_latent_out<T>, dim3(ceil_div(d.vdim, kLatentOut), d.heads), dim3(kSeqThreads), 0, st, o);
+                   d.heads, d.vdim, L.lpitch, L.ns, L.least, L.rp};
+    hipLaunchKernelGGL(k_seq_latent_out<T>, dim3(d.heads, ceil_div(d.vdim, kLatentOut)), dim3(kSeqThreads), 0, st, o);
     return 3;
 }
 
@@ -2017,7 +2050,8 @@ int cfpp_seq_create(const cfpp_seq_desc* desc, cfpp_seq** out) {
             L.gate_at = L.n_qkv;
             if (d.gated) L.n_qkv += d.heads * d.vdim;
             const int groups = ceil_div(d.heads, 16 * latent_sets(d.heads)), keys = esize == 2 ? LatentTile<bf16_t>::keys : LatentTile<float>::keys;
-            L.ns = std::max(1, std::min({kLatentSplits, ceil_div(s->cus, groups), ceil_div(D.capacity, keys)}));
+            L.least = 2;
+            L.ns = std::max(1, std::min({kLatentSplits, ceil_div(s->cus, groups), ceil_div(D.capacity, keys * L.least)}));
             L.kc = L.own ? s->alloc<char>((size_t)D.slots * C * L.crow) : s->layers[d.kv_from].kc;
             q_bytes = std::max({q_bytes, P * d.heads * L.qrow, (size_t)d.heads * L.crow});
             k_bytes = std::max(k_bytes, C * d.heads * L.plain);

@@ -144,20 +144,47 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_latent_q(SeqLatentQ a) {
     if (rb == 0) rotate_row<T>(z + a.D, q + a.kv.rot_off, a.R, a.kv.crow - a.kv.rot_off, a.kv.half, cs, tid, kSeqThreads);
 }
 
-// Tiles of keys of a decode step, and how many workgroups share them.
+// Tiles of keys of a decode step, and how many workgroups share them: a few tiles each while that keeps the number of partial
+// results, which every workgroup of k_seq_latent_out reads for its head, small.
 template <typename T> struct LatentTile { static constexpr int keys = sizeof(T) == 2 ? 32 : 16; };
 template <typename T> __device__ __forceinline__ int latent_tiles(int pos) { return (pos + LatentTile<T>::keys) / LatentTile<T>::keys; }
+__device__ __forceinline__ int latent_splits(int tiles, int most, int least) { return min(most, (tiles + least - 1) / least); }
 
-// Column fragment of c^T for the second product: keys 4g .. 4g + 3 (and 16 + 4g ..) of latent column r0 + (lane & 15), from a
-// tile of cache rows in LDS.
-__device__ __forceinline__ u32x2 tr_read(const char* p) {
-    typedef short s16x4 __attribute__((ext_vector_type(4)));
-    return __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)(uintptr_t)p));
+// Column fragments of c^T for the second product, for eight (or two) sets of 16 latent columns: keys 4g .. 4g + 3 (x) and 16 + 4g .. (y) of
+// column lane & 15, from a tile of cache rows in LDS; `p`, `q`: the lane's place in the rows of the one and the other.  The reads
+// and their wait are written out: behind its own transposed reads the compiler would also wait for the copies to the other buffers.
+struct TrCols { u32x2 x, y; };
+__device__ __forceinline__ void tr_read8(TrCols (&f)[8], uint32_t p, uint32_t q) {
+    asm volatile(
+        "ds_read_b64_tr_b16 %0, %16\n\tds_read_b64_tr_b16 %1, %17\n\t"
+        "ds_read_b64_tr_b16 %2, %16 offset:32\n\tds_read_b64_tr_b16 %3, %17 offset:32\n\t"
+        "ds_read_b64_tr_b16 %4, %16 offset:64\n\tds_read_b64_tr_b16 %5, %17 offset:64\n\t"
+        "ds_read_b64_tr_b16 %6, %16 offset:96\n\tds_read_b64_tr_b16 %7, %17 offset:96\n\t"
+        "ds_read_b64_tr_b16 %8, %16 offset:128\n\tds_read_b64_tr_b16 %9, %17 offset:128\n\t"
+        "ds_read_b64_tr_b16 %10, %16 offset:160\n\tds_read_b64_tr_b16 %11, %17 offset:160\n\t"
+        "ds_read_b64_tr_b16 %12, %16 offset:192\n\tds_read_b64_tr_b16 %13, %17 offset:192\n\t"
+        "ds_read_b64_tr_b16 %14, %16 offset:224\n\tds_read_b64_tr_b16 %15, %17 offset:224\n\t"
+        "s_waitcnt lgkmcnt(0)"
+        : "=&v"(f[0].x), "=&v"(f[0].y), "=&v"(f[1].x), "=&v"(f[1].y), "=&v"(f[2].x), "=&v"(f[2].y), "=&v"(f[3].x), "=&v"(f[3].y), "=&v"(f[4].x),
+          "=&v"(f[4].y), "=&v"(f[5].x), "=&v"(f[5].y), "=&v"(f[6].x), "=&v"(f[6].y), "=&v"(f[7].x), "=&v"(f[7].y)
+        : "v"(p), "v"(q)
+        : "memory");
+}
+__device__ __forceinline__ void tr_read2(TrCols (&f)[2], uint32_t p, uint32_t q) {
+    asm volatile(
+        "ds_read_b64_tr_b16 %0, %4\n\tds_read_b64_tr_b16 %1, %5\n\t"
+        "ds_read_b64_tr_b16 %2, %4 offset:32\n\tds_read_b64_tr_b16 %3, %5 offset:32\n\t"
+        "s_waitcnt lgkmcnt(0)"
+        : "=&v"(f[0].x), "=&v"(f[0].y), "=&v"(f[1].x), "=&v"(f[1].y)
+        : "v"(p), "v"(q)
+        : "memory");
 }
 
 // Workgroup (split, group of heads).  Four waves: RW of them share 16 heads and the latent columns of the output (each one
-// computes all scores of its heads), 4 / RW sets of 16 heads.  Tiles of cache rows go through a double buffer in LDS, with an
-// odd number of 16-byte units per row, and serve as keys (row fragments) and as values (transposed reads).
+// computes all scores of its heads), 4 / RW sets of 16 heads.  Tiles of cache rows go through buffers in LDS, two ahead, and
+// serve as keys (row fragments) and as values (transposed reads).  A row in LDS has room for NR latents and 128 rotated values
+// and an odd number of 16-byte units; past the end of the cache row its last unit is repeated, which meets zeros in the query
+// and columns that are not stored.
 struct SeqLatentAttn {
     const char* q;           // T [H][crow bytes]
     const char* kc;          // caches, slot 0
@@ -165,108 +192,148 @@ struct SeqLatentAttn {
     const int* state;
     float *acc, *ml;         // [ns][H][rp], [ns][H][2]
     float scale_log2;
-    int H, crow, ns, rp, tile_bytes;
+    int H, crow, ns, least, rp;      // least: tiles of a split
 };
+template <typename T, int NR> struct LatentLds {
+    static constexpr int ksteps = (NR + 128) * (int)sizeof(T) / 64, up = ksteps * 4 + 1;
+    static constexpr int copies = (LatentTile<T>::keys * up + 255) / 256;            // 1 KB copies per wave and tile
+    static constexpr int tile = copies * kSeqWaves * 1024, buffers = 3;
+};
+
+// 64 units of the tile per copy, the waves in turn
+template <typename T, int NR>
+__device__ __forceinline__ void latent_stage(char* __restrict__ tile, const char* __restrict__ kc, int crow, int kb, int last, int wave, int lane) {
+    using L = LatentLds<T, NR>;
+    const int units = crow / 16;
+#pragma unroll
+    for (int i = 0; i < L::copies; ++i) {
+        const int c = i * kSeqWaves + wave, l = c * 64 + lane, r = l / L::up, u = l - r * L::up;
+        copy_to_lds16(kc + (size_t)min(kb + r, last) * crow + min(u, units - 1) * 16, tile + c * 1024);
+    }
+}
+
+// One tile: the next one's copies, scores, softmax, second product.
+template <typename T, int NR, int RW>
+__device__ __forceinline__ void latent_tile(AttnState<NR / RW>& st, const u32x4 (&qf)[LatentLds<T, NR>::ksteps], const char* __restrict__ tile,
+                                            char* __restrict__ next, bool more, const char* __restrict__ kc, int crow, int kb, int kn, int k1,
+                                            float scale_log2, int rw, int wave, int lane) {
+    using L = LatentLds<T, NR>;
+    constexpr int KT = LatentTile<T>::keys, KF = KT / 16, NW = NR / RW, G = 4;       // G: steps of the first product read together
+    static_assert(L::ksteps % G == 0, "");
+    const int col = lane & 15, g = lane >> 4;
+    if (more) latent_stage<T, NR>(next, kc, crow, kn, k1 - 1, wave, lane);
+    f32x4 s[KF];
+#pragma unroll
+    for (int kt = 0; kt < KF; ++kt) s[kt] = f32x4{0.f, 0.f, 0.f, 0.f};
+    u32x4 kf[2][G][KF];
+    auto read = [&](int d0, u32x4 (&f)[G][KF]) __attribute__((always_inline)) {
+#pragma unroll
+        for (int d = 0; d < G; ++d)
+#pragma unroll
+            for (int kt = 0; kt < KF; ++kt) f[d][kt] = *reinterpret_cast<const u32x4*>(tile + ((kt * 16 + col) * L::up + (d0 + d) * 4 + g) * 16);
+    };
+    read(0, kf[0]);
+#pragma unroll
+    for (int d0 = 0; d0 < L::ksteps; d0 += G) {
+        if (d0 + G < L::ksteps) read(d0 + G, kf[(d0 / G + 1) & 1]);
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int d = 0; d < G; ++d)
+#pragma unroll
+            for (int kt = 0; kt < KF; ++kt) s[kt] = mma16<T>(kf[(d0 / G) & 1][d][kt], qf[d0 + d], s[kt]);
+        __builtin_amdgcn_sched_barrier(0);
+    }
+#pragma unroll
+    for (int kt = 0; kt < KF; ++kt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) s[kt][r] = kb + kt * 16 + g * 4 + r < k1 ? s[kt][r] * scale_log2 : kMasked;
+    attn_softmax<NW, KF>(st, s, NW / 16);
+    if constexpr (sizeof(T) == 2) {
+        u32x4 hi, lo;
+#pragma unroll
+        for (int kt = 0; kt < 2; ++kt) {
+            f32x4 rest;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) rest[r] = s[kt][r] - (float)(bf16_t)s[kt][r];
+            hi[2 * kt] = pack_bf16(s[kt][0], s[kt][1]);
+            hi[2 * kt + 1] = pack_bf16(s[kt][2], s[kt][3]);
+            lo[2 * kt] = pack_bf16(rest[0], rest[1]);
+            lo[2 * kt + 1] = pack_bf16(rest[2], rest[3]);
+        }
+        constexpr int B = NW >= 128 ? 8 : 2;             // sets of 16 columns read together
+        const uint32_t v = (uint32_t)(uintptr_t)(tile + (4 * g + (col >> 2)) * L::up * 16 + rw * NW * 2 + (col & 3) * 8);
+#pragma unroll
+        for (int i = 0; i < NW / 16; i += B) {
+            TrCols c[B];
+            if constexpr (B == 8) tr_read8(c, v + i * 32, v + i * 32 + 16 * L::up * 16);
+            else tr_read2(c, v + i * 32, v + i * 32 + 16 * L::up * 16);
+#pragma unroll
+            for (int j = 0; j < B; ++j) {
+                const u32x4 f = {c[j].x.x, c[j].x.y, c[j].y.x, c[j].y.y};
+                st.acc[i + j] = mma16<T>(f, hi, st.acc[i + j]);
+                st.acc[i + j] = mma16<T>(f, lo, st.acc[i + j]);
+            }
+        }
+    } else {
+        const char* v = tile + 4 * g * L::up * 16 + (rw * NW + col) * 4;
+#pragma unroll
+        for (int i = 0; i < NW / 16; ++i) {
+            f32x4 f;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) f[j] = *reinterpret_cast<const float*>(v + j * L::up * 16 + i * 64);
+            st.acc[i] = mma16<T>(__builtin_bit_cast(u32x4, f), __builtin_bit_cast(u32x4, s[0]), st.acc[i]);
+        }
+    }
+}
+
 template <typename T, int NR, int RW>
 __global__ __launch_bounds__(kSeqThreads, 1) void k_seq_latent_attn(SeqLatentAttn a) {
-    constexpr int KT = LatentTile<T>::keys, KF = KT / 16, NW = NR / RW, KS = (NR + 128) * (int)sizeof(T) / 64;
+    using L = LatentLds<T, NR>;
+    constexpr int KT = LatentTile<T>::keys, NW = NR / RW;
     extern __shared__ __align__(1024) char tiles[];
     const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, col = lane & 15, g = lane >> 4;
     const int rw = wave % RW, h0 = ((int)blockIdx.y * (kSeqWaves / RW) + wave / RW) * 16;
-    const int pos = a.state[1], ntiles = latent_tiles<T>(pos), nsplit = min(a.ns, ntiles), sp = blockIdx.x;
+    const int pos = a.state[1], ntiles = latent_tiles<T>(pos), nsplit = latent_splits(ntiles, a.ns, a.least), sp = blockIdx.x;
     if (sp >= nsplit) return;
     const int k0 = mul_div(ntiles, sp, nsplit) * KT, k1 = min(mul_div(ntiles, sp + 1, nsplit) * KT, pos + 1);
     const char* kc = a.kc + a.state[3] * a.slot_bytes;
-    const int units = a.crow / 16, up = units | 1, ksteps = a.crow / 64;
-
-    // copies: 64 units of the padded tile each, wave after wave
-    const int copies = (KT * up + 63) / 64, du = 256 % up, dr = 256 / up;
-    auto stage = [&](int buf, int kb) {
-        int r = (wave * 64 + lane) / up, u = wave * 64 + lane - r * up;
-        for (int i = wave; i < copies; i += kSeqWaves) {
-            copy_to_lds16(kc + (size_t)min(kb + r, k1 - 1) * a.crow + min(u, units - 1) * 16, tiles + buf * a.tile_bytes + i * 1024);
-            r += dr;
-            u += du;
-            if (u >= up) {
-                u -= up;
-                ++r;
-            }
-        }
-    };
-    stage(0, k0);
+    const int ksteps = a.crow / 64;
     const char* qr = a.q + (size_t)min(h0 + col, a.H - 1) * a.crow + g * 16;
-    u32x4 qf[KS];
+    u32x4 qf[L::ksteps];
 #pragma unroll
-    for (int s = 0; s < KS; ++s)
-        if (s < ksteps) qf[s] = ld16(qr + s * 64);
+    for (int s = 0; s < L::ksteps; ++s) {
+        qf[s] = ld16(qr + min(s, ksteps - 1) * 64);
+        if (s >= ksteps) qf[s] = u32x4{0, 0, 0, 0};
+    }
+    latent_stage<T, NR>(tiles, kc, a.crow, k0, k1 - 1, wave, lane);
+    if (k0 + KT < k1) latent_stage<T, NR>(tiles + L::tile, kc, a.crow, k0 + KT, k1 - 1, wave, lane);
     AttnState<NW> st;
     attn_reset(st);
-    const int r0 = rw * NW, rtiles = max(0, min(NW, a.rp - r0)) / 16;
     int buf = 0;
-    for (int kb = k0; kb < k1; kb += KT, buf ^= 1) {
-        __syncthreads();                                 // the tile is there; nobody reads the other buffer any more
-        if (kb + KT < k1) stage(buf ^ 1, kb + KT);
-        const char* tile = tiles + buf * a.tile_bytes;
-        f32x4 s[KF];
-#pragma unroll
-        for (int kt = 0; kt < KF; ++kt) s[kt] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int d = 0; d < KS; ++d)
-            if (d < ksteps) {
-#pragma unroll
-                for (int kt = 0; kt < KF; ++kt)
-                    s[kt] = mma16<T>(*reinterpret_cast<const u32x4*>(tile + ((kt * 16 + col) * up + d * 4 + g) * 16), qf[d], s[kt]);
-            }
-#pragma unroll
-        for (int kt = 0; kt < KF; ++kt)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) s[kt][r] = kb + kt * 16 + g * 4 + r < k1 ? s[kt][r] * a.scale_log2 : kMasked;
-        attn_softmax<NW, KF>(st, s, rtiles);
-        if constexpr (sizeof(T) == 2) {
-            u32x4 hi, lo;
-#pragma unroll
-            for (int kt = 0; kt < 2; ++kt) {
-                f32x4 rest;
-#pragma unroll
-                for (int r = 0; r < 4; ++r) rest[r] = s[kt][r] - (float)(bf16_t)s[kt][r];
-                hi[2 * kt] = pack_bf16(s[kt][0], s[kt][1]);
-                hi[2 * kt + 1] = pack_bf16(s[kt][2], s[kt][3]);
-                lo[2 * kt] = pack_bf16(rest[0], rest[1]);
-                lo[2 * kt + 1] = pack_bf16(rest[2], rest[3]);
-            }
-            const char* v = tile + (4 * g + (col >> 2)) * up * 16 + r0 * 2 + (col & 3) * 8;
-#pragma unroll
-            for (int i = 0; i < NW / 16; ++i)
-                if (i < rtiles) {
-                    const u32x2 x = tr_read(v + i * 32), y = tr_read(v + 16 * up * 16 + i * 32);
-                    const u32x4 f = {x.x, x.y, y.x, y.y};
-                    st.acc[i] = mma16<T>(f, hi, st.acc[i]);
-                    st.acc[i] = mma16<T>(f, lo, st.acc[i]);
-                }
-        } else {
-            const char* v = tile + 4 * g * up * 16 + (r0 + col) * 4;
-#pragma unroll
-            for (int i = 0; i < NW / 16; ++i)
-                if (i < rtiles) {
-                    f32x4 f;
-#pragma unroll
-                    for (int j = 0; j < 4; ++j) f[j] = *reinterpret_cast<const float*>(v + j * up * 16 + i * 64);
-                    st.acc[i] = mma16<T>(__builtin_bit_cast(u32x4, f), __builtin_bit_cast(u32x4, s[0]), st.acc[i]);
-                }
-        }
+    for (int kb = k0; kb < k1; kb += KT) {
+        // this wave's copies of the tile have arrived (the next tile's may be on their way), then everybody's; and nobody reads
+        // the buffer of the tile before any more
+        if (kb + KT < k1) wait_vm<L::copies>();
+        else wait_vm<0>();
+        lds_barrier();
+        const int ahead = buf == 0 ? 2 : buf - 1;        // (buf + 2) % 3
+        latent_tile<T, NR, RW>(st, qf, tiles + buf * L::tile, tiles + ahead * L::tile, kb + 2 * KT < k1, kc, a.crow, kb, kb + 2 * KT, k1, a.scale_log2, rw,
+                               wave, lane);
+        buf = buf == 2 ? 0 : buf + 1;
     }
     if (h0 + col >= a.H) return;
     const size_t row = (size_t)sp * a.H + h0 + col;
     if (rw == 0 && g == 0) *reinterpret_cast<float2*>(a.ml + row * 2) = make_float2(st.m, st.l);
 #pragma unroll
     for (int i = 0; i < NW / 16; ++i)
-        if (i < rtiles) *reinterpret_cast<f32x4*>(a.acc + row * a.rp + r0 + i * 16 + g * 4) = st.acc[i];
+        if (rw * NW + i * 16 < a.rp) *reinterpret_cast<f32x4*>(a.acc + row * a.rp + rw * NW + i * 16 + g * 4) = st.acc[i];
 }
 
-// Workgroup (kLatentOut outputs of a head): merges the splits of the head, then its rows of W_uv, four per wave, in fp32, and
+// Workgroup (head, kLatentOut of its outputs; the head runs fastest, which keeps the workgroups of one head, who read the same
+// partial results, on few XCDs): merges the splits of the head, then its rows of W_uv, four per wave, in fp32, and
 // the output gate.
 constexpr int kLatentOut = 16;
-constexpr int kLatentSplits = 64;
+constexpr int kLatentSplits = kSeqThreads;
 struct SeqLatentOut {
     const float *acc, *ml;
     const int* state;
@@ -274,15 +341,15 @@ struct SeqLatentOut {
     const float* gate;       // nullable: [H * V] before the sigmoid
     const char* w_uv;        // T [H * V][pitch bytes]
     char* out;               // T [H * V]
-    int H, V, pitch, ns, rp;
+    int H, V, pitch, ns, least, rp;
 };
 template <typename T>
 __global__ __launch_bounds__(kSeqThreads) void k_seq_latent_out(SeqLatentOut a) {
     constexpr int U = Unit<T>::n, RPW = kLatentOut / kSeqWaves, NC = sizeof(T) == 2 ? 1 : 2;     // rows per wave, 1 KB loads per row
-    __shared__ float f[kLatentSplits];
+    __shared__ float f[kLatentSplits], red[kSeqWaves];
     __shared__ __align__(16) float sum[kSeqThreads * 4];
     __shared__ __align__(16) float lat[NC * 64 * U];
-    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = blockIdx.y, v0 = blockIdx.x * kLatentOut;
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = blockIdx.x, v0 = blockIdx.y * kLatentOut;
     u32x4 b[RPW][NC];
 #pragma unroll
     for (int i = 0; i < RPW; ++i) {
@@ -290,25 +357,35 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_latent_out(SeqLatentOut a) 
 #pragma unroll
         for (int c = 0; c < NC; ++c) b[i][c] = ld16(a.w_uv + ((size_t)h * a.V + v) * a.pitch + min(c * 1024 + lane * 16, a.pitch - 16));
     }
-    const int nsplit = min(a.ns, latent_tiles<T>(a.state[1]));
+    const int nsplit = latent_splits(latent_tiles<T>(a.state[1]), a.ns, a.least);
+    // a thread sums four latent columns over every nsg-th split; the first kM of these are requested before their weights
+    // are known
+    constexpr int kM = 16;
     const int r4 = a.rp / 4, nsg = kSeqThreads / r4, sg = tid / r4, x = tid - sg * r4;
-    if (wave == 0) {                                     // (at most one split per lane)
-        const float2 t = lane < nsplit ? *reinterpret_cast<const float2*>(a.ml + ((size_t)lane * a.H + h) * 2) : make_float2(kNegBig, 0.0f);
+    const float* p = a.acc + (size_t)h * a.rp + x * 4;
+    const size_t split_stride = (size_t)a.H * a.rp;
+    f32x4 t[kM];
+    auto request = [&](int s0) {
+#pragma unroll
+        for (int j = 0; j < kM; ++j) t[j] = *reinterpret_cast<const f32x4*>(p + min(s0 + j * nsg, nsplit - 1) * split_stride);
+    };
+    request(sg);
+    {                                                    // (at most one split per thread)
+        const float2 ml = tid < nsplit ? *reinterpret_cast<const float2*>(a.ml + ((size_t)tid * a.H + h) * 2) : make_float2(kNegBig, 0.0f);
         const float snk = a.sink != nullptr ? a.sink[h] * kLog2e : kNegBig;
-        const float m = fmaxf(wave_max(t.x), snk), e = fast_exp2(t.x - m);
-        const float l = wave_sum(t.y * e) + (a.sink != nullptr ? fast_exp2(snk - m) : 0.0f);
-        f[lane] = e / l;
+        const float wm = wave_max(ml.x);
+        if (lane == 0) red[wave] = wm;
+        __syncthreads();
+        const float m = fmaxf(fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])), snk), e = fast_exp2(ml.x - m);
+        const float l = block_sum(ml.y * e, red) + (a.sink != nullptr ? fast_exp2(snk - m) : 0.0f);
+        f[tid] = e / l;
     }
     for (int i = tid; i < NC * 64 * U; i += kSeqThreads) lat[i] = 0.0f;
     __syncthreads();
     if (sg < nsg) {
         f32x4 s = {0.f, 0.f, 0.f, 0.f};
-        const float* p = a.acc + (size_t)h * a.rp + x * 4;
-        constexpr int kM = 8;
         for (int s0 = sg; s0 < nsplit; s0 += nsg * kM) {
-            f32x4 t[kM];
-#pragma unroll
-            for (int j = 0; j < kM; ++j) t[j] = *reinterpret_cast<const f32x4*>(p + (size_t)min(s0 + j * nsg, nsplit - 1) * a.H * a.rp);
+            if (s0 != sg) request(s0);
 #pragma unroll
             for (int j = 0; j < kM; ++j)
                 if (s0 + j * nsg < nsplit) {

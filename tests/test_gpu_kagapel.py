@@ -124,6 +124,22 @@ def test_far_key_with_many_splits(heads, rank, length, at, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES, ids=IDS)
+@pytest.mark.parametrize("heads,rank", [(3, 500), (40, 60)])
+def test_very_long_caches_decoded_like_a_prompt(heads, rank, dtype):
+    """More splits than a workgroup that merges them takes at a time, against the same positions of a whole prompt."""
+    length, n = 9000, 4
+    for at in (8990, 77):
+        cfg, w, toks = M.far_key_model(heads, rank, length, at)
+        m = build(cfg, w, dtype, capacity=length, max_portion=length)
+        want = m.forward(0, toks, 0, range(length - n, length)).cpu()
+        other = m.forward(0, [1 if t == 0 else t for t in toks], 0, [length - 1]).cpu()
+        assert M.error(other, want[-1:]) > 0.2       # the key is seen
+        m.forward(0, toks[:length - n], 0)
+        got = torch.cat([m.forward(0, [t], length - n + i, [0]) for i, t in enumerate(toks[length - n:])])
+        assert M.error(got, want) < LIMIT[dtype]
+
+
+@pytest.mark.parametrize("dtype", DTYPES, ids=IDS)
 @pytest.mark.parametrize("level", [-20.0, 0.0, 12.0])
 def test_sinks_of_any_size(level, dtype):
     cfg, w, toks, _, _ = reference("sinks")
