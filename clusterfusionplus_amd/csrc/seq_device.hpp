@@ -90,12 +90,9 @@ __device__ __forceinline__ void copy_to_lds16(const void* g, void* lds) {
 // waits until at most N of the wave's vector memory operations are still on their way
 template <int N> __device__ __forceinline__ void wait_vm() { asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory"); }
 
-// A barrier of the workgroup behind its LDS accesses only: __syncthreads() would also wait for loads in flight.
-__device__ __forceinline__ void lds_barrier() {
-    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
-    __builtin_amdgcn_s_barrier();
-    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
-}
+// A barrier of the workgroup behind its LDS accesses only.  Written out: __syncthreads(), and a fence over LDS as well, would
+// also wait for the loads in flight, those that go straight to LDS among them.
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 
 __device__ __forceinline__ float wave_max(float v) {
 #pragma unroll
@@ -294,25 +291,27 @@ __device__ __forceinline__ void attn_softmax(AttnState<NT>& st, f32x4 (&s)[NKT],
         if (i < vtiles) st.acc[i] *= c;
 }
 
-// acc += V^T p for the keys of one tile
-template <typename T, int NT, int KT>
-__device__ __forceinline__ void attn_pv(AttnState<NT>& st, const f32x4 (&p)[KT / 16], const char* vt, int vtiles, int lane) {
+// acc += V^T p for the keys of one tile and CT column tiles, which share the reads of V^T
+template <typename T, int NT, int KT, int CT>
+__device__ __forceinline__ void attn_pv(AttnState<NT>* st, const f32x4 (*p)[KT / 16], const char* vt, int vtiles, int lane) {
     const int col = lane & 15, g = lane >> 4;
     if constexpr (sizeof(T) == 2) {
-        u32x4 hi[KT / 32], lo[KT / 32];
+        u32x4 hi[CT][KT / 32], lo[CT][KT / 32];
 #pragma unroll
-        for (int s = 0; s < KT / 32; ++s)
+        for (int ct = 0; ct < CT; ++ct)
 #pragma unroll
-            for (int h = 0; h < 2; ++h) {
-                const f32x4 v = p[2 * s + h];
-                f32x4 rest;
+            for (int s = 0; s < KT / 32; ++s)
 #pragma unroll
-                for (int r = 0; r < 4; ++r) rest[r] = v[r] - (float)(bf16_t)v[r];
-                hi[s][2 * h] = pack_bf16(v[0], v[1]);
-                hi[s][2 * h + 1] = pack_bf16(v[2], v[3]);
-                lo[s][2 * h] = pack_bf16(rest[0], rest[1]);
-                lo[s][2 * h + 1] = pack_bf16(rest[2], rest[3]);
-            }
+                for (int h = 0; h < 2; ++h) {
+                    const f32x4 v = p[ct][2 * s + h];
+                    f32x4 rest;
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) rest[r] = v[r] - (float)(bf16_t)v[r];
+                    hi[ct][s][2 * h] = pack_bf16(v[0], v[1]);
+                    hi[ct][s][2 * h + 1] = pack_bf16(v[2], v[3]);
+                    lo[ct][s][2 * h] = pack_bf16(rest[0], rest[1]);
+                    lo[ct][s][2 * h + 1] = pack_bf16(rest[2], rest[3]);
+                }
 #pragma unroll
         for (int i = 0; i < NT / 16; ++i)
             if (i < vtiles) {
@@ -321,8 +320,11 @@ __device__ __forceinline__ void attn_pv(AttnState<NT>& st, const f32x4 (&p)[KT /
                 for (int s = 0; s < KT / 32; ++s) {
                     const u32x2 a = *reinterpret_cast<const u32x2*>(row + s * 64), b = *reinterpret_cast<const u32x2*>(row + s * 64 + 32);
                     const u32x4 f = {a.x, a.y, b.x, b.y};
-                    st.acc[i] = mma16<T>(f, hi[s], st.acc[i]);
-                    st.acc[i] = mma16<T>(f, lo[s], st.acc[i]);
+#pragma unroll
+                    for (int ct = 0; ct < CT; ++ct) {
+                        st[ct].acc[i] = mma16<T>(f, hi[ct][s], st[ct].acc[i]);
+                        st[ct].acc[i] = mma16<T>(f, lo[ct][s], st[ct].acc[i]);
+                    }
                 }
             }
     } else {
@@ -331,8 +333,11 @@ __device__ __forceinline__ void attn_pv(AttnState<NT>& st, const f32x4 (&p)[KT /
             if (i < vtiles) {
                 const char* row = vt + (i * 16 + col) * VtTile<T, KT>::pitch + g * 16;
 #pragma unroll
-                for (int s = 0; s < KT / 16; ++s)
-                    st.acc[i] = mma16<T>(*reinterpret_cast<const u32x4*>(row + s * 64), __builtin_bit_cast(u32x4, p[s]), st.acc[i]);
+                for (int s = 0; s < KT / 16; ++s) {
+                    const u32x4 f = *reinterpret_cast<const u32x4*>(row + s * 64);
+#pragma unroll
+                    for (int ct = 0; ct < CT; ++ct) st[ct].acc[i] = mma16<T>(f, __builtin_bit_cast(u32x4, p[ct][s]), st[ct].acc[i]);
+                }
             }
     }
 }

@@ -478,7 +478,8 @@ struct SeqAttn {
 template <int UN> __device__ __forceinline__ int swz_key(int row) { return UN % 16 ? (row >> 1) & 7 : row & 15; }
 
 // (the next tile's keys go straight to the other LDS buffer and its values into registers while this one is worked on)
-// (NK: elements of a key row in LDS, NT: value columns)
+// (NK: elements of a key row in LDS, NT: value columns.  The products run over all of them, without branches between the reads
+// of LDS: past the end of the query there are zeros, and of the columns past the end of a value nothing is stored)
 template <typename T, int NK, int NT, int CT>
 __global__ __launch_bounds__(kSeqThreads, (NT <= 128 ? 2 : 1)) void k_seq_attn(SeqAttn a) {
     constexpr int KT = sizeof(T) == 2 ? 64 : 32;
@@ -487,7 +488,12 @@ __global__ __launch_bounds__(kSeqThreads, (NT <= 128 ? 2 : 1)) void k_seq_attn(S
     __shared__ __align__(1024) char ks[2][KT * NB];
     __shared__ __align__(16) char vt[NT * VtTile<T, KT>::pitch];
     const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, col = lane & 15, g = lane >> 4;
-    const int gq = blockIdx.y, ncols = a.T * a.R, c0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * 64 * CT;
+    // the longest walks first; every second group of eight runs backwards, so that each XCD (workgroups go round them) gets as
+    // many long ones as the others
+    const int gq = blockIdx.y, ncols = a.T * a.R, gx = gridDim.x;
+    int bx = blockIdx.x;
+    if (((bx >> 3) & 1) && (bx | 7) < gx) bx ^= 7;
+    const int c0 = (gx - 1 - bx) * 64 * CT;
 
     int pq[CT], first[CT], tok[CT], head[CT];
     u32x4 qf[CT][NB / 64];
@@ -501,8 +507,10 @@ __global__ __launch_bounds__(kSeqThreads, (NT <= 128 ? 2 : 1)) void k_seq_attn(S
         first[ct] = chunk_start(pq[ct], a.chunk);
         const char* qr = a.q + ((size_t)tok[ct] * a.H + head[ct]) * a.qrow + g * 16;
 #pragma unroll
-        for (int s = 0; s < NB / 64; ++s)
-            if (s < a.dsteps) qf[ct][s] = ld16(qr + s * 64);
+        for (int s = 0; s < NB / 64; ++s) {
+            qf[ct][s] = ld16(qr + min(s, a.dsteps - 1) * 64);
+            if (s >= a.dsteps) qf[ct][s] = u32x4{0, 0, 0, 0};
+        }
         attn_reset(st[ct]);
     }
     // keys the workgroup needs, and those every column of this wave sees / any column sees
@@ -543,20 +551,28 @@ __global__ __launch_bounds__(kSeqThreads, (NT <= 128 ? 2 : 1)) void k_seq_attn(S
         }
         lds_barrier();                                   // (waits for the stores to LDS, not for the next tile)
         if (t.k0 <= any_hi && next > any_lo) {
+            // the fragments of the next 16 keys are read while these are multiplied
             f32x4 s[CT][KT / 16];
-#pragma unroll
-            for (int kt = 0; kt < KT / 16; ++kt) {
-#pragma unroll
-                for (int ct = 0; ct < CT; ++ct) s[ct][kt] = f32x4{0.f, 0.f, 0.f, 0.f};
+            u32x4 kf[2][NB / 64];
+            auto read = [&](int kt) __attribute__((always_inline)) {
                 const int r = kt * 16 + col;
 #pragma unroll
                 for (int d = 0; d < NB / 64; ++d)
-                    if (d < a.dsteps) {
-                        const u32x4 kf = *reinterpret_cast<const u32x4*>(ks[buf] + r * NB + ((d * 4 + g) ^ swz_key<UN>(r)) * 16);
+                    kf[kt & 1][d] = *reinterpret_cast<const u32x4*>(ks[buf] + r * NB + ((d * 4 + g) ^ swz_key<UN>(r)) * 16);
+            };
+            read(0);
 #pragma unroll
-                        for (int ct = 0; ct < CT; ++ct) s[ct][kt] = mma16<T>(kf, qf[ct][d], s[ct][kt]);
-                    }
+            for (int kt = 0; kt < KT / 16; ++kt) {
+                if (kt + 1 < KT / 16) read(kt + 1);
+                __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+                for (int ct = 0; ct < CT; ++ct) {
+                    s[ct][kt] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                    for (int d = 0; d < NB / 64; ++d) s[ct][kt] = mma16<T>(kf[kt & 1][d], qf[ct][d], s[ct][kt]);
+                }
             }
+            __builtin_amdgcn_sched_barrier(0);
             const bool full = t.k0 + KT <= t.hi && t.k0 >= all_lo && t.k0 + KT - 1 <= all_hi;
 #pragma unroll
             for (int ct = 0; ct < CT; ++ct) {
@@ -573,9 +589,10 @@ __global__ __launch_bounds__(kSeqThreads, (NT <= 128 ? 2 : 1)) void k_seq_attn(S
                             if (key >= t.hi || key > pq[ct] || key < first[ct]) s[ct][kt][r] = kMasked;
                         }
                 }
-                attn_softmax<NT, KT / 16>(st[ct], s[ct], a.vtiles);
-                attn_pv<T, NT, KT>(st[ct], s[ct], vt, a.vtiles, lane);
+                attn_softmax<NT, KT / 16>(st[ct], s[ct], NT / 16);
             }
+            __builtin_amdgcn_sched_barrier(0);           // (values read ahead of the softmax would take its registers)
+            attn_pv<T, NT, KT, CT>(st, s, vt, NT / 16, lane);
         }
         if (next >= k_end) break;
         t = tn;
@@ -726,7 +743,7 @@ __global__ __launch_bounds__(kSeqThreads) void k_seq_attn_decode(SeqAttnDec a) {
         attn_softmax<NT, KF>(st, s, a.vtiles);
         __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
         __builtin_amdgcn_wave_barrier();                 // the tile in LDS belongs to this wave alone
-        attn_pv<T, NT, KT>(st, s, vt, a.vtiles, lane);
+        attn_pv<T, NT, KT, 1>(&st, &s, vt, a.vtiles, lane);
         __builtin_amdgcn_wave_barrier();
     }
     // waves of the workgroup
@@ -1322,10 +1339,13 @@ void expert_gemm(const cfpp_seq* s, const LayerPlan& L, SeqGemm g, int n, hipStr
 template <typename T, int NK, int NT>
 void launch_attn(const SeqAttn& a, int G, int cus, hipStream_t st) {
     const int cols = a.T * a.R;
-    if (ceil_div(cols, 128) * G >= 2 * cus)
-        hipLaunchKernelGGL((k_seq_attn<T, NK, NT, 2>), dim3(ceil_div(cols, 128), G), dim3(kSeqThreads), 0, st, a);
-    else
-        hipLaunchKernelGGL((k_seq_attn<T, NK, NT, 1>), dim3(ceil_div(cols, 64), G), dim3(kSeqThreads), 0, st, a);
+    if constexpr (sizeof(T) == 2) {                      // (fp32: two column tiles do not fit the registers)
+        if (ceil_div(cols, 128) * G >= 2 * cus) {
+            hipLaunchKernelGGL((k_seq_attn<T, NK, NT, 2>), dim3(ceil_div(cols, 128), G), dim3(kSeqThreads), 0, st, a);
+            return;
+        }
+    }
+    hipLaunchKernelGGL((k_seq_attn<T, NK, NT, 1>), dim3(ceil_div(cols, 64), G), dim3(kSeqThreads), 0, st, a);
 }
 
 template <typename T>

@@ -180,8 +180,9 @@ __device__ __forceinline__ void tr_read2(TrCols (&f)[2], uint32_t p, uint32_t q)
         : "memory");
 }
 
-// Workgroup (split, group of heads).  Four waves: RW of them share 16 heads and the latent columns of the output (each one
-// computes all scores of its heads), 4 / RW sets of 16 heads.  Tiles of cache rows go through buffers in LDS, two ahead, and
+// Workgroup (split, group of heads).  Four waves: RW of them share 16 heads, each with its part of the scores' dimensions (the
+// parts are added through LDS, in the same order by all of them) and of the output's latent columns; 4 / RW sets of 16 heads.
+// Tiles of cache rows go through buffers in LDS, two ahead, and
 // serve as keys (row fragments) and as values (transposed reads).  A row in LDS has room for NR latents and 128 rotated values
 // and an odd number of 16-byte units; past the end of the cache row its last unit is repeated, which meets zeros in the query
 // and columns that are not stored.
@@ -212,36 +213,40 @@ __device__ __forceinline__ void latent_stage(char* __restrict__ tile, const char
     }
 }
 
-// One tile: the next one's copies, scores, softmax, second product.
+// One tile: the copies of a later one, scores, softmax, second product.  `parts`: [wave][KF][lane].
 template <typename T, int NR, int RW>
-__device__ __forceinline__ void latent_tile(AttnState<NR / RW>& st, const u32x4 (&qf)[LatentLds<T, NR>::ksteps], const char* __restrict__ tile,
-                                            char* __restrict__ next, bool more, const char* __restrict__ kc, int crow, int kb, int kn, int k1,
-                                            float scale_log2, int rw, int wave, int lane) {
+__device__ __forceinline__ void latent_tile(AttnState<NR / RW>& st, const u32x4 (&qf)[LatentLds<T, NR>::ksteps / RW], const char* __restrict__ tile,
+                                            char* __restrict__ next, bool more, f32x4* __restrict__ parts, const char* __restrict__ kc, int crow, int kb, int kn,
+                                            int k1, float scale_log2, int rw, int wave, int lane) {
     using L = LatentLds<T, NR>;
-    constexpr int KT = LatentTile<T>::keys, KF = KT / 16, NW = NR / RW, G = 4;       // G: steps of the first product read together
-    static_assert(L::ksteps % G == 0, "");
+    constexpr int KT = LatentTile<T>::keys, KF = KT / 16, NW = NR / RW, KS = L::ksteps / RW;
+    static_assert(L::ksteps % RW == 0, "");
     const int col = lane & 15, g = lane >> 4;
     if (more) latent_stage<T, NR>(next, kc, crow, kn, k1 - 1, wave, lane);
     f32x4 s[KF];
+    u32x4 kf[KS][KF];
 #pragma unroll
-    for (int kt = 0; kt < KF; ++kt) s[kt] = f32x4{0.f, 0.f, 0.f, 0.f};
-    u32x4 kf[2][G][KF];
-    auto read = [&](int d0, u32x4 (&f)[G][KF]) __attribute__((always_inline)) {
+    for (int d = 0; d < KS; ++d)
 #pragma unroll
-        for (int d = 0; d < G; ++d)
+        for (int kt = 0; kt < KF; ++kt) kf[d][kt] = *reinterpret_cast<const u32x4*>(tile + ((kt * 16 + col) * L::up + (rw * KS + d) * 4 + g) * 16);
+    __builtin_amdgcn_sched_barrier(0);                   // (all reads are requested before the first product waits for one)
 #pragma unroll
-            for (int kt = 0; kt < KF; ++kt) f[d][kt] = *reinterpret_cast<const u32x4*>(tile + ((kt * 16 + col) * L::up + (d0 + d) * 4 + g) * 16);
-    };
-    read(0, kf[0]);
+    for (int kt = 0; kt < KF; ++kt) {
+        s[kt] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int d0 = 0; d0 < L::ksteps; d0 += G) {
-        if (d0 + G < L::ksteps) read(d0 + G, kf[(d0 / G + 1) & 1]);
-        __builtin_amdgcn_sched_barrier(0);
+        for (int d = 0; d < KS; ++d) s[kt] = mma16<T>(kf[d][kt], qf[d], s[kt]);
+    }
 #pragma unroll
-        for (int d = 0; d < G; ++d)
+    for (int kt = 0; kt < KF; ++kt) parts[(wave * KF + kt) * kWave + lane] = s[kt];
+    lds_barrier();
 #pragma unroll
-            for (int kt = 0; kt < KF; ++kt) s[kt] = mma16<T>(kf[(d0 / G) & 1][d][kt], qf[d0 + d], s[kt]);
-        __builtin_amdgcn_sched_barrier(0);
+    for (int kt = 0; kt < KF; ++kt) {
+        f32x4 p[RW];
+#pragma unroll
+        for (int w = 0; w < RW; ++w) p[w] = parts[((wave - rw + w) * KF + kt) * kWave + lane];
+        s[kt] = p[0];
+#pragma unroll
+        for (int w = 1; w < RW; ++w) s[kt] += p[w];
     }
 #pragma unroll
     for (int kt = 0; kt < KF; ++kt)
@@ -289,8 +294,9 @@ __device__ __forceinline__ void latent_tile(AttnState<NR / RW>& st, const u32x4 
 template <typename T, int NR, int RW>
 __global__ __launch_bounds__(kSeqThreads, 1) void k_seq_latent_attn(SeqLatentAttn a) {
     using L = LatentLds<T, NR>;
-    constexpr int KT = LatentTile<T>::keys, NW = NR / RW;
+    constexpr int KT = LatentTile<T>::keys, NW = NR / RW, KS = L::ksteps / RW;
     extern __shared__ __align__(1024) char tiles[];
+    __shared__ f32x4 parts[kSeqWaves * (KT / 16) * kWave];
     const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, col = lane & 15, g = lane >> 4;
     const int rw = wave % RW, h0 = ((int)blockIdx.y * (kSeqWaves / RW) + wave / RW) * 16;
     const int pos = a.state[1], ntiles = latent_tiles<T>(pos), nsplit = latent_splits(ntiles, a.ns, a.least), sp = blockIdx.x;
@@ -299,11 +305,11 @@ __global__ __launch_bounds__(kSeqThreads, 1) void k_seq_latent_attn(SeqLatentAtt
     const char* kc = a.kc + a.state[3] * a.slot_bytes;
     const int ksteps = a.crow / 64;
     const char* qr = a.q + (size_t)min(h0 + col, a.H - 1) * a.crow + g * 16;
-    u32x4 qf[L::ksteps];
+    u32x4 qf[KS];
 #pragma unroll
-    for (int s = 0; s < L::ksteps; ++s) {
-        qf[s] = ld16(qr + min(s, ksteps - 1) * 64);
-        if (s >= ksteps) qf[s] = u32x4{0, 0, 0, 0};
+    for (int s = 0; s < KS; ++s) {
+        qf[s] = ld16(qr + min(rw * KS + s, ksteps - 1) * 64);
+        if (rw * KS + s >= ksteps) qf[s] = u32x4{0, 0, 0, 0};
     }
     latent_stage<T, NR>(tiles, kc, a.crow, k0, k1 - 1, wave, lane);
     if (k0 + KT < k1) latent_stage<T, NR>(tiles + L::tile, kc, a.crow, k0 + KT, k1 - 1, wave, lane);
@@ -317,7 +323,7 @@ __global__ __launch_bounds__(kSeqThreads, 1) void k_seq_latent_attn(SeqLatentAtt
         else wait_vm<0>();
         lds_barrier();
         const int ahead = buf == 0 ? 2 : buf - 1;        // (buf + 2) % 3
-        latent_tile<T, NR, RW>(st, qf, tiles + buf * L::tile, tiles + ahead * L::tile, kb + 2 * KT < k1, kc, a.crow, kb, kb + 2 * KT, k1, a.scale_log2, rw,
+        latent_tile<T, NR, RW>(st, qf, tiles + buf * L::tile, tiles + ahead * L::tile, kb + 2 * KT < k1, parts, kc, a.crow, kb, kb + 2 * KT, k1, a.scale_log2, rw,
                                wave, lane);
         buf = buf == 2 ? 0 : buf + 1;
     }
