@@ -110,7 +110,7 @@ def resource_report(out=None):
         if nice.startswith("_Z") or "_Accum" in nice:
             # c++filt does not know the manglings of _Float16 and __bf16 (DF16_, DF16b; it may take the latter for something
             # else): take the kernel's name and its type, integer and bool template arguments out of the mangled name by hand
-            m = re.match(r"_ZN12_GLOBAL__N_1(\d+)", name)
+            m = re.match(r"_ZN(?:12_GLOBAL__N_1|4cfpp)(\d+)", name)
             if m:
                 n = int(m.group(1))
                 base = name[m.end():m.end() + n]
@@ -120,7 +120,7 @@ def resource_report(out=None):
                     vals += [v if k == "i" else ("true" if v == "1" else "false") for k, v in re.findall(r"L([ib])(\d+)E", targs.group(2))]
                     base += "<" + ", ".join(vals) + ">"
                 nice = base
-        nice = nice.replace("(anonymous namespace)::", "").replace("void ", "")
+        nice = nice.replace("(anonymous namespace)::", "").replace("cfpp::", "").replace("void ", "")
         nice = re.sub(r"\(.*\)$", "", nice)
 
         def g(key):

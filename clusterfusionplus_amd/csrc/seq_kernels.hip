@@ -11,10 +11,11 @@
 //   k_seq_gemv (output rows)
 //   k_seq_gemv (residual sum + norm | up rows of the chosen and the shared experts | activation)
 //   k_seq_gemv (down rows of all of them, weighted and summed)
-// Latent mixers: k_seq_latent_finish, a product that makes keys and values of all heads, k_seq_attn in portions; k_seq_latent_q,
-// k_seq_latent_attn, k_seq_latent_out in decode (seq_latent.hpp).  Residual streams: k_seq_streams after every product that
-// ends a sublayer of a portion; in decode the output rows' own launch updates them.
 // then k_seq_gemv over the vocabulary (both last norms | head rows | soft cap | best logit per workgroup) and k_seq_pick.
+// Latent mixers (seq_latent.hpp): in portions k_seq_latent_finish and a product that makes the keys and values of all heads come
+// before k_seq_attn, and nothing is appended after it; in decode k_seq_latent_q, k_seq_latent_attn and k_seq_latent_out take the
+// place of k_seq_attn_decode.  Residual streams: k_seq_streams instead of k_seq_postnorm; in decode the launches of the output
+// and down rows update the streams themselves.
 #include <hip/hip_runtime.h>
 #include <math.h>
 #include <stdint.h>
